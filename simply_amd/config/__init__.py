@@ -15,6 +15,7 @@ from .zenuzen import ZenuzenConfig
 from .nemidra import NemidraConfig
 from .tabupel import TabupelConfig
 from .rudutar import RudutarConfig
+from .kolorax import KoloraxConfig
 
 
 def architecture_name(d: Mapping[str, Any]) -> str:
@@ -51,4 +52,5 @@ def load_config(model_dir: str):
 
 
 __all__ = ["EngineConfig", "parse_dtype", "LayerSpec", "ModelSpec", "PartSpec", "ScheduleEntry",
-           "ConfigError", "Gemma2Config", "ZenuzenConfig", "NemidraConfig", "TabupelConfig", "RudutarConfig", "architecture_name", "config_from_dict", "load_config"]
+           "ConfigError", "Gemma2Config", "ZenuzenConfig", "NemidraConfig", "TabupelConfig", "RudutarConfig", "KoloraxConfig",
+           "architecture_name", "config_from_dict", "load_config"]

@@ -48,6 +48,9 @@ class ScheduleEntry:
     #: the embedding's output of this step is added to the residual stream before this entry runs (a pass of a loop
     #: over layers that is given the input again)
     add_embedding: bool = False
+    #: the number of the pass of a loop over layers that begins with this entry: the model's `pass_input` part is run on
+    #: the stream before it (None: no pass begins here)
+    begins_pass: int | None = None
 
 
 @dataclasses.dataclass(frozen=True)
@@ -69,6 +72,8 @@ class ModelSpec:
     #: tensor names that a model folder may hold and that the model does not read (norms around a feed-forward that
     #: a layer does not have)
     ignorable: tuple[str, ...] = ()
+    #: what is done to the stream before every pass of a loop (registry PASS_INPUTS), for entries with `begins_pass`
+    pass_input: "PartSpec | None" = None
 
     def validate(self) -> None:
         n = len(self.layers)
@@ -82,6 +87,8 @@ class ModelSpec:
                 if self.schedule[e.cache_from].cache_from is not None:
                     raise ValueError(
                         f"schedule entry {i} reads the cache of entry {e.cache_from}, which itself has none")
+        if self.pass_input is None and any(e.begins_pass is not None for e in self.schedule):
+            raise ValueError("a schedule entry begins a pass, but the model has no pass input")
         for name, of in self.copies.items():
             if name == of:
                 raise ValueError(f"tensor {name!r} is declared a copy of itself")

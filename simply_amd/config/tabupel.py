@@ -160,7 +160,7 @@ class TabupelConfig:
                 "key_dim": _positive(_get(m, "dim", where, int), "dim"), "rot_dim": rot_dim,
                 "value_dim": _positive(_get(m, "vdim", where, int), "vdim"), "q_rank": _positive(int(q_rank), "q_rank"),
                 "kv_rank": _positive(_get(m, "kv_rank", where, int), "kv_rank"), "scale": _get(m, "scale", where, float),
-                "norm_eps": eps, "window": _window(m, where), "output_gate": True,
+                "norm_eps": eps, "window": _window(m, where), "output_gate": "head",
                 "position_encoding": _rotation(m, where, rot_dim, default_dims=rot_dim),
             }, {"dq_proj": p + "dq", "dq_norm": p + "dq.norm", "uq_proj": p + "uq", "dkv_proj": p + "dkv",
                 "dkv_norm": p + "dkv.norm", "uk_proj": p + "uk", "uv_proj": p + "uv", "gate_proj": p + "g",

@@ -9,6 +9,10 @@
 namespace sa {
 
 enum Activation : int { kActGeluTanh = 0, kActSilu = 1, kActSquaredRelu = 2, kActGeluErf = 3, kNumActivations = 4 };
+// Rules that join the two factors of a gated product otherwise than act(g) * u; they exist for gated products only.
+//   kActClampedGlu: g' = min(g, limit), u' = clamp(u, -limit, limit), g' sigmoid(1.702 g') (u' + 1)
+enum GatedRule : int { kActClampedGlu = 4, kNumGatedRules = 5 };
+constexpr float kClampedGluSlope = 1.702f;
 
 // kEpilogueActivated: C = act(A.W^T), the product rounded to the output type first (a feed-forward without a gate)
 constexpr int kEpilogueNone = 0, kEpilogueGated = 1, kEpilogueSoftCap = 2, kEpilogueActivated = 3;
@@ -39,6 +43,17 @@ __device__ inline float gated_activation(int act, float x) {
   }
 }
 
+// The two factors of a gated product joined by the rule `act`; limit: what kActClampedGlu clamps to (in the entry
+// points of products it travels as `cap`, which a gated product has no other use for).
+__device__ inline float gated_product(int act, float limit, float g, float u) {
+  if (act == kActClampedGlu) {
+    g = fminf(g, limit);
+    u = fminf(fmaxf(u, -limit), limit);
+    return g * __builtin_amdgcn_rcpf(1.f + __expf(-kClampedGluSlope * g)) * (u + 1.f);
+  }
+  return gated_activation(act, g) * u;
+}
+
 // For the 32-bit path: the library's tanhf and expf, no approximations.
 __device__ inline float gated_activation_exact(int act, float x) {
   switch (act) {
@@ -47,6 +62,14 @@ __device__ inline float gated_activation_exact(int act, float x) {
     case kActGeluErf: return gelu_erf(x);
     default: return 0.5f * x * (1.f + tanhf(0.7978845608028654f * (x + 0.044715f * x * x * x)));
   }
+}
+__device__ inline float gated_product_exact(int act, float limit, float g, float u) {
+  if (act == kActClampedGlu) {
+    g = fminf(g, limit);
+    u = fminf(fmaxf(u, -limit), limit);
+    return g / (1.f + expf(-kClampedGluSlope * g)) * (u + 1.f);
+  }
+  return gated_activation_exact(act, g) * u;
 }
 
 }  // namespace sa

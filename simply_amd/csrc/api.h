@@ -258,7 +258,7 @@ int paged_attention_prefill(const void* q, int64_t q_stride, const void* k_pages
 bool gemm_wide_takes(int M, int N, int K, int64_t lda, int64_t ldc, const void* A, const void* W, const void* W2,
                      const void* C, int c_dtype, int epi, int packed);
 int gemm_wide(const void* A, int64_t lda, const void* W, void* C, int64_t ldc, int M, int N, int K, int epi, int act,
-              int shape, int ks, void* workspace, size_t workspace_bytes, hipStream_t stream, int* planes_left = nullptr);
+              float limit, int shape, int ks, void* workspace, size_t workspace_bytes, hipStream_t stream, int* planes_left = nullptr);
 // C = epilogue(sum over z of partials[z][M][NW]): the second kernel of every product that cuts K over workgroups
 int gemm_sum_partials(const float* partials, int ks, void* C, int c_dtype, int64_t ldc, int M, int N, int NW, int epi,
                       int act, float cap, hipStream_t stream);
@@ -318,11 +318,11 @@ int sa_residual_add_norm(const void* y, int y_dtype, int64_t y_stride, const voi
                          hipStream_t stream);
 
 // out[t, h, :] = (w null ? x[t, h, :] : x[t, h, :] / sqrt(mean(x[t, h, :]^2) + eps) * w) * gate(g[t, h, :]) for H
-// heads of `size` elements; w [size] is shared by the heads; gate 0: sigmoid, 1: silu.  out may be x.  gate_per_head: a
+// heads of `size` elements; w [size] is shared by the heads, or (w_per_head) [H * size]; gate 0: sigmoid, 1: silu.  out may be x.  gate_per_head: a
 // gate row holds H numbers, one for all entries of a head.
 int sa_gated_heads(const void* x, int x_dtype, int64_t x_stride, const void* g, int g_dtype, int64_t g_stride,
                    const void* w, int w_dtype, float eps, int gate, void* out, int out_dtype, int64_t out_stride, int T,
-                   int H, int size, int gate_per_head, hipStream_t stream);
+                   int H, int size, int gate_per_head, int w_per_head, hipStream_t stream);
 
 // x[t, n] = act(x[t, n]) in place (activation codes of activations.h).
 int sa_activation(void* x, int dtype, int64_t stride, int T, int N, int act, hipStream_t stream);
@@ -338,9 +338,11 @@ int sa_qk_norm_rope_cache_write(void* proj, int dtype, int64_t row_stride, const
                                 void* v_pages, int T, int H, int K, int dk, int dv, int page_size, hipStream_t stream);
 
 // residual += mult * y (y null: nothing is added), then out = residual / sqrt(mean(residual^2) + eps) * (w + plus_one):
-// the sum of a block whose parts read normed input, with the norm in front of the next part.  Rows of up to 8192.
+// the sum of a block whose parts read normed input, with the norm in front of the next part.  Rows of up to 8192.  b
+// (of w's type) given: a layer norm, out = (residual - mean) / sqrt(variance + eps) * (w + plus_one) + b.  y_stride 0:
+// the same row is added to every row.
 int sa_residual_add_next_norm(const void* y, int y_dtype, int64_t y_stride, float mult, float* residual, const void* w,
-                              int w_dtype, float eps, int plus_one, void* out, int out_dtype, int T, int D,
+                              const void* b, int w_dtype, float eps, int plus_one, void* out, int out_dtype, int T, int D,
                               hipStream_t stream);
 
 // On fused projection rows [H * dk queries | K * dk keys | K * dv values | ...]: every query and key vector is cut into
@@ -366,10 +368,11 @@ int sa_short_conv(const void* x, int x_dtype, int64_t x_stride, const void* in_b
 // A product per head: out[t, h, o] = sum_i w[h][o][i] x[t, h, i] for o < O (w [H, O, I], row-major), summed in 32-bit
 // in the order of i.  x rows hold the heads x_head_stride apart, out rows out_head_stride apart.  tail > 0: the `tail`
 // entries behind a head's I inputs are copied behind its O outputs.  gate (null: none): one number per token and head,
-// gate[t * gate_stride + h]; the head's outputs are multiplied by sigmoid(gate).
+// gate[t * gate_stride + h] (gate_per_output: one per output, gate[t * gate_stride + h * O + o]); the head's outputs are
+// multiplied by sigmoid(gate).
 int sa_head_product(const void* x, int x_dtype, int64_t x_stride, int64_t x_head_stride, const void* w, int w_dtype,
                     void* out, int out_dtype, int64_t out_stride, int64_t out_head_stride, int T, int H, int I, int O,
-                    int tail, const void* gate, int gate_dtype, int64_t gate_stride, hipStream_t stream);
+                    int tail, const void* gate, int gate_dtype, int64_t gate_stride, int gate_per_output, hipStream_t stream);
 
 // The real-gated linear recurrence over each request's tokens (seq_meta [S, 4]: state slot, first row, rows, first
 // position), channel by channel, from and into state[slot] [C] float32:
@@ -453,10 +456,11 @@ int sa_exp_gates(const float* raw, int64_t raw_stride, const void* bias, int bia
 // S <- diag(a) S + c k v^T, out = S^T (q * q_mult) along every request's tokens; q, k, v are columns q_at, k_at, v_at
 // of proj's rows.  scalar: gates [T, >= 2 H] hold a and c per head; else gates [T, H dk] hold a per key channel and
 // c = 1; with tau > 0 these gates are z and a = sigmoid(z + gate_bias)^(1 / tau) (gate_bias [H dk] or null).  ones: the
-// state has a column dv whose value is always 1.  state [slot][H][dv + ones][dk]; out [T, H (dv + ones)].
+// state has a column dv whose value is always 1.  bonus [H dk] (null: none; with decays per key channel): out_t =
+// (S_(t-1) + diag(bonus) k v^T)^T q, the state before the token.  state [slot][H][dv + ones][dk]; out [T, H (dv + ones)].
 int sa_linear_state(const void* proj, int dtype, int64_t proj_stride, int q_at, int k_at, int v_at, float q_mult,
                     const float* gates, int64_t gates_stride, const void* gate_bias, int bias_dtype, float tau, int scalar,
-                    int H, int dk, int dv, int ones, float* state, int64_t state_stride, const int* seq_meta, int num_seqs,
+                    const void* bonus, int bonus_dtype, int H, int dk, int dv, int ones, float* state, int64_t state_stride, const int* seq_meta, int num_seqs,
                     float* out, hipStream_t stream);
 // x [T, H, size + 1] -> out[t, h, :] = unit_rms(x[t, h, :size] / (max(|x[t, h, size]|, floor[t, h]) + 1e-6)) * w[h, :]
 // * sigmoid(g[t, h, :]).
@@ -486,26 +490,38 @@ int sa_attention_inputs(const void* proj, int dtype, int64_t row_stride, int H, 
 // softmax over E logits, the top largest: experts [T, top], weights [T, top] = score * scale.
 int sa_route(const float* logits, int64_t stride, int T, int E, int top, float scale, int* experts, float* weights,
              hipStream_t stream);
-// Scores are sigmoids of the logits.  The choice goes by score + correction[e] (null: by the score); the experts form
-// `groups` equal groups of neighbours, a group's score is the sum of its two largest choice scores, and only experts of
-// the `keep` best groups can be chosen.  weights = score * scale (without the correction, not renormalized).
+// Scores are sigmoids of the logits, or their softmax.  The choice goes by score + correction[e] (null: by the score);
+// the experts form `groups` equal groups of neighbours, a group's score is the sum of its two largest choice scores
+// (group_best 2) or its largest one (1), and only experts of the `keep` best groups can be chosen.  weights = score *
+// scale (without the correction), with renorm >= 0 divided by the chosen scores' sum + renorm.
 int sa_route_choice(const float* logits, int64_t stride, int T, int E, int top, float scale, const void* correction,
-                    int corr_dtype, int groups, int keep, int* experts, float* weights, hipStream_t stream);
+                    int corr_dtype, int groups, int keep, int softmax, int group_best, float renorm, int* experts,
+                    float* weights, hipStream_t stream);
 // The most tiles of tile_rows (16 or 64) rows of one expert that P pairs over E experts make.
 int sa_expert_tiles_max(int P, int E, int tile_rows);
 // sorted [P]: the pairs by expert; plan [1 + 2 * sa_expert_tiles_max(P, E, tile_rows)]: the tiles.
 int sa_expert_sort(const int* experts, int P, int E, int tile_rows, int* sorted, int* plan, int plan_words,
                    hipStream_t stream);
-// w2 given: out[row] = act(a . w1[e]^T) * (a . w2[e]^T) in a's type; else out[row] = a . w1[e]^T in 32-bit, or, with
+// w2 given: out[row] = act(a . w1[e]^T) * (a . w2[e]^T) in a's type (or another rule of activations.h, with its limit); else out[row] = a . w1[e]^T in 32-bit, or, with
 // `activate`, act(a . w1[e]^T) in a's type (experts without a gate).  a's row is
 // the pair's token (a_by_token) or its place in the sorted order; out's row the pair (out_by_pair) or that place.
 // bfloat16 weights are tiled [E][ceil(N / 16)][ceil(K / 32)][64][8], 32-bit ones row-major [E][N][K].
 int sa_expert_product(const void* a, int dtype, int64_t a_stride, int a_by_token, int top, const void* w1, const void* w2,
-                      int N, int K, const int* sorted, const int* plan, int P, int E, int tile_rows, int act, void* out,
-                      int64_t out_stride, int out_by_pair, int activate, hipStream_t stream);
+                      int N, int K, const int* sorted, const int* plan, int P, int E, int tile_rows, int act, float limit,
+                      void* out, int64_t out_stride, int out_by_pair, int activate, hipStream_t stream);
 // out[t] = sum_k weights[t, k] y[t * top + k] + sigmoid(gate[t]) * shared[t]  (shared null: none; gate null: 1).
 int sa_expert_combine(const float* y, const float* weights, int top, const void* shared, int shared_dtype,
                       int64_t shared_stride, const float* gate, int64_t gate_stride, void* out, int out_dtype,
                       int64_t out_stride, int T, int D, hipStream_t stream);
 
+// out[t, s, :] = h[t] + (h[t - 1] - h[t]) * mu[s, :] for `streams` rows mu [streams, D]; the row before a request's first
+// one of the step is tails[slot] (float32 [slots, >= D]), which is set to the request's last row.  out [T, streams * D].
+int sa_token_shift(const void* h, int dtype, int64_t h_stride, const void* mu, int mu_dtype, int streams, float* tails,
+                   int64_t tail_stride, const int* seq_meta, int num_seqs, int max_q_len, void* out, int D,
+                   hipStream_t stream);
+// out[t, c] = exp(-exp(sum_r w[r, c] tanh(p[t, r]) + w0[c])), 32-bit; w [rank, C].
+int sa_low_rank_decay(const void* p, int p_dtype, int64_t p_stride, const void* w, int w_dtype, const void* w0, int w0_dtype,
+                      float* out, int T, int C, int rank, hipStream_t stream);
+// out[t] = [x[t] (D) | y[t] (E)] in out's type.
+int sa_concat_rows(const float* x, const float* y, void* out, int out_dtype, int T, int D, int E, hipStream_t stream);
 }

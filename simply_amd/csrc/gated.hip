@@ -99,14 +99,15 @@ static bool launch_residual_add_norm_typed(const void* y, int64_t y_stride, cons
 // ------------------------------------------------------------------ residual += mult * y; out = norm(residual)
 // The sum of a block that norms what its parts read (their results are added as they are, times a constant), fused
 // with the norm in front of the next part: out = h / sqrt(mean(h^2) + eps) * (w + plus_one) over the updated row h,
-// which is held in registers between the two.  y null: nothing is added.
-template <typename YT, typename OT, int NP>
+// which is held in registers between the two.  y null: nothing is added.  CENTERED: a layer norm instead, out =
+// (h - mean) / sqrt(mean((h - mean)^2) + eps) * (w + plus_one) + b.  A y_stride of 0 adds the same row to every row.
+template <typename YT, typename OT, int NP, bool CENTERED>
 __global__ __launch_bounds__(256) void residual_add_next_norm_kernel(
     const YT* __restrict__ y, int64_t y_stride, float mult, float* __restrict__ residual, const void* __restrict__ w,
-    int w_dtype, float eps, float plus_one, OT* __restrict__ out, int D) {
+    const void* __restrict__ b, int w_dtype, float eps, float plus_one, OT* __restrict__ out, int D) {
   __shared__ float scratch[16];
   const size_t yb = static_cast<size_t>(blockIdx.x) * y_stride, rb = static_cast<size_t>(blockIdx.x) * D;
-  float hv[NP], wv[NP];
+  float hv[NP], wv[NP], bv[CENTERED ? NP : 1];
   float ss = 0.f;
 #pragma unroll
   for (int p = 0; p < NP; ++p) {
@@ -115,38 +116,50 @@ __global__ __launch_bounds__(256) void residual_add_next_norm_kernel(
     const float yv = (ok && y != nullptr) ? to_float(y[yb + d]) : 0.f;
     const float h = ok ? residual[rb + d] : 0.f;
     wv[p] = ok ? load_f(w, w_dtype, d) + plus_one : 0.f;
+    if constexpr (CENTERED) bv[p] = ok ? load_f(b, w_dtype, d) : 0.f;
     hv[p] = y != nullptr ? h + mult * yv : h;
     if (ok && y != nullptr) residual[rb + d] = hv[p];
-    ss = fmaf(hv[p], hv[p], ss);
+    if constexpr (CENTERED) ss += hv[p];   // (entries beyond the row are zero)
+    else ss = fmaf(hv[p], hv[p], ss);
   }
   ss = block_sum(ss, scratch);
+  if constexpr (CENTERED) {
+    const float mean = ss / static_cast<float>(D);
+    ss = 0.f;
+#pragma unroll
+    for (int p = 0; p < NP; ++p) {
+      hv[p] -= mean;
+      if (threadIdx.x + p * 256 < D) ss = fmaf(hv[p], hv[p], ss);
+    }
+    ss = block_sum(ss, scratch);
+  }
   const float r = 1.f / sqrtf(ss / static_cast<float>(D) + eps);
 #pragma unroll
   for (int p = 0; p < NP; ++p) {
     const int d = threadIdx.x + p * 256;
-    if (d < D) out[rb + d] = from_float<OT>(hv[p] * r * wv[p]);
+    if (d < D) out[rb + d] = from_float<OT>(CENTERED ? fmaf(hv[p] * r, wv[p], bv[p]) : hv[p] * r * wv[p]);
   }
 }
 
-template <typename YT, typename OT>
-static void launch_residual_add_next_norm(const void* y, int64_t y_stride, float mult, float* residual, const void* w,
+template <typename YT, typename OT, bool CENTERED>
+static void launch_residual_add_next_norm(const void* y, int64_t y_stride, float mult, float* residual, const void* w, const void* b,
                                           int w_dtype, float eps, float plus_one, void* out, int T, int D,
                                           hipStream_t stream) {
   const YT* yp = static_cast<const YT*>(y);
   OT* op = static_cast<OT*>(out);
   if (D <= 1024)
-    residual_add_next_norm_kernel<YT, OT, 4><<<T, 256, 0, stream>>>(yp, y_stride, mult, residual, w, w_dtype, eps, plus_one, op, D);
+    residual_add_next_norm_kernel<YT, OT, 4, CENTERED><<<T, 256, 0, stream>>>(yp, y_stride, mult, residual, w, b, w_dtype, eps, plus_one, op, D);
   else if (D <= 2048)
-    residual_add_next_norm_kernel<YT, OT, 8><<<T, 256, 0, stream>>>(yp, y_stride, mult, residual, w, w_dtype, eps, plus_one, op, D);
+    residual_add_next_norm_kernel<YT, OT, 8, CENTERED><<<T, 256, 0, stream>>>(yp, y_stride, mult, residual, w, b, w_dtype, eps, plus_one, op, D);
   else if (D <= 4096)
-    residual_add_next_norm_kernel<YT, OT, 16><<<T, 256, 0, stream>>>(yp, y_stride, mult, residual, w, w_dtype, eps, plus_one, op, D);
+    residual_add_next_norm_kernel<YT, OT, 16, CENTERED><<<T, 256, 0, stream>>>(yp, y_stride, mult, residual, w, b, w_dtype, eps, plus_one, op, D);
   else
-    residual_add_next_norm_kernel<YT, OT, 32><<<T, 256, 0, stream>>>(yp, y_stride, mult, residual, w, w_dtype, eps, plus_one, op, D);
+    residual_add_next_norm_kernel<YT, OT, 32, CENTERED><<<T, 256, 0, stream>>>(yp, y_stride, mult, residual, w, b, w_dtype, eps, plus_one, op, D);
 }
 
 // ------------------------------------------------------------------ heads normed and gated
 // out[t, h, :] = (w ? x[t, h, :] / sqrt(mean(x[t, h, :]^2) + eps) * w : x[t, h, :]) * gate(g[t, h, :]),
-// gate 0: sigmoid, 1: silu.  One wave per (token, head); w [size] is shared by the heads.
+// gate 0: sigmoid, 1: silu.  One wave per (token, head); w [size] is shared by the heads, or (w_per_head) [H * size].
 __device__ inline float gate_value(int kind, float g) {
   const float s = 1.f / (1.f + expf(-g));
   return kind == 1 ? g * s : s;
@@ -155,7 +168,7 @@ __device__ inline float gate_value(int kind, float g) {
 __global__ __launch_bounds__(kWave) void gated_heads_kernel(
     const void* __restrict__ x, int x_dtype, int64_t x_stride, const void* __restrict__ g, int g_dtype,
     int64_t g_stride, const void* __restrict__ w, int w_dtype, float eps, int gate, void* __restrict__ out,
-    int out_dtype, int64_t out_stride, int size, int gate_per_head) {
+    int out_dtype, int64_t out_stride, int size, int gate_per_head, int w_per_head) {
   // gate_per_head: a gate row holds one number per head, which all of the head's entries share
   const int t = blockIdx.x, h = blockIdx.y;
   const size_t xb = static_cast<size_t>(t) * x_stride + static_cast<size_t>(h) * size;
@@ -173,7 +186,7 @@ __global__ __launch_bounds__(kWave) void gated_heads_kernel(
   }
   for (int d = threadIdx.x; d < size; d += kWave) {
     float v = load_f(x, x_dtype, xb + d);
-    if (w != nullptr) v = v * r * load_f(w, w_dtype, d);
+    if (w != nullptr) v = v * r * load_f(w, w_dtype, w_per_head ? static_cast<size_t>(h) * size + d : d);
     store_f(out, out_dtype, ob + d, v * gate_value(gate, load_f(g, g_dtype, gate_per_head ? gb : gb + d)));
   }
 }
@@ -379,7 +392,7 @@ extern "C" int sa_residual_add_norm(const void* y, int y_dtype, int64_t y_stride
   if (T == 0) return 0;
   SA_REQUIRE(T > 0 && D > 0 && residual != nullptr, "residual_add_norm: bad sizes T=%d D=%d", T, D);
   SA_REQUIRE(y != nullptr || out != nullptr, "residual_add_norm: nothing to add and nowhere to hand the residual on");
-  SA_REQUIRE(y == nullptr || y_stride >= D, "residual_add_norm: row stride %lld is below the width %d",
+  SA_REQUIRE(y == nullptr || y_stride == 0 || y_stride >= D, "residual_add_norm: row stride %lld is below the width %d",
              (long long)y_stride, D);
   SA_REQUIRE(eps >= 0.f, "residual_add_norm: eps must not be negative");
   // the usual combinations of element types have kernels of their own (a bfloat16 run, a 32-bit run)
@@ -396,32 +409,37 @@ extern "C" int sa_residual_add_norm(const void* y, int y_dtype, int64_t y_stride
 }
 
 extern "C" int sa_residual_add_next_norm(const void* y, int y_dtype, int64_t y_stride, float mult, float* residual,
-                                         const void* w, int w_dtype, float eps, int plus_one, void* out, int out_dtype,
-                                         int T, int D, hipStream_t stream) {
+                                         const void* w, const void* b, int w_dtype, float eps, int plus_one, void* out,
+                                         int out_dtype, int T, int D, hipStream_t stream) {
   if (T == 0) return 0;
   SA_REQUIRE(T > 0 && D > 0 && D <= 8192 && residual != nullptr && w != nullptr && out != nullptr,
              "residual_add_next_norm: bad sizes T=%d D=%d (rows of at most 8192), or a null pointer", T, D);
-  SA_REQUIRE(y == nullptr || y_stride >= D, "residual_add_next_norm: row stride %lld is below the width %d",
+  SA_REQUIRE(y == nullptr || y_stride == 0 || y_stride >= D, "residual_add_next_norm: row stride %lld is below the width %d",
              (long long)y_stride, D);
   SA_REQUIRE(eps >= 0.f, "residual_add_next_norm: eps must not be negative");
   const float plus = plus_one ? 1.f : 0.f;
   const bool yb = y == nullptr ? out_dtype == kBF16 : y_dtype == kBF16;
   SA_REQUIRE((y == nullptr || y_dtype == kBF16 || y_dtype == kF32) && (out_dtype == kBF16 || out_dtype == kF32),
              "residual_add_next_norm: rows are bfloat16 or float32");
-  if (yb && out_dtype == kBF16)
-    launch_residual_add_next_norm<bf16, bf16>(y, y_stride, mult, residual, w, w_dtype, eps, plus, out, T, D, stream);
-  else if (yb)
-    launch_residual_add_next_norm<bf16, float>(y, y_stride, mult, residual, w, w_dtype, eps, plus, out, T, D, stream);
-  else if (out_dtype == kBF16)
-    launch_residual_add_next_norm<float, bf16>(y, y_stride, mult, residual, w, w_dtype, eps, plus, out, T, D, stream);
-  else
-    launch_residual_add_next_norm<float, float>(y, y_stride, mult, residual, w, w_dtype, eps, plus, out, T, D, stream);
+#define SA_NEXT_NORM(YT, OT)                                                                                            \
+  do {                                                                                                                  \
+    if (b != nullptr)                                                                                                   \
+      launch_residual_add_next_norm<YT, OT, true>(y, y_stride, mult, residual, w, b, w_dtype, eps, plus, out, T, D, stream); \
+    else                                                                                                                \
+      launch_residual_add_next_norm<YT, OT, false>(y, y_stride, mult, residual, w, b, w_dtype, eps, plus, out, T, D, stream); \
+  } while (0)
+  if (yb && out_dtype == kBF16) SA_NEXT_NORM(bf16, bf16);
+  else if (yb) SA_NEXT_NORM(bf16, float);
+  else if (out_dtype == kBF16) SA_NEXT_NORM(float, bf16);
+  else SA_NEXT_NORM(float, float);
+#undef SA_NEXT_NORM
   return check_launch("residual_add_next_norm");
 }
 
 extern "C" int sa_gated_heads(const void* x, int x_dtype, int64_t x_stride, const void* g, int g_dtype, int64_t g_stride,
                               const void* w, int w_dtype, float eps, int gate, void* out, int out_dtype,
-                              int64_t out_stride, int T, int H, int size, int gate_per_head, hipStream_t stream) {
+                              int64_t out_stride, int T, int H, int size, int gate_per_head, int w_per_head,
+                              hipStream_t stream) {
   if (T == 0) return 0;
   SA_REQUIRE(T > 0 && H > 0 && size > 0 && x != nullptr && g != nullptr && out != nullptr,
              "gated_heads: bad sizes T=%d H=%d size=%d", T, H, size);
@@ -431,7 +449,7 @@ extern "C" int sa_gated_heads(const void* x, int x_dtype, int64_t x_stride, cons
   SA_REQUIRE(gate == 0 || gate == 1, "gated_heads: unknown gate %d (0: sigmoid, 1: silu)", gate);
   SA_REQUIRE(H <= 65535, "gated_heads: at most 65535 heads");
   gated_heads_kernel<<<dim3(T, H), kWave, 0, stream>>>(x, x_dtype, x_stride, g, g_dtype, g_stride, w, w_dtype, eps, gate,
-                                                       out, out_dtype, out_stride, size, gate_per_head);
+                                                       out, out_dtype, out_stride, size, gate_per_head, w_per_head);
   return check_launch("gated_heads");
 }
 

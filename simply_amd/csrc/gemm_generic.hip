@@ -81,7 +81,7 @@ __global__ __launch_bounds__(256) void gemm_generic_kernel(const TA* __restrict_
       float v = acc[i][j];
       if (EPI == 1) {
         // both products are rounded to the activation type first, as separate matrix products would be
-        v = gated_activation_exact(act, to_float(from_float<TC>(v))) * to_float(from_float<TC>(acc2[i][j]));
+        v = gated_product_exact(act, cap, to_float(from_float<TC>(v)), to_float(from_float<TC>(acc2[i][j])));
       } else if (EPI == 2) {
         v = cap * tanhf(v / cap);
       }

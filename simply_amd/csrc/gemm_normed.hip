@@ -425,7 +425,7 @@ __global__ __launch_bounds__(kWaves* kWave) void gemm_normed_kernel(
           sum[p] = t;
         }
         float v = sum[0];
-        if (EPI == 1) v = gated_activation(activation, to_float(float_to_bf16(v))) * to_float(float_to_bf16(sum[NP - 1]));
+        if (EPI == 1) v = gated_product(activation, cap, to_float(float_to_bf16(v)), to_float(float_to_bf16(sum[NP - 1])));
         else if (EPI == 2) v = cap * tanhf(v / cap);
         store_f(C, c_dtype, static_cast<size_t>(ml) * ldc + n, v);
       }
@@ -505,7 +505,7 @@ extern "C" int sa_gemm_normed(const void* y, const float* h_in, float* h_out, co
   const int activation = epilogue_activation(epilogue);
   epilogue = epilogue_kind(epilogue);
   SA_REQUIRE(epilogue >= 0 && epilogue <= 2 && (epilogue != 2 || cap > 0.f), "gemm_normed: bad epilogue");
-  SA_REQUIRE(activation >= 0 && activation < kNumActivations && (epilogue == 1 || activation == 0),
+  SA_REQUIRE(activation >= 0 && activation < kNumGatedRules && (epilogue == 1 || activation == 0),
              "gemm_normed: unknown activation %d", activation);
   const bf16* yb = static_cast<const bf16*>(y);
   const bf16* w = static_cast<const bf16*>(W);

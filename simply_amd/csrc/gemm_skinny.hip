@@ -210,7 +210,7 @@ __global__ __launch_bounds__(1024) void gemm_skinny_kernel(const bf16* __restric
     float v = sum[0];
     if (EPI == 1) {
       // both products are rounded to bfloat16 first, as separate matrix products would be
-      v = gated_activation(act, to_float(float_to_bf16(v))) * to_float(float_to_bf16(sum[NP - 1]));
+      v = gated_product(act, cap, to_float(float_to_bf16(v)), to_float(float_to_bf16(sum[NP - 1])));
     } else if (EPI == 2) {
       v = cap * tanhf(v / cap);
     } else if (act > 0) {

@@ -202,7 +202,7 @@ void gemm_tiled_kernel(const bf16* __restrict__ A, int64_t lda, const bf16* __re
         if (n >= N) continue;
         float x;
         if (EPI == 1)
-          x = gated_activation(act, to_float(float_to_bf16(acc[i][2 * j][v]))) * to_float(float_to_bf16(acc[i][2 * j + 1][v]));
+          x = gated_product(act, cap, to_float(float_to_bf16(acc[i][2 * j][v])), to_float(float_to_bf16(acc[i][2 * j + 1][v])));
         else if (EPI == 2) x = cap * tanhf(acc[i][j][v] / cap);
         else x = acc[i][j][v];
         store_f(C, c_dtype, static_cast<size_t>(m) * ldc + n, x);
@@ -237,7 +237,7 @@ __global__ void gemm_reduce_kernel(const float* __restrict__ partials, int KS, v
         y += py[j];
       }
     }
-    if (EPI == 1) x = gated_activation(act, to_float(float_to_bf16(x))) * to_float(float_to_bf16(y));
+    if (EPI == 1) x = gated_product(act, cap, to_float(float_to_bf16(x)), to_float(float_to_bf16(y)));
     else if (EPI == 2) x = cap * tanhf(x / cap);
     store_f(C, c_dtype, m * ldc + n, x);
   }
@@ -274,7 +274,7 @@ __global__ __launch_bounds__(256) void gemm_reduce4_kernel(const float* __restri
     const float g[4] = {y.x, y.y, y.z, y.w};
 #pragma unroll
     for (int v = 0; v < 4; ++v) {
-      if (EPI == 1) r[v] = gated_activation(act, to_float(float_to_bf16(r[v]))) * to_float(float_to_bf16(g[v]));
+      if (EPI == 1) r[v] = gated_product(act, cap, to_float(float_to_bf16(r[v])), to_float(float_to_bf16(g[v])));
       else if (EPI == 2) r[v] = cap * tanhf(r[v] / cap);
     }
     if (c_dtype == kF32) {

@@ -67,7 +67,7 @@ __device__ __forceinline__ void load_to_lds(const bf16* base, uint32_t offset, u
 template <int WM, int WN, int WAVES_M, int EPI, int NSTAGE, int WAVES>
 __global__ __launch_bounds__(WAVES * 64) void gemm_wide_kernel(const bf16* __restrict__ A, int64_t lda,
                                                         const bf16* __restrict__ W, bf16* __restrict__ C, int64_t ldc,
-                                                        int M, int N, int K, int chunks, int act,
+                                                        int M, int N, int K, int chunks, int act, float limit,
                                                         float* __restrict__ partials) {
   constexpr int WAVES_N = WAVES / WAVES_M;
   constexpr int MT = WAVES_M * WM, NT = WAVES_N * WN;  // 16-row tiles of A and of W per workgroup
@@ -283,8 +283,8 @@ __global__ __launch_bounds__(WAVES * 64) void gemm_wide_kernel(const bf16* __res
 #pragma unroll
       for (int v = 0; v < 4; ++v) {
         if (EPI == 1)
-          x[v] = gated_activation(act, to_float(float_to_bf16(acc[i][2 * j][v]))) *
-                 to_float(float_to_bf16(acc[i][2 * j + 1][v]));
+          x[v] = gated_product(act, limit, to_float(float_to_bf16(acc[i][2 * j][v])),
+                               to_float(float_to_bf16(acc[i][2 * j + 1][v])));
         else
           x[v] = acc[i][j][v];
         // (without another epilogue, act > 0 asks for the activation act - 1 of the product rounded to bfloat16)
@@ -300,19 +300,19 @@ __global__ __launch_bounds__(WAVES * 64) void gemm_wide_kernel(const bf16* __res
 
 template <int WM, int WN, int WAVES_M, int NSTAGE, int WAVES = 8>
 static void launch(const bf16* A, int64_t lda, const bf16* W, bf16* C, int64_t ldc, int M, int N, int K, int epi,
-                   int act, int ks, float* partials, hipStream_t stream) {
+                   int act, float limit, int ks, float* partials, hipStream_t stream) {
   constexpr int BM = WAVES_M * WM * 16, BNW = (WAVES / WAVES_M) * WN * 16;
   const int NW = epi == 1 ? 2 * ((N + 15) / 16) * 16 : N;
   const dim3 grid((NW + BNW - 1) / BNW, (M + BM - 1) / BM, ks);
   if (epi == 1)
     gemm_wide_kernel<WM, WN, WAVES_M, 1, NSTAGE, WAVES><<<grid, WAVES * 64, 0, stream>>>(A, lda, W, C, ldc, M, N, K, K / 32,
-                                                                                         act, nullptr);
+                                                                                         act, limit, nullptr);
   else if (ks > 1)
     gemm_wide_kernel<WM, WN, WAVES_M, 3, NSTAGE, WAVES><<<grid, WAVES * 64, 0, stream>>>(A, lda, W, C, ldc, M, N, K, K / 32,
-                                                                                         act, partials);
+                                                                                         act, limit, partials);
   else
     gemm_wide_kernel<WM, WN, WAVES_M, 0, NSTAGE, WAVES><<<grid, WAVES * 64, 0, stream>>>(A, lda, W, C, ldc, M, N, K, K / 32,
-                                                                                         act, nullptr);
+                                                                                         act, limit, nullptr);
 }
 
 }  // namespace wide
@@ -405,7 +405,7 @@ static double plan_shape(int M, int N, int K, int epi, bool have_workspace, size
 // ks > 1 cuts K over that many workgroups per tile (no epilogue only; the partial tiles go through `workspace`,
 // which must hold ks * M * N floats).
 int gemm_wide(const void* A, int64_t lda, const void* W, void* C, int64_t ldc, int M, int N, int K, int epi, int act,
-              int shape, int ks, void* workspace, size_t workspace_bytes, hipStream_t stream, int* planes_left) {
+              float limit, int shape, int ks, void* workspace, size_t workspace_bytes, hipStream_t stream, int* planes_left) {
   if (ks < 1) ks = 1;
   if (ks > K / wide::BK) ks = K / wide::BK;
   if (ks > 1 && (epi != 0 || workspace == nullptr || static_cast<size_t>(ks) * M * N * sizeof(float) > workspace_bytes)) {
@@ -418,21 +418,21 @@ int gemm_wide(const void* A, int64_t lda, const void* W, void* C, int64_t ldc, i
   bf16* c = static_cast<bf16*>(C);
   if (shape == 0) plan_shape(M, N, K, epi, ws != nullptr, workspace_bytes, shape, ks);
   switch (shape) {
-    case 2256192: wide::launch<4, 6, 4, 2>(a, lda, w, c, ldc, M, N, K, epi, act, ks, ws, stream); break;
-    case 3256128: wide::launch<4, 4, 4, 3>(a, lda, w, c, ldc, M, N, K, epi, act, ks, ws, stream); break;
-    case 3128256: wide::launch<4, 4, 2, 3>(a, lda, w, c, ldc, M, N, K, epi, act, ks, ws, stream); break;
-    case 3192128: wide::launch<3, 4, 4, 3>(a, lda, w, c, ldc, M, N, K, epi, act, ks, ws, stream); break;
-    case 2128192: wide::launch<4, 6, 2, 2, 4>(a, lda, w, c, ldc, M, N, K, epi, act, ks, ws, stream); break;  // two workgroups per CU
+    case 2256192: wide::launch<4, 6, 4, 2>(a, lda, w, c, ldc, M, N, K, epi, act, limit, ks, ws, stream); break;
+    case 3256128: wide::launch<4, 4, 4, 3>(a, lda, w, c, ldc, M, N, K, epi, act, limit, ks, ws, stream); break;
+    case 3128256: wide::launch<4, 4, 2, 3>(a, lda, w, c, ldc, M, N, K, epi, act, limit, ks, ws, stream); break;
+    case 3192128: wide::launch<3, 4, 4, 3>(a, lda, w, c, ldc, M, N, K, epi, act, limit, ks, ws, stream); break;
+    case 2128192: wide::launch<4, 6, 2, 2, 4>(a, lda, w, c, ldc, M, N, K, epi, act, limit, ks, ws, stream); break;  // two workgroups per CU
     // small tiles, for products of a few hundred rows whose large tiles would leave most CUs idle (two or more
     // workgroups per CU fit: 36 to 72 KiB of LDS each)
-    case 3128128: wide::launch<2, 4, 4, 3>(a, lda, w, c, ldc, M, N, K, epi, act, ks, ws, stream); break;
-    case 3128064: wide::launch<2, 2, 4, 3>(a, lda, w, c, ldc, M, N, K, epi, act, ks, ws, stream); break;
-    case 3064128: wide::launch<1, 4, 4, 3>(a, lda, w, c, ldc, M, N, K, epi, act, ks, ws, stream); break;
-    case 3064064: wide::launch<1, 2, 4, 3>(a, lda, w, c, ldc, M, N, K, epi, act, ks, ws, stream); break;
-    case 6064064: wide::launch<1, 2, 4, 6>(a, lda, w, c, ldc, M, N, K, epi, act, ks, ws, stream); break;
-    case 5128064: wide::launch<2, 2, 4, 5>(a, lda, w, c, ldc, M, N, K, epi, act, ks, ws, stream); break;
-    case 4128128: wide::launch<2, 4, 4, 4>(a, lda, w, c, ldc, M, N, K, epi, act, ks, ws, stream); break;
-    case 6064128: wide::launch<1, 4, 4, 6>(a, lda, w, c, ldc, M, N, K, epi, act, ks, ws, stream); break;
+    case 3128128: wide::launch<2, 4, 4, 3>(a, lda, w, c, ldc, M, N, K, epi, act, limit, ks, ws, stream); break;
+    case 3128064: wide::launch<2, 2, 4, 3>(a, lda, w, c, ldc, M, N, K, epi, act, limit, ks, ws, stream); break;
+    case 3064128: wide::launch<1, 4, 4, 3>(a, lda, w, c, ldc, M, N, K, epi, act, limit, ks, ws, stream); break;
+    case 3064064: wide::launch<1, 2, 4, 3>(a, lda, w, c, ldc, M, N, K, epi, act, limit, ks, ws, stream); break;
+    case 6064064: wide::launch<1, 2, 4, 6>(a, lda, w, c, ldc, M, N, K, epi, act, limit, ks, ws, stream); break;
+    case 5128064: wide::launch<2, 2, 4, 5>(a, lda, w, c, ldc, M, N, K, epi, act, limit, ks, ws, stream); break;
+    case 4128128: wide::launch<2, 4, 4, 4>(a, lda, w, c, ldc, M, N, K, epi, act, limit, ks, ws, stream); break;
+    case 6064128: wide::launch<1, 4, 4, 6>(a, lda, w, c, ldc, M, N, K, epi, act, limit, ks, ws, stream); break;
     default:
       set_error("gemm: unknown wide tile %d", shape);
       return 1;

@@ -75,13 +75,14 @@ __global__ __launch_bounds__(kWave) void exp_gates_kernel(const float* __restric
 // decays of kStateTokens tokens at a time go through LDS, asked for a tile ahead.  SCALAR: one decay and one input
 // factor per head and token (gates [T, >= 2 H]: decays, then factors); else a decay per key channel (gates
 // [T, H * dk]) and no factor.  `ones`: 1 if the state has one more column whose value is always 1 (column dv).
-// The state of a head is kept column by column, [dv + ones][dk].
+// The state of a head is kept column by column, [dv + ones][dk].  BONUS: a token reads the state as it was before it
+// and its own k v^T through a factor per key channel, o = (S_(t-1) + diag(bonus) k v^T)^T q (bonus [H * dk]).
 constexpr int kStateTokens = 16;
-template <int DK, int LPC, bool SCALAR, typename XT>
+template <int DK, int LPC, bool SCALAR, bool BONUS, typename XT>
 __global__ __launch_bounds__(256) void linear_state_kernel(
     const XT* __restrict__ proj, int64_t proj_stride, int q_at, int k_at, int v_at, float q_mult,
     const float* __restrict__ gates, int64_t gates_stride, const void* __restrict__ gate_bias, int bias_dtype,
-    float inv_tau, int H, int dk, int dv, int ones, float* __restrict__ state, int64_t state_stride,
+    float inv_tau, const void* __restrict__ bonus, int bonus_dtype, int H, int dk, int dv, int ones, float* __restrict__ state, int64_t state_stride,
     const int* __restrict__ seq_meta, float* __restrict__ out) {
   constexpr int R = DK / LPC, COLS = 256 / LPC;
   constexpr int AD = SCALAR ? 1 : DK;
@@ -94,10 +95,11 @@ __global__ __launch_bounds__(256) void linear_state_kernel(
   const int col = blockIdx.z * COLS + tid / LPC, part = tid % LPC;
   const bool live = col < CT;
   float* S = state + static_cast<size_t>(slot) * state_stride + static_cast<size_t>(h) * dk * CT;
-  float s[R];
+  float s[R], bo[BONUS ? R : 1];
 #pragma unroll
   for (int r = 0; r < R; ++r) {
     const int i = r * LPC + part;
+    if constexpr (BONUS) bo[r] = i < dk ? load_f(bonus, bonus_dtype, static_cast<size_t>(h) * dk + i) : 0.f;
     s[r] = (live && i < dk) ? S[static_cast<size_t>(col) * dk + i] : 0.f;
   }
   constexpr int PQ = kStateTokens * DK / 256, PV = (kStateTokens * COLS + 255) / 256;
@@ -178,8 +180,14 @@ __global__ __launch_bounds__(256) void linear_state_kernel(
           for (int r = 0; r < R; ++r) {
             float a = a0;
             if constexpr (!SCALAR) a = as[j][(r * LPC + part) % AD];
-            s[r] = fmaf(ks[j][r * LPC + part], u, s[r] * a);
-            d[r % 4] = fmaf(s[r], qs[j][r * LPC + part], d[r % 4]);
+            if constexpr (BONUS) {
+              const float kv = ks[j][r * LPC + part] * u;
+              d[r % 4] = fmaf(fmaf(bo[r], kv, s[r]), qs[j][r * LPC + part], d[r % 4]);
+              s[r] = fmaf(s[r], a, kv);
+            } else {
+              s[r] = fmaf(ks[j][r * LPC + part], u, s[r] * a);
+              d[r % 4] = fmaf(s[r], qs[j][r * LPC + part], d[r % 4]);
+            }
           }
           o[i] = (d[0] + d[1]) + (d[2] + d[3]);
         }
@@ -250,7 +258,7 @@ extern "C" int sa_exp_gates(const float* raw, int64_t raw_stride, const void* bi
 
 extern "C" int sa_linear_state(const void* proj, int dtype, int64_t proj_stride, int q_at, int k_at, int v_at,
                                float q_mult, const float* gates, int64_t gates_stride, const void* gate_bias,
-                               int bias_dtype, float tau, int scalar, int H, int dk, int dv, int ones, float* state,
+                               int bias_dtype, float tau, int scalar, const void* bonus, int bonus_dtype, int H, int dk, int dv, int ones, float* state,
                                int64_t state_stride, const int* seq_meta, int num_seqs, float* out, hipStream_t stream) {
   if (num_seqs == 0) return 0;
   SA_REQUIRE(num_seqs > 0 && num_seqs <= 65535 && H > 0 && H <= 65535 && dk > 0 && dv > 0 && (ones == 0 || ones == 1),
@@ -268,24 +276,28 @@ extern "C" int sa_linear_state(const void* proj, int dtype, int64_t proj_stride,
   SA_REQUIRE(CT <= 65535 * 4, "linear_state: too many columns");
   SA_REQUIRE(tau >= 0.f && (scalar == 0 || tau == 0.f), "linear_state: tau belongs to decays per channel and is not negative");
   const float inv_tau = tau > 0.f ? 1.f / tau : 0.f;
-#define SA_STATE_LAUNCH(DK, LPC, SC, XT)                                                                             \
-  linear_state_kernel<DK, LPC, SC, XT><<<dim3(num_seqs, H, (CT + 256 / LPC - 1) / (256 / LPC)), 256, 0, stream>>>(   \
+  SA_REQUIRE(bonus == nullptr || (scalar == 0 && (bonus_dtype == kF32 || bonus_dtype == kBF16)),
+             "linear_state: a bonus goes with decays per key channel");
+#define SA_STATE_LAUNCH(DK, LPC, SC, BO, XT)                                                                             \
+  linear_state_kernel<DK, LPC, SC, BO, XT><<<dim3(num_seqs, H, (CT + 256 / LPC - 1) / (256 / LPC)), 256, 0, stream>>>(   \
       static_cast<const XT*>(proj), proj_stride, q_at, k_at, v_at, q_mult, gates, gates_stride, gate_bias, bias_dtype, \
-      inv_tau, H, dk, dv, ones, state, state_stride, seq_meta, out)
-#define SA_STATE_SIZES(SC, XT)                       \
+      inv_tau, bonus, bonus_dtype, H, dk, dv, ones, state, state_stride, seq_meta, out)
+#define SA_STATE_SIZES(SC, BO, XT)                       \
   do {                                               \
-    if (dk <= 16) SA_STATE_LAUNCH(16, 4, SC, XT);    \
-    else if (dk <= 32) SA_STATE_LAUNCH(32, 4, SC, XT);    \
-    else if (dk <= 64) SA_STATE_LAUNCH(64, 16, SC, XT);   \
-    else if (dk <= 128) SA_STATE_LAUNCH(128, 32, SC, XT); \
-    else SA_STATE_LAUNCH(256, 64, SC, XT);           \
+    if (dk <= 16) SA_STATE_LAUNCH(16, 4, SC, BO, XT);    \
+    else if (dk <= 32) SA_STATE_LAUNCH(32, 4, SC, BO, XT);    \
+    else if (dk <= 64) SA_STATE_LAUNCH(64, 16, SC, BO, XT);   \
+    else if (dk <= 128) SA_STATE_LAUNCH(128, 32, SC, BO, XT); \
+    else SA_STATE_LAUNCH(256, 64, SC, BO, XT);           \
   } while (0)
   if (dtype == kBF16) {
-    if (scalar) SA_STATE_SIZES(true, bf16);
-    else SA_STATE_SIZES(false, bf16);
+    if (scalar) SA_STATE_SIZES(true, false, bf16);
+    else if (bonus != nullptr) SA_STATE_SIZES(false, true, bf16);
+    else SA_STATE_SIZES(false, false, bf16);
   } else {
-    if (scalar) SA_STATE_SIZES(true, float);
-    else SA_STATE_SIZES(false, float);
+    if (scalar) SA_STATE_SIZES(true, false, float);
+    else if (bonus != nullptr) SA_STATE_SIZES(false, true, float);
+    else SA_STATE_SIZES(false, false, float);
   }
 #undef SA_STATE_SIZES
 #undef SA_STATE_LAUNCH

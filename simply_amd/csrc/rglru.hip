@@ -22,7 +22,7 @@ constexpr int kHpChunk = 32;    // inputs staged at a time
 __global__ __launch_bounds__(256) void head_product_kernel(
     const void* __restrict__ x, int x_dtype, int64_t x_stride, int64_t x_head_stride, const void* __restrict__ w,
     int w_dtype, void* __restrict__ out, int out_dtype, int64_t out_stride, int64_t out_head_stride, int T, int I, int O,
-    int tail, const void* __restrict__ gate, int gate_dtype, int64_t gate_stride) {
+    int tail, const void* __restrict__ gate, int gate_dtype, int64_t gate_stride, int gate_per_output) {
   // (rows four words longer: a staging write's 32 inputs of one output then fall into 16 banks, and rows stay 16-byte aligned)
   __shared__ __align__(16) float ws[kHpChunk][kHpOutputs + 4];
   __shared__ __align__(16) float xs[kHpChunk][kHpTokens + 4];
@@ -63,12 +63,18 @@ __global__ __launch_bounds__(256) void head_product_kernel(
     const int t = t0 + 4 * ty + k;
     if (t >= T) continue;
     const size_t ob = static_cast<size_t>(t) * out_stride + static_cast<size_t>(h) * out_head_stride;
-    const float gv = gate != nullptr
+    const float gv = gate != nullptr && !gate_per_output
                          ? 1.f / (1.f + expf(-load_f(gate, gate_dtype, static_cast<size_t>(t) * gate_stride + h)))
                          : 1.f;
 #pragma unroll
-    for (int j = 0; j < 4; ++j)
-      if (o0 + 4 * tx + j < O) store_f(out, out_dtype, ob + o0 + 4 * tx + j, acc[k][j] * gv);
+    for (int j = 0; j < 4; ++j) {
+      const int o = o0 + 4 * tx + j;
+      if (o >= O) continue;
+      float g = gv;
+      if (gate_per_output)
+        g = 1.f / (1.f + expf(-load_f(gate, gate_dtype, static_cast<size_t>(t) * gate_stride + static_cast<size_t>(h) * O + o)));
+      store_f(out, out_dtype, ob + o, acc[k][j] * g);
+    }
     if (blockIdx.z == 0) {
       const size_t xb = static_cast<size_t>(t) * x_stride + static_cast<size_t>(h) * x_head_stride + I;
       for (int e = tx; e < tail; e += 16) store_f(out, out_dtype, ob + O + e, load_f(x, x_dtype, xb + e));
@@ -83,7 +89,7 @@ constexpr int kHpFewTokens = 8;
 __global__ __launch_bounds__(256) void head_product_few_kernel(
     const void* __restrict__ x, int x_dtype, int64_t x_stride, int64_t x_head_stride, const void* __restrict__ w,
     int w_dtype, void* __restrict__ out, int out_dtype, int64_t out_stride, int64_t out_head_stride, int T, int I, int O,
-    int tail, const void* __restrict__ gate, int gate_dtype, int64_t gate_stride) {
+    int tail, const void* __restrict__ gate, int gate_dtype, int64_t gate_stride, int gate_per_output) {
   const int lane = threadIdx.x % kWave, o = blockIdx.x * 4 + threadIdx.x / kWave, h = blockIdx.y;
   const int t0 = blockIdx.z * kHpFewTokens;
   if (o >= O) return;   // (a whole wave)
@@ -108,7 +114,8 @@ __global__ __launch_bounds__(256) void head_product_few_kernel(
     const size_t ob = static_cast<size_t>(t) * out_stride + static_cast<size_t>(h) * out_head_stride;
     if (lane == 0) {
       const float gv = gate != nullptr
-                           ? 1.f / (1.f + expf(-load_f(gate, gate_dtype, static_cast<size_t>(t) * gate_stride + h)))
+                           ? 1.f / (1.f + expf(-load_f(gate, gate_dtype, static_cast<size_t>(t) * gate_stride +
+                                                                               (gate_per_output ? static_cast<size_t>(h) * O + o : h))))
                            : 1.f;
       store_f(out, out_dtype, ob + o, v * gv);
     }
@@ -243,7 +250,7 @@ using namespace sa;
 extern "C" int sa_head_product(const void* x, int x_dtype, int64_t x_stride, int64_t x_head_stride, const void* w,
                                int w_dtype, void* out, int out_dtype, int64_t out_stride, int64_t out_head_stride, int T,
                                int H, int I, int O, int tail, const void* gate, int gate_dtype, int64_t gate_stride,
-                               hipStream_t stream) {
+                               int gate_per_output, hipStream_t stream) {
   if (T == 0) return 0;
   SA_REQUIRE(T > 0 && H > 0 && I > 0 && O > 0 && tail >= 0 && x != nullptr && w != nullptr && out != nullptr,
              "head_product: bad sizes T=%d H=%d I=%d O=%d tail=%d", T, H, I, O, tail);
@@ -251,18 +258,19 @@ extern "C" int sa_head_product(const void* x, int x_dtype, int64_t x_stride, int
                  x_stride >= static_cast<int64_t>(H - 1) * x_head_stride + I + tail &&
                  out_stride >= static_cast<int64_t>(H - 1) * out_head_stride + O + tail,
              "head_product: a stride is below what %d heads of %d inputs and %d outputs need", H, I + tail, O + tail);
-  SA_REQUIRE(gate == nullptr || gate_stride >= H, "head_product: the gates' row stride is below the heads");
+  SA_REQUIRE(gate == nullptr || gate_stride >= static_cast<int64_t>(H) * (gate_per_output ? O : 1), "head_product: the gates' row stride is below the heads");
   const int tiles = (T + kHpTokens - 1) / kHpTokens, cols = (O + kHpOutputs - 1) / kHpOutputs;
   SA_REQUIRE(H <= 65535 && cols <= 65535, "head_product: too many heads or outputs");
   if (T <= 2 * kHpFewTokens && (O + 3) / 4 <= 65535) {
     head_product_few_kernel<<<dim3((O + 3) / 4, H, (T + kHpFewTokens - 1) / kHpFewTokens), 256, 0, stream>>>(
         x, x_dtype, x_stride, x_head_stride, w, w_dtype, out, out_dtype, out_stride, out_head_stride, T, I, O, tail, gate,
-        gate_dtype, gate_stride);
+        gate_dtype, gate_stride, gate != nullptr && gate_per_output);
     return check_launch("head_product_few");
   }
   head_product_kernel<<<dim3(tiles, H, cols), 256, 0, stream>>>(x, x_dtype, x_stride, x_head_stride, w, w_dtype, out,
                                                                 out_dtype, out_stride, out_head_stride, T, I, O, tail,
-                                                                gate, gate_dtype, gate_stride);
+                                                                gate, gate_dtype, gate_stride,
+                                                                gate != nullptr && gate_per_output);
   return check_launch("head_product");
 }
 

@@ -50,7 +50,7 @@ __global__ __launch_bounds__(kWave) void route_kernel(const float* __restrict__ 
     for (int i = kRouteSlots - 1; i >= 0; --i)
       if (z[i] == best) mine = static_cast<float>(lane + i * kWave);
     const float first = -wave_max(-mine);
-    const int e = static_cast<int>(first);
+    const int e = first < static_cast<float>(E) ? static_cast<int>(first) : E - 1;   // (logits that are no numbers: some expert)
 #pragma unroll
     for (int i = 0; i < kRouteSlots; ++i)
       if (lane + i * kWave == e) z[i] = -1.f;
@@ -61,28 +61,48 @@ __global__ __launch_bounds__(kWave) void route_kernel(const float* __restrict__ 
   }
 }
 
-// A wave per token, for routers whose scores are sigmoids of the logits.  The choice is made by score + correction[e]
-// (correction null: by the score); the experts form `groups` equal groups of neighbours, a group's score is the sum of
-// its two largest choice scores (of its only one, in groups of one), and only experts of the `keep` groups with the
-// largest scores can be chosen (of equal ones the lowest index, for groups and for experts).  weight = score * scale,
-// without the correction and not renormalized.  Choice scores can be negative: what is taken or shut out is -inf.
+// A wave per token, for routers with options.  Scores are sigmoids of the logits or (`softmax`) their softmax over all
+// experts.  The choice is made by score + correction[e] (correction null: by the score); the experts form `groups`
+// equal groups of neighbours, a group's score is the sum of its two largest choice scores (group_best 2; of its only
+// one, in groups of one) or the largest one (group_best 1), and only experts of the `keep` groups with the largest
+// scores can be chosen (of equal ones the lowest index, for groups and for experts).  weight = score * scale without
+// the correction, with renorm >= 0 divided by the chosen scores' sum + renorm.  Choice scores can be negative: what is
+// taken or shut out is -inf.
 __global__ __launch_bounds__(kWave) void route_choice_kernel(const float* __restrict__ logits, int64_t stride, int E,
                                                              int top, float scale, const void* __restrict__ correction,
-                                                             int corr_dtype, int groups, int keep,
-                                                             int* __restrict__ experts, float* __restrict__ weights) {
+                                                             int corr_dtype, int groups, int keep, int softmax,
+                                                             int group_best, float renorm, int* __restrict__ experts,
+                                                             float* __restrict__ weights) {
   __shared__ float choice_s[kRouteSlots * kWave];
   __shared__ float group_s[kRouteSlots * kWave];
   const int t = blockIdx.x, lane = threadIdx.x;
   float s[kRouteSlots], c[kRouteSlots];
+  float mx = -INFINITY, sum = 0.f;
 #pragma unroll
   for (int i = 0; i < kRouteSlots; ++i) {
     const int e = lane + i * kWave;
-    s[i] = 0.f;
+    s[i] = e < E ? logits[static_cast<size_t>(t) * stride + e] : -INFINITY;
+    mx = fmaxf(mx, s[i]);
+  }
+  if (softmax) {
+    mx = wave_max(mx);
+#pragma unroll
+    for (int i = 0; i < kRouteSlots; ++i) {
+      s[i] = lane + i * kWave < E ? expf(s[i] - mx) : 0.f;
+      sum += s[i];
+    }
+    sum = wave_sum(sum);
+  }
+#pragma unroll
+  for (int i = 0; i < kRouteSlots; ++i) {
+    const int e = lane + i * kWave;
     c[i] = -INFINITY;
     if (e < E) {
-      s[i] = 1.f / (1.f + expf(-logits[static_cast<size_t>(t) * stride + e]));
+      s[i] = softmax ? s[i] / sum : 1.f / (1.f + expf(-s[i]));
       c[i] = correction != nullptr ? s[i] + load_f(correction, corr_dtype, e) : s[i];
       choice_s[e] = c[i];
+    } else {
+      s[i] = 0.f;
     }
   }
   if (groups > 1) {
@@ -99,7 +119,7 @@ __global__ __launch_bounds__(kWave) void route_choice_kernel(const float* __rest
           b = v;
         }
       }
-      group_s[g] = per > 1 ? a + b : a;
+      group_s[g] = per > 1 && group_best > 1 ? a + b : a;
     }
     __syncthreads();
     // the `keep` best groups, one after the other; lane 0 marks them by sign in LDS
@@ -107,7 +127,7 @@ __global__ __launch_bounds__(kWave) void route_choice_kernel(const float* __rest
       float best = -INFINITY;
       for (int g = lane; g < groups; g += kWave) best = fmaxf(best, group_s[g]);
       best = wave_max(best);
-      float mine = 1e9f;
+      float mine = static_cast<float>(groups - 1);
       for (int g = lane; g < groups; g += kWave)
         if (group_s[g] == best && static_cast<float>(g) < mine) mine = static_cast<float>(g);
       const int g_best = static_cast<int>(-wave_max(-mine));
@@ -121,6 +141,8 @@ __global__ __launch_bounds__(kWave) void route_choice_kernel(const float* __rest
       if (e < E && group_s[e / per] != -INFINITY) c[i] = -INFINITY;
     }
   }
+  __syncthreads();   // the choice scores in LDS have been read: the chosen scores take their place
+  float total = 0.f;
   for (int r = 0; r < top; ++r) {
     float best = -INFINITY;
 #pragma unroll
@@ -130,7 +152,8 @@ __global__ __launch_bounds__(kWave) void route_choice_kernel(const float* __rest
 #pragma unroll
     for (int i = kRouteSlots - 1; i >= 0; --i)
       if (c[i] == best && lane + i * kWave < E) mine = static_cast<float>(lane + i * kWave);
-    const int e = static_cast<int>(-wave_max(-mine));
+    const float first = -wave_max(-mine);
+    const int e = first < static_cast<float>(E) ? static_cast<int>(first) : E - 1;   // (logits that are no numbers: some expert)
     float w = 0.f;
 #pragma unroll
     for (int i = 0; i < kRouteSlots; ++i)
@@ -139,11 +162,15 @@ __global__ __launch_bounds__(kWave) void route_choice_kernel(const float* __rest
         w = s[i];
       }
     w = wave_sum(w);   // (one lane holds it, the others 0)
+    total += w;
     if (lane == 0) {
       experts[static_cast<size_t>(t) * top + r] = e;
-      weights[static_cast<size_t>(t) * top + r] = w * scale;
+      choice_s[r] = w;
     }
   }
+  __syncthreads();
+  const float by = renorm >= 0.f ? total + renorm : 1.f;
+  for (int r = lane; r < top; r += kWave) weights[static_cast<size_t>(t) * top + r] = choice_s[r] / by * scale;
 }
 
 // One workgroup.  plan: [0] number of tiles; [1 .. 1 + 2 * max_tiles): per tile its expert and its first row in the
@@ -204,8 +231,8 @@ __device__ __forceinline__ bf16x8 load8(const bf16* p) { return *reinterpret_cas
 template <typename T, bool GATED, int RT>
 __global__ __launch_bounds__(256) void expert_product_kernel(
     const T* __restrict__ a, int64_t a_stride, int a_by_token, int top, const T* __restrict__ w1, const T* __restrict__ w2,
-    int N, int K, const int* __restrict__ sorted, const int* __restrict__ plan, int act, void* __restrict__ out,
-    int64_t out_stride, int out_by_pair, int activate) {
+    int N, int K, const int* __restrict__ sorted, const int* __restrict__ plan, int act, float limit,
+    void* __restrict__ out, int64_t out_stride, int out_by_pair, int activate) {
   // activate (without a second weight): out[row] = act(a . w1[e]^T) in a's type instead of the 32-bit product
   const int tile = blockIdx.x;
   if (tile >= plan[0]) return;
@@ -286,7 +313,7 @@ __global__ __launch_bounds__(256) void expert_product_kernel(
         const int n = n0 + kq * 4 + i;
         if (n >= N) continue;
         if constexpr (GATED) {
-          const float v = gated_activation(act, to_float(float_to_bf16(accg[s][i]))) * to_float(float_to_bf16(accu[s][i]));
+          const float v = gated_product(act, limit, to_float(float_to_bf16(accg[s][i])), to_float(float_to_bf16(accu[s][i])));
           static_cast<bf16*>(out)[orow + n] = float_to_bf16(v);
         } else if (activate) {
           static_cast<bf16*>(out)[orow + n] = float_to_bf16(gated_activation(act, to_float(float_to_bf16(accg[s][i]))));
@@ -309,7 +336,7 @@ __global__ __launch_bounds__(256) void expert_product_kernel(
       if constexpr (GATED) {
         const T* u = w2 + (static_cast<size_t>(e) * N + n) * K;
         for (int k = 0; k < K; ++k) su = fmaf(to_float(arow[k]), to_float(u[k]), su);
-        static_cast<float*>(out)[orow + n] = gated_activation_exact(act, sg) * su;
+        static_cast<float*>(out)[orow + n] = gated_product_exact(act, limit, sg, su);
       } else {
         static_cast<float*>(out)[orow + n] = activate ? gated_activation_exact(act, sg) : sg;
       }
@@ -326,7 +353,7 @@ constexpr int kChunkK = 64;
 template <bool GATED>
 __global__ __launch_bounds__(256) void expert_product_rows64_kernel(
     const bf16* __restrict__ a, int64_t a_stride, int a_by_token, int top, const bf16* __restrict__ w1,
-    const bf16* __restrict__ w2, int N, int K, const int* __restrict__ sorted, const int* __restrict__ plan, int act,
+    const bf16* __restrict__ w2, int N, int K, const int* __restrict__ sorted, const int* __restrict__ plan, int act, float limit,
     void* __restrict__ out, int64_t out_stride, int out_by_pair, int activate) {
   __shared__ bf16x8 rows_lds[4][kChunkK / 32][kWave];   // [sub-tile of 16 rows][k tile of the chunk][lane]
   __shared__ int pair_of[kTileRowsMax];
@@ -420,7 +447,7 @@ __global__ __launch_bounds__(256) void expert_product_rows64_kernel(
         const int n = n0 + j * 16 + kq * 4 + i;
         if (n >= N) continue;
         if constexpr (GATED) {
-          const float v = gated_activation(act, to_float(float_to_bf16(accg[s][j][i]))) * to_float(float_to_bf16(accu[s][j][i]));
+          const float v = gated_product(act, limit, to_float(float_to_bf16(accg[s][j][i])), to_float(float_to_bf16(accu[s][j][i])));
           static_cast<bf16*>(out)[orow + n] = float_to_bf16(v);
         } else if (activate) {
           static_cast<bf16*>(out)[orow + n] =
@@ -464,19 +491,20 @@ extern "C" int sa_route(const float* logits, int64_t stride, int T, int E, int t
 }
 
 extern "C" int sa_route_choice(const float* logits, int64_t stride, int T, int E, int top, float scale,
-                               const void* correction, int corr_dtype, int groups, int keep, int* experts,
-                               float* weights, hipStream_t stream) {
+                               const void* correction, int corr_dtype, int groups, int keep, int softmax,
+                               int group_best, float renorm, int* experts, float* weights, hipStream_t stream) {
   if (T == 0) return 0;
   SA_REQUIRE(T > 0 && E > 0 && E <= kRouteSlots * kWave && top > 0 && stride >= E,
              "route_choice: bad sizes T=%d E=%d top=%d (at most %d experts)", T, E, top, kRouteSlots * kWave);
   SA_REQUIRE(groups >= 1 && E % groups == 0 && keep >= 1 && keep <= groups,
              "route_choice: %d experts in %d groups of which %d stay", E, groups, keep);
+  SA_REQUIRE(group_best == 1 || group_best == 2, "route_choice: a group's score is its largest or its two largest");
   SA_REQUIRE(top <= keep * (E / groups), "route_choice: %d experts cannot be chosen from %d groups of %d", top, keep,
              E / groups);
   SA_REQUIRE(correction == nullptr || corr_dtype == kF32 || corr_dtype == kBF16, "route_choice: unknown dtype %d",
              corr_dtype);
   route_choice_kernel<<<T, kWave, 0, stream>>>(logits, stride, E, top, scale, correction, corr_dtype, groups, keep,
-                                               experts, weights);
+                                               softmax, group_best, renorm, experts, weights);
   return check_launch("route_choice");
 }
 
@@ -499,7 +527,7 @@ extern "C" int sa_expert_sort(const int* experts, int P, int E, int tile_rows, i
 
 extern "C" int sa_expert_product(const void* a, int dtype, int64_t a_stride, int a_by_token, int top, const void* w1,
                                  const void* w2, int N, int K, const int* sorted, const int* plan, int P, int E,
-                                 int tile_rows, int act, void* out, int64_t out_stride, int out_by_pair, int activate,
+                                 int tile_rows, int act, float limit, void* out, int64_t out_stride, int out_by_pair, int activate,
                                  hipStream_t stream) {
   if (P == 0) return 0;
   SA_REQUIRE(!activate || w2 == nullptr, "expert_product: a gated product has its activation already");
@@ -507,7 +535,8 @@ extern "C" int sa_expert_product(const void* a, int dtype, int64_t a_stride, int
              "expert_product: bad sizes P=%d E=%d N=%d K=%d", P, E, N, K);
   SA_REQUIRE(a != nullptr && w1 != nullptr && sorted != nullptr && plan != nullptr && out != nullptr,
              "expert_product: a null pointer");
-  SA_REQUIRE(act >= 0 && act < kNumActivations, "expert_product: unknown activation %d", act);
+  SA_REQUIRE(act >= 0 && act < (w2 != nullptr ? kNumGatedRules : kNumActivations), "expert_product: unknown activation %d", act);
+  SA_REQUIRE(act != kActClampedGlu || limit > 0.f, "expert_product: the clamped gated product needs a positive limit");
   SA_REQUIRE(dtype == kF32 || dtype == kBF16, "expert_product: unknown dtype %d", dtype);
   SA_REQUIRE(tile_rows == 16 || tile_rows == kTileRowsMax, "expert_product: tiles of 16 or %d rows", kTileRowsMax);
   const dim3 grid(sa_expert_tiles_max(P, E, tile_rows), (N + 63) / 64);
@@ -516,7 +545,7 @@ extern "C" int sa_expert_product(const void* a, int dtype, int64_t a_stride, int
 #define SA_EXPERT(T, G, RT)                                                                                            \
   expert_product_kernel<T, G, RT><<<grid, 256, 0, stream>>>(static_cast<const T*>(a), a_stride, a_by_token, top,        \
                                                              static_cast<const T*>(w1), static_cast<const T*>(w2), N,  \
-                                                             K, sorted, plan, act, out, out_stride, out_by_pair,       \
+                                                             K, sorted, plan, act, limit, out, out_stride, out_by_pair, \
                                                              activate)
   if (dtype == kBF16) {
     if (tile_rows == 16) {
@@ -527,11 +556,11 @@ extern "C" int sa_expert_product(const void* a, int dtype, int64_t a_stride, int
       if (gated)
         expert_product_rows64_kernel<true><<<wide, 256, 0, stream>>>(
             static_cast<const bf16*>(a), a_stride, a_by_token, top, static_cast<const bf16*>(w1),
-            static_cast<const bf16*>(w2), N, K, sorted, plan, act, out, out_stride, out_by_pair, 0);
+            static_cast<const bf16*>(w2), N, K, sorted, plan, act, limit, out, out_stride, out_by_pair, 0);
       else
         expert_product_rows64_kernel<false><<<wide, 256, 0, stream>>>(
             static_cast<const bf16*>(a), a_stride, a_by_token, top, static_cast<const bf16*>(w1), nullptr, N, K, sorted,
-            plan, act, out, out_stride, out_by_pair, activate);
+            plan, act, limit, out, out_stride, out_by_pair, activate);
     }
   } else {
     if (gated) SA_EXPERT(float, true, 1);

@@ -44,8 +44,9 @@ static int gemm_routed(const void* A, int a_dtype, int64_t lda, const void* W, c
   int act = epilogue_activation(epilogue);
   epilogue = epilogue_kind(epilogue);
   SA_REQUIRE(epilogue >= 0 && epilogue <= 3, "gemm: unknown epilogue %d", epilogue);
-  SA_REQUIRE(act >= 0 && act < kNumActivations && (epilogue == 1 || epilogue == 3 || act == 0),
+  SA_REQUIRE(act >= 0 && act < (epilogue == 1 ? kNumGatedRules : kNumActivations) && (epilogue == 1 || epilogue == 3 || act == 0),
              "gemm: unknown activation %d", act);
+  SA_REQUIRE(act != kActClampedGlu || cap > 0.f, "gemm: the clamped gated product needs a positive limit");
   // an activation without a gate: the product as without an epilogue, the activation in the wide kernel's epilogue
   // or, behind every other kernel, by a kernel of its own
   const int activated = epilogue == kEpilogueActivated ? act + 1 : 0;
@@ -92,7 +93,7 @@ static int gemm_routed(const void* A, int a_dtype, int64_t lda, const void* W, c
   }
   // (a shape given by the caller for the wide kernel may carry a cut of K in front: cuts * 10000000 + shape)
   if (kernel == 4)
-    return gemm_wide(A, lda, W, C, ldc, M, N, K, epilogue, activated ? activated : act, algo == 4 ? shape % 10000000 : 0,
+    return gemm_wide(A, lda, W, C, ldc, M, N, K, epilogue, activated ? activated : act, cap, algo == 4 ? shape % 10000000 : 0,
                      algo == 4 ? shape / 10000000 : 1, workspace, ws_bytes, stream, planes_left);
   // (the few-rows kernel has the activation in its epilogue too, for bfloat16 results)
   if (kernel == 2 && activated && c_dtype == kBF16)

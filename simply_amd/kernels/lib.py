@@ -58,7 +58,7 @@ _SIGNATURES = {
     "sa_paged_attention_sink": [_P, _I, _L, _P, _P, _P, _I, _P, _P, _P, _L, _I, _I, _I, _I, _I, _I, _I, _F, _F, _P, _I, _P,
                                 _P],
     "sa_residual_add_norm": [_P, _I, _L, _P, _I, _F, _I, _F, _P, _P, _I, _I, _I, _P],
-    "sa_gated_heads": [_P, _I, _L, _P, _I, _L, _P, _I, _F, _I, _P, _I, _L, _I, _I, _I, _I, _P],
+    "sa_gated_heads": [_P, _I, _L, _P, _I, _L, _P, _I, _F, _I, _P, _I, _L, _I, _I, _I, _I, _I, _P],
     "sa_activation": [_P, _I, _L, _I, _I, _I, _P],
     "sa_qk_norm_rope_cache_write": [_P, _I, _L, _P, _P, _I, _F, _F, _P, _L, _P, _I, _P, _P, _P, _I, _I, _I, _I, _I, _I, _P],
     "sa_paged_attention_decode_sink": [_P, _L, _P, _P, _P, _I, _P, _I, _I, _P, _L, _I, _I, _I, _I, _I, _F, _I, _I, _I, _P,
@@ -73,9 +73,9 @@ _SIGNATURES = {
     "sa_paged_attention_maps_units_takes": [_I, _I, _I, _I, _I, _I, _L, _P],
     "sa_paged_attention_maps_units": [_P, _L, _P, _P, _P, _I, _P, _I, _I, _P, _L, _I, _I, _I, _I, _I, _I, _F, _I, _I, _F,
                                       _F, _F, _I, _I, _P, _L, _P],
-    "sa_residual_add_next_norm": [_P, _I, _L, _F, _P, _P, _I, _F, _I, _P, _I, _I, _I, _P],
+    "sa_residual_add_next_norm": [_P, _I, _L, _F, _P, _P, _P, _I, _F, _I, _P, _I, _I, _I, _P],
     "sa_short_conv": [_P, _I, _L, _P, _P, _I, _I, _P, _I, _I, _P, _L, _P, _I, _I, _P, _I, _I, _P],
-    "sa_head_product": [_P, _I, _L, _L, _P, _I, _P, _I, _L, _L, _I, _I, _I, _I, _I, _P, _I, _L, _P],
+    "sa_head_product": [_P, _I, _L, _L, _P, _I, _P, _I, _L, _L, _I, _I, _I, _I, _I, _P, _I, _L, _I, _P],
     "sa_rglru_scan": [_P, _P, _I, _P, _P, _P, _I, _F, _P, _I, _L, _P, _P, _L, _P, _I, _I, _P, _L, _P, _I, _I, _P],
     "sa_short_conv_silu": [_P, _I, _L, _P, _I, _I, _P, _L, _P, _I, _I, _P, _I, _I, _P],
     "sa_delta_inputs_few": [_P, _I, _L, _P, _I, _I, _P, _L, _P, _I, _I, _P, _I, _I, _I, _P, _I, _L, _P, _P, _I, _I, _P, _P],
@@ -87,12 +87,15 @@ _SIGNATURES = {
     "sa_bias_add": [_P, _I, _L, _P, _I, _I, _I, _P],
     "sa_weighted_sum": [_P, _L, _F, _P, _L, _F, _I, _P, _L, _I, _I, _P],
     "sa_exp_gates": [_P, _L, _P, _I, _F, _I, _P, _L, _P, _I, _P, _P],
-    "sa_linear_state": [_P, _I, _L, _I, _I, _I, _F, _P, _L, _P, _I, _F, _I, _I, _I, _I, _I, _P, _L, _P, _I, _P, _P],
+    "sa_linear_state": [_P, _I, _L, _I, _I, _I, _F, _P, _L, _P, _I, _F, _I, _P, _I, _I, _I, _I, _I, _P, _L, _P, _I, _P, _P],
     "sa_normalized_readout": [_P, _P, _L, _P, _I, _L, _P, _I, _F, _P, _I, _L, _I, _I, _I, _P],
     "sa_route": [_P, _L, _I, _I, _I, _F, _P, _P, _P],
     "sa_expert_sort": [_P, _I, _I, _I, _P, _P, _I, _P],
-    "sa_expert_product": [_P, _I, _L, _I, _I, _P, _P, _I, _I, _P, _P, _I, _I, _I, _I, _P, _L, _I, _I, _P],
-    "sa_route_choice": [_P, _L, _I, _I, _I, _F, _P, _I, _I, _I, _P, _P, _P],
+    "sa_expert_product": [_P, _I, _L, _I, _I, _P, _P, _I, _I, _P, _P, _I, _I, _I, _I, _F, _P, _L, _I, _I, _P],
+    "sa_route_choice": [_P, _L, _I, _I, _I, _F, _P, _I, _I, _I, _I, _I, _F, _P, _P, _P],
+    "sa_token_shift": [_P, _I, _L, _P, _I, _I, _P, _L, _P, _I, _I, _P, _I, _P],
+    "sa_low_rank_decay": [_P, _I, _L, _P, _I, _P, _I, _P, _I, _I, _I, _P],
+    "sa_concat_rows": [_P, _P, _P, _I, _I, _I, _I, _P],
     "sa_attention_inputs": [_P, _I, _L, _I, _I, _I, _I, _I, _I, _I, _P, _I, _I, _P, _L, _I, _P, _P, _I, _F, _P, _I, _F, _I,
                             _F, _P, _I, _I, _P, _P, _L, _P, _P, _I, _P, _P, _I, _P],
     "sa_expert_combine": [_P, _P, _I, _P, _I, _L, _P, _L, _P, _I, _L, _I, _I, _P],

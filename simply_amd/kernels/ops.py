@@ -376,12 +376,21 @@ def decode_slots(positions: torch.Tensor, token_seq: torch.Tensor, block_table: 
 EPILOGUE_NONE, EPILOGUE_GATED, EPILOGUE_SOFT_CAP, EPILOGUE_ACTIVATED = 0, 1, 2, 3
 #: activations of the gated epilogue (simply_amd/csrc/activations.h); the epilogue argument is 1 + 16 * activation
 ACT_GELU_TANH, ACT_SILU, ACT_SQUARED_RELU, ACT_GELU_ERF = 0, 1, 2, 3
+#: a rule of the gated epilogue alone: min(g, limit) sigmoid(1.702 min(g, limit)) (clamp(u, -limit, limit) + 1)
+ACT_CLAMPED_GLU = 4
 
 
 def _gated(activation: int) -> int:
-    if activation not in (ACT_GELU_TANH, ACT_SILU, ACT_SQUARED_RELU, ACT_GELU_ERF):
+    if activation not in (ACT_GELU_TANH, ACT_SILU, ACT_SQUARED_RELU, ACT_GELU_ERF, ACT_CLAMPED_GLU):
         raise KernelError(f"unknown activation code {activation!r}")
     return EPILOGUE_GATED + 16 * activation
+
+
+def _gate_limit(activation: int, limit: float | None) -> float:
+    """The limit of a gated product's clamped rule, which travels where a soft-cap's cap does (0 without one)."""
+    if (activation == ACT_CLAMPED_GLU) != (limit is not None) or (limit is not None and not limit > 0):
+        raise KernelError("a limit (positive) goes with the clamped gated product and with it alone")
+    return float(limit or 0.0)
 
 
 #: scratch memory for partial results (attention over key ranges, products with K cut over workgroups), one per
@@ -410,9 +419,9 @@ def workspace_uses(device) -> int:
 def gemm(a: torch.Tensor, w: "torch.Tensor | TiledWeight", *, w2: "torch.Tensor | TiledWeight | None" = None,
          soft_cap: float | None = None, out_dtype: torch.dtype | None = None, out: torch.Tensor | None = None,
          algo: int = ALGO_AUTO, shape: int = 0, activation: int = ACT_GELU_TANH,
-         defer_sum: bool = False, activate: int | None = None) -> "torch.Tensor | PartialSums":
+         defer_sum: bool = False, activate: int | None = None, limit: float | None = None) -> "torch.Tensor | PartialSums":
     """a[M, K] . w[N, K]^T.  With w2 (row-major weights) or a paired `TiledWeight`: act(a.wg^T) * (a.wu^T) with
-    the activation of that code.  With soft_cap: cap * tanh(. / cap).  With activate (an activation code): act(a.w^T),
+    the activation of that code (ACT_CLAMPED_GLU: the rule with the limit `limit`).  With soft_cap: cap * tanh(. / cap).  With activate (an activation code): act(a.w^T),
     the product rounded to the output type first.  w is a row-major tensor or a `TiledWeight`.
     defer_sum: where the product is computed in cuts of K, leave their sum to the caller: the result is then a
     `PartialSums` (else the tensor as always)."""
@@ -436,17 +445,17 @@ def gemm(a: torch.Tensor, w: "torch.Tensor | TiledWeight", *, w2: "torch.Tensor 
         raise KernelError(f"gemm: a is {a.dtype} but the weight is {wd.dtype}")
     epi, cap = EPILOGUE_NONE, 0.0
     if paired:
-        epi = _gated(activation)
+        epi, cap = _gated(activation), _gate_limit(activation, limit)
     elif w2 is not None:
         if soft_cap:
             raise KernelError("gemm: the gated and the soft-cap epilogue do not combine")
         if tuple(w2.shape) != tuple(w.shape) or w2d.dtype != wd.dtype or not w2d.is_contiguous():
             raise KernelError("gemm: the second weight must match the first")
-        epi = _gated(activation)
+        epi, cap = _gated(activation), _gate_limit(activation, limit)
     elif soft_cap:
         epi, cap = EPILOGUE_SOFT_CAP, float(soft_cap)
     if activate is not None:
-        if epi != EPILOGUE_NONE or defer_sum:
+        if epi != EPILOGUE_NONE or defer_sum or activate == ACT_CLAMPED_GLU:
             raise KernelError("gemm: an activation of the product combines with no other epilogue and no deferred sum")
         epi = _gated(activate) - EPILOGUE_GATED + EPILOGUE_ACTIVATED
     if out is None:
@@ -465,6 +474,36 @@ def gemm(a: torch.Tensor, w: "torch.Tensor | TiledWeight", *, w2: "torch.Tensor 
         return out
     _lib.call("sa_gemm", _ptr(a), _code(a), lda, _ptr(wd), _ptr(w2d), _code(wd), _ptr(out), _code(out), ldc, M, N, K, epi,
               cap, algo, int(packed), int(shape), _ptr(ws), ws.numel(), _stream())
+    return out
+
+
+class SectionedWeight:
+    """Weights [N, K] of several products that are run as one: section s of the result, columns s N .. (s + 1) N, is
+    section s of the input rows, columns s K .. (s + 1) K, times the s-th weight."""
+
+    def __init__(self, parts: list, rows: int, cols: int):
+        self.parts, self.rows, self.cols = parts, rows, cols   # (parts: one product weight per section)
+
+    @classmethod
+    def of(cls, ws) -> "SectionedWeight":
+        from .packing import pack_tiles
+
+        ws = list(ws)
+        N, K = ws[0].shape
+        if any(tuple(w.shape) != (N, K) or w.dtype != ws[0].dtype for w in ws):
+            raise KernelError("SectionedWeight: the sections' weights differ in shape or type")
+        tiled = ws[0].dtype == torch.bfloat16 and ws[0].is_cuda
+        return cls([pack_tiles(w.contiguous()) if tiled else w.contiguous() for w in ws], N, K)
+
+
+def gemm_sections(a: torch.Tensor, w: SectionedWeight) -> torch.Tensor:
+    """[T, S * N] from rows a [T, S * K] (a view is fine): every section's columns times its own weight."""
+    S, N, K = len(w.parts), w.rows, w.cols
+    if a.dim() != 2 or a.shape[1] != S * K:
+        raise KernelError(f"gemm_sections: rows {tuple(a.shape)} for {S} sections of {K}")
+    out = torch.empty((a.shape[0], S * N), dtype=a.dtype, device=a.device)
+    for s, part in enumerate(w.parts):
+        gemm(a[:, s * K:(s + 1) * K], part, out=out[:, s * N:(s + 1) * N])
     return out
 
 
@@ -509,7 +548,7 @@ def gemm_normed(y: torch.Tensor | None, h_in: torch.Tensor, h_out: torch.Tensor 
                 post_weight: torch.Tensor | None, post_eps: float, post_plus_one: bool, next_weight: torch.Tensor,
                 next_eps: float, next_plus_one: bool, soft_cap: float | None = None,
                 out_dtype: torch.dtype = torch.bfloat16, out: torch.Tensor | None = None,
-                activation: int = ACT_GELU_TANH) -> torch.Tensor:
+                activation: int = ACT_GELU_TANH, limit: float | None = None) -> torch.Tensor:
     """h_out = h_in + norm(y; post) (y None: the residual stays h_in); returns epilogue(norm(h_out; next) . w^T),
     in one kernel, for up to 16 rows.  The residual buffers are float32 [M, K] and must differ."""
     _dev(y, h_in, h_out, post_weight, next_weight, w.data)
@@ -527,7 +566,7 @@ def gemm_normed(y: torch.Tensor | None, h_in: torch.Tensor, h_out: torch.Tensor 
             raise KernelError("gemm_normed: a norm weight does not match the width")
     epi, cap = EPILOGUE_NONE, 0.0
     if w.paired:
-        epi = _gated(activation)
+        epi, cap = _gated(activation), _gate_limit(activation, limit)
     elif soft_cap:
         epi, cap = EPILOGUE_SOFT_CAP, float(soft_cap)
     if out is None:
@@ -880,14 +919,17 @@ def residual_add_norm(y: "torch.Tensor | PartialSums | None", residual: torch.Te
 
 
 def residual_add_next_norm(y: "torch.Tensor | PartialSums | None", residual: torch.Tensor, weight: torch.Tensor, *,
-                           eps: float, plus_one: bool = False, mult: float = 1.0,
+                           eps: float, plus_one: bool = False, mult: float = 1.0, bias: torch.Tensor | None = None,
                            out_dtype: torch.dtype | None = None) -> torch.Tensor:
-    """residual += mult * y (y None: nothing is added); returns residual / sqrt(mean(residual^2) + eps) * (weight +
-    plus_one) in out_dtype: one pass over the rows."""
+    """residual += mult * y (y None: nothing is added; a y whose rows are one row expanded adds that row to all);
+    returns residual / sqrt(mean(residual^2) + eps) * (weight + plus_one) in out_dtype, or with a bias the layer norm
+    (residual - mean) / sqrt(variance + eps) * (weight + plus_one) + bias: one pass over the rows."""
     if isinstance(y, PartialSums):
         y = y.materialize()
-    _dev(y, residual, weight)
+    _dev(y, residual, weight, bias)
     T, D = residual.shape
+    if bias is not None and (bias.numel() != D or not bias.is_contiguous() or bias.dtype != weight.dtype or D > 8192):
+        raise KernelError("residual_add_next_norm: a layer norm's bias matches its weight (rows of at most 8192)")
     if residual.dtype != torch.float32 or not residual.is_contiguous():
         raise KernelError("residual_add_next_norm: the residual stream must be contiguous float32")
     if weight.numel() != D or not weight.is_contiguous():
@@ -902,7 +944,7 @@ def residual_add_next_norm(y: "torch.Tensor | PartialSums | None", residual: tor
         return rmsnorm(residual, weight, eps, plus_one, out_dtype or (y.dtype if y is not None else torch.float32))
     out = torch.empty((T, D), dtype=out_dtype or (y.dtype if y is not None else torch.float32), device=residual.device)
     _lib.call("sa_residual_add_next_norm", _ptr(y), _code(y) if y is not None else 0, ys, float(mult), _ptr(residual),
-              _ptr(weight), _code(weight), float(eps), int(plus_one), _ptr(out), _code(out), T, D, _stream())
+              _ptr(weight), _ptr(bias), _code(weight), float(eps), int(plus_one), _ptr(out), _code(out), T, D, _stream())
     return out
 
 
@@ -912,8 +954,8 @@ GATE_SIGMOID, GATE_SILU = 0, 1
 def gated_heads(x: torch.Tensor, gate: torch.Tensor, num_heads: int, size: int, *, kind: int,
                 weight: torch.Tensor | None = None, eps: float = 0.0, out_dtype: torch.dtype | None = None,
                 out: torch.Tensor | None = None, per_head: bool = False) -> torch.Tensor:
-    """out[t, h] = (x[t, h] normed over the head's `size` entries and times weight [size], if a weight is given,
-    else x[t, h]) * sigmoid(gate[t, h]) or * silu(gate[t, h]).  x, gate: rows of num_heads * size (views with a
+    """out[t, h] = (x[t, h] normed over the head's `size` entries and times weight [size] (shared by the heads) or
+    [num_heads * size] (entry by entry), if a weight is given, else x[t, h]) * sigmoid(gate[t, h]) or * silu(gate[t, h]).  x, gate: rows of num_heads * size (views with a
     row stride are fine); per_head: gate rows of num_heads, one number for all entries of a head."""
     _dev(x, gate, weight, out)
     T = x.shape[0]
@@ -921,8 +963,8 @@ def gated_heads(x: torch.Tensor, gate: torch.Tensor, num_heads: int, size: int, 
     xs, gs = _rows(x, "gated_heads: x"), _rows(gate, "gated_heads: gate")
     if x.shape[1] != width or tuple(gate.shape) != (T, num_heads if per_head else width):
         raise KernelError(f"gated_heads: rows of {width} expected, got x {tuple(x.shape)} gate {tuple(gate.shape)}")
-    if weight is not None and (weight.numel() != size or not weight.is_contiguous()):
-        raise KernelError("gated_heads: the norm weight has one entry per element of a head")
+    if weight is not None and (weight.numel() not in (size, width) or not weight.is_contiguous()):
+        raise KernelError("gated_heads: the norm weight has one entry per element of a head or of the row")
     if kind not in (GATE_SIGMOID, GATE_SILU):
         raise KernelError(f"gated_heads: unknown gate {kind!r}")
     if out is None:
@@ -932,7 +974,7 @@ def gated_heads(x: torch.Tensor, gate: torch.Tensor, num_heads: int, size: int, 
     os_ = _rows(out, "gated_heads: out")
     _lib.call("sa_gated_heads", _ptr(x), _code(x), xs, _ptr(gate), _code(gate), gs, _ptr(weight),
               _code(weight) if weight is not None else 0, float(eps), int(kind), _ptr(out), _code(out), os_, T,
-              num_heads, size, int(bool(per_head)), _stream())
+              num_heads, size, int(bool(per_head)), int(weight is not None and weight.numel() != size), _stream())
     return out
 
 
@@ -1155,7 +1197,8 @@ def head_product(x: torch.Tensor, w: torch.Tensor, *, in_stride: int | None = No
                  gate: torch.Tensor | None = None, out_dtype: torch.dtype | None = None) -> torch.Tensor:
     """A product per head: out[t, h, :O] = w[h] x[t, h, :I] with w [H, O, I], summed in 32-bit.  x rows hold the
     heads `in_stride` entries apart (default I + tail).  tail: the entries behind a head's inputs are copied behind its
-    outputs.  gate [T, H] (a view is fine): the outputs are multiplied by sigmoid(gate).  Returns [T, H * (O + tail)]."""
+    outputs.  gate (a view is fine): [T, H], one number per head, or [T, H * O], one per output; the outputs are
+    multiplied by sigmoid(gate).  Returns [T, H * (O + tail)]."""
     _dev(x, w, gate)
     xs = _rows(x, "head_product: x")
     T = x.shape[0]
@@ -1168,11 +1211,12 @@ def head_product(x: torch.Tensor, w: torch.Tensor, *, in_stride: int | None = No
     gs = 0
     if gate is not None:
         gs = _rows(gate, "head_product: gate")
-        if gate.shape[0] != T or gate.shape[1] != H:
-            raise KernelError(f"head_product: gates {tuple(gate.shape)} are not [T, H]")
+        if gate.shape[0] != T or gate.shape[1] not in (H, H * O):
+            raise KernelError(f"head_product: gates {tuple(gate.shape)} are neither [T, H] nor [T, H * O]")
     out = torch.empty((T, H * (O + tail)), dtype=out_dtype or x.dtype, device=x.device)
     _lib.call("sa_head_product", _ptr(x), _code(x), xs, hs, _ptr(w), _code(w), _ptr(out), _code(out), out.stride(0),
-              O + tail, T, H, I, O, int(tail), _ptr(gate), _code(gate) if gate is not None else 0, gs, _stream())
+              O + tail, T, H, I, O, int(tail), _ptr(gate), _code(gate) if gate is not None else 0, gs,
+              int(gate is not None and gate.shape[1] != H), _stream())
     return out
 
 
@@ -1511,11 +1555,13 @@ def exp_gates(raw: torch.Tensor, bias: torch.Tensor | None, cap: float, num_head
 
 def linear_state(proj: torch.Tensor, q_at: int, k_at: int, v_at: int, q_mult: float, gates: torch.Tensor, scalar: bool,
                  num_heads: int, key_dim: int, value_dim: int, ones: bool, state: torch.Tensor, seq_meta: torch.Tensor,
-                 num_seqs: int, *, decay_bias: torch.Tensor | None = None, tau: float | None = None) -> torch.Tensor:
+                 num_seqs: int, *, decay_bias: torch.Tensor | None = None, tau: float | None = None,
+                 bonus: torch.Tensor | None = None) -> torch.Tensor:
     """S <- diag(a) S + c k v^T, o = S^T (q * q_mult) along each request's tokens, from and into state float32 [slots,
     >= H * dk * (dv + ones)] (per head [dv + ones][dk]).  q, k, v: columns q_at, k_at, v_at of proj's rows, H heads
     each.  scalar: gates float32 [T, >= 2 H] hold a and c per head; else [T, H * dk] hold a per key channel, c = 1;
     with `tau` these hold z instead, and a = sigmoid(z + decay_bias)^(1 / tau) (decay_bias [H * dk] or None).
+    bonus [H * dk] (decays per key channel): o = (S_before + diag(bonus) k v^T)^T q, the state before the token.
     ones: one more column whose value is always 1 (a normalizer).  Returns float32 [T, H * (dv + ones)]."""
     _dev(proj, gates, state, seq_meta)
     T = proj.shape[0]
@@ -1529,11 +1575,14 @@ def linear_state(proj: torch.Tensor, q_at: int, k_at: int, v_at: int, q_mult: fl
         raise KernelError("linear_state: tau (positive) and a bias belong to decays per channel")
     if decay_bias is not None and (decay_bias.numel() != H * dk or not decay_bias.is_contiguous()):
         raise KernelError("linear_state: one bias per key channel")
-    _dev(decay_bias)
+    if bonus is not None and (scalar or bonus.numel() != H * dk or not bonus.is_contiguous()):
+        raise KernelError("linear_state: a bonus has one entry per head and key channel and goes with decays per channel")
+    _dev(decay_bias, bonus)
     out = torch.empty((T, H * CT), dtype=torch.float32, device=proj.device)
     _lib.call("sa_linear_state", _ptr(proj), _code(proj), _rows(proj, "linear_state: proj"), int(q_at), int(k_at), int(v_at),
               float(q_mult), _ptr(gates), _rows(gates, "linear_state: gates"), _ptr(decay_bias),
-              _code(decay_bias) if decay_bias is not None else 0, float(tau or 0.0), int(bool(scalar)), H, dk, dv,
+              _code(decay_bias) if decay_bias is not None else 0, float(tau or 0.0), int(bool(scalar)), _ptr(bonus),
+              _code(bonus) if bonus is not None else 0, H, dk, dv,
               int(bool(ones)), _ptr(state), state.stride(0), _ptr(seq_meta), int(num_seqs), _ptr(out), _stream())
     return out
 
@@ -1557,6 +1606,53 @@ def normalized_readout(x: torch.Tensor, floor: torch.Tensor, gate: torch.Tensor,
     return out
 
 
+# --------------------------------------------------------------------------- token shift, data-dependent decays, passes
+
+def token_shift(h: torch.Tensor, mu: torch.Tensor, tails: torch.Tensor, seq_meta: torch.Tensor, num_seqs: int,
+                max_q_len: int) -> torch.Tensor:
+    """[T, S * D] in h's type: stream s of token t is h[t] + (h[t - 1] - h[t]) * mu[s], mu [S, D].  A request's row before
+    its first one of the step is tails[slot] (float32 [slots, >= D], a view with a row stride), brought up to date."""
+    _dev(h, mu, tails, seq_meta)
+    stride = _rows(h, "token_shift: h")
+    T, D = h.shape
+    if mu.dim() != 2 or mu.shape[1] != D or not mu.is_contiguous():
+        raise KernelError(f"token_shift: mu {tuple(mu.shape)} for rows of {D}")
+    if tails.dtype != torch.float32 or tails.dim() != 2 or tails.stride(1) != 1 or tails.shape[1] < D:
+        raise KernelError("token_shift: tails must be float32 [slots, >= width]")
+    _seq_meta(seq_meta, num_seqs, "token_shift")
+    S = mu.shape[0]
+    out = torch.empty((T, S * D), dtype=h.dtype, device=h.device)
+    _lib.call("sa_token_shift", _ptr(h), _code(h), stride, _ptr(mu), _code(mu), S, _ptr(tails), tails.stride(0),
+              _ptr(seq_meta), int(num_seqs), int(max_q_len), _ptr(out), D, _stream())
+    return out
+
+
+def low_rank_decay(p: torch.Tensor, w: torch.Tensor, base: torch.Tensor) -> torch.Tensor:
+    """float32 [T, C]: exp(-exp(tanh(p) w + base)) with p [T, rank], w [rank, C], base [C]; all of it 32-bit."""
+    _dev(p, w, base)
+    stride = _rows(p, "low_rank_decay: p")
+    T, rank = p.shape
+    if w.dim() != 2 or w.shape[0] != rank or not w.is_contiguous() or base.numel() != w.shape[1] or not base.is_contiguous():
+        raise KernelError(f"low_rank_decay: w {tuple(w.shape)} and base {tuple(base.shape)} for {rank} factors")
+    C = w.shape[1]
+    out = torch.empty((T, C), dtype=torch.float32, device=p.device)
+    _lib.call("sa_low_rank_decay", _ptr(p), _code(p), stride, _ptr(w), _code(w), _ptr(base), _code(base), _ptr(out), T, C,
+              rank, _stream())
+    return out
+
+
+def concat_rows(x: torch.Tensor, y: torch.Tensor, out_dtype: torch.dtype) -> torch.Tensor:
+    """[x | y] row by row (contiguous float32) in out_dtype."""
+    _dev(x, y)
+    T = x.shape[0]
+    for t in (x, y):
+        if t.dtype != torch.float32 or t.dim() != 2 or not t.is_contiguous() or t.shape[0] != T:
+            raise KernelError("concat_rows: contiguous float32 rows expected")
+    out = torch.empty((T, x.shape[1] + y.shape[1]), dtype=out_dtype, device=x.device)
+    _lib.call("sa_concat_rows", _ptr(x), _ptr(y), _ptr(out), _code(out), T, x.shape[1], y.shape[1], _stream())
+    return out
+
+
 # --------------------------------------------------------------------------- routed experts
 
 def route(logits: torch.Tensor, top: int, scale: float) -> tuple[torch.Tensor, torch.Tensor]:
@@ -1574,11 +1670,13 @@ def route(logits: torch.Tensor, top: int, scale: float) -> tuple[torch.Tensor, t
 
 
 def route_choice(logits: torch.Tensor, top: int, scale: float, *, correction: torch.Tensor | None = None,
-                 groups: int = 1, keep: int = 1) -> tuple[torch.Tensor, torch.Tensor]:
-    """Scores are sigmoids of the logits (float32 [T, E]); the `top` experts with the largest score + correction[e] are
-    chosen, among the `keep` groups (of `groups` equal groups of neighbouring experts) whose two largest choice scores
-    have the largest sums.  Returns (experts int32 [T, top], weights float32 [T, top] = score * scale, the score
-    without the correction), largest choice first."""
+                 groups: int = 1, keep: int = 1, softmax: bool = False, group_best: int = 2,
+                 renorm: float | None = None) -> tuple[torch.Tensor, torch.Tensor]:
+    """Scores are sigmoids of the logits (float32 [T, E]), or their softmax; the `top` experts with the largest score +
+    correction[e] are chosen, among the `keep` groups (of `groups` equal groups of neighbouring experts) with the
+    largest group scores: the sum of a group's two largest choice scores (group_best 2) or its largest (1).  Returns
+    (experts int32 [T, top], weights float32 [T, top] = score * scale, the score without the correction, divided by the
+    chosen scores' sum + renorm unless renorm is None), largest choice first."""
     _dev(logits, correction)
     T, E = logits.shape
     if logits.dtype != torch.float32:
@@ -1589,17 +1687,18 @@ def route_choice(logits: torch.Tensor, top: int, scale: float, *, correction: to
     weights = torch.empty((T, top), dtype=torch.float32, device=logits.device)
     _lib.call("sa_route_choice", _ptr(logits), _rows(logits, "route_choice: logits"), T, E, int(top), float(scale),
               _ptr(correction), _code(correction) if correction is not None else 0, int(groups), int(keep),
-              _ptr(experts), _ptr(weights), _stream())
+              int(bool(softmax)), int(group_best), -1.0 if renorm is None else float(renorm), _ptr(experts), _ptr(weights),
+              _stream())
     return experts, weights
 
 
 def routed_experts(x: torch.Tensor, experts: torch.Tensor, weights: torch.Tensor, gate_w, up_w, down_w, activation: int,
                    *, shared: torch.Tensor | None = None, shared_gate: torch.Tensor | None = None,
-                   out_dtype: torch.dtype | None = None) -> torch.Tensor:
+                   out_dtype: torch.dtype | None = None, limit: float | None = None) -> torch.Tensor:
     """sum_k weights[t, k] * down[e](act(gate[e] x) * (up[e] x)) with e = experts[t, k], plus sigmoid(shared_gate[t]) *
     shared[t] (shared None: nothing; shared_gate None: shared as it is).  gate_w, up_w, down_w: `packing.ExpertStack`s
     (every expert's matrix, tiled if bfloat16).  x [T, D] in the weights' type; shared_gate float32 [T, 1].
-    gate_w None: experts without a gate, down[e](act(up[e] x))."""
+    gate_w None: experts without a gate, down[e](act(up[e] x)).  limit: of the clamped gated rule (ACT_CLAMPED_GLU)."""
     _dev(x, experts, weights, gate_w.data if gate_w is not None else None, up_w.data, down_w.data, shared, shared_gate)
     T, D = x.shape
     top, E, F = experts.shape[1], up_w.experts, up_w.rows
@@ -1611,6 +1710,9 @@ def routed_experts(x: torch.Tensor, experts: torch.Tensor, weights: torch.Tensor
     if experts.dtype != torch.int32 or not experts.is_contiguous() or tuple(weights.shape) != (T, top) \
             or weights.dtype != torch.float32 or not weights.is_contiguous():
         raise KernelError("routed_experts: experts int32 [T, top] and weights float32 [T, top] expected")
+    if gate_w is None and activation == ACT_CLAMPED_GLU:
+        raise KernelError("routed_experts: the clamped rule joins two factors")
+    limit = _gate_limit(activation, limit)
     P = T * top
     dev = x.device
     # tiles of 64 rows share the weights' operands between four sub-tiles: for steps that bring an expert many rows
@@ -1622,11 +1724,11 @@ def routed_experts(x: torch.Tensor, experts: torch.Tensor, weights: torch.Tensor
     h = torch.empty((P, F), dtype=x.dtype, device=dev)
     first, second = (gate_w.data, up_w.data) if gate_w is not None else (up_w.data, None)
     _lib.call("sa_expert_product", _ptr(x), _code(x), _rows(x, "routed_experts: x"), 1, top, _ptr(first),
-              _ptr(second), F, D, _ptr(sorted_), _ptr(plan), P, E, tile_rows, int(activation), _ptr(h), F, 0,
+              _ptr(second), F, D, _ptr(sorted_), _ptr(plan), P, E, tile_rows, int(activation), limit, _ptr(h), F, 0,
               int(gate_w is None), _stream())
     y = torch.empty((P, D), dtype=torch.float32, device=dev)
     _lib.call("sa_expert_product", _ptr(h), _code(h), F, 0, top, _ptr(down_w.data), None, D, F, _ptr(sorted_), _ptr(plan), P,
-              E, tile_rows, 0, _ptr(y), D, 1, 0, _stream())
+              E, tile_rows, 0, 0.0, _ptr(y), D, 1, 0, _stream())
     out = torch.empty((T, D), dtype=out_dtype or x.dtype, device=dev)
     if shared is not None and tuple(shared.shape) != (T, D):
         raise KernelError("routed_experts: the shared expert's rows do not match")

@@ -15,7 +15,7 @@ from .. import parts as _parts  # noqa: F401  (registers the built-in parts)
 from ..config.spec import LayerSpec, ModelSpec, PartSpec
 from ..kernels import ops
 from ..parts.base import Block, ParamSpec, Part, PendingNorm
-from ..registry import BLOCKS, EMBEDDINGS, FEED_FORWARDS, HEADS, MIXERS, NORMS, STREAM_PARTS
+from ..registry import BLOCKS, EMBEDDINGS, FEED_FORWARDS, HEADS, MIXERS, NORMS, PASS_INPUTS, STREAM_PARTS
 from ..weights import binding
 
 
@@ -36,12 +36,15 @@ class DecoderModel:
         self.embedding = EMBEDDINGS.build(spec.embedding.kind, **spec.embedding.params)
         self.head = HEADS.build(spec.head.kind, **spec.head.params)
         self.final_norm = NORMS.build(spec.final_norm.kind, **spec.final_norm.params)
+        self.pass_input = None if spec.pass_input is None else PASS_INPUTS.build(spec.pass_input.kind, **spec.pass_input.params)
         self.layers: list[Block] = [_build_layer(ls) for ls in spec.layers]
         self.loaded = False
 
     # ------------------------------------------------------------------ tensors
     def _bindings(self) -> list[tuple[Part, PartSpec]]:
         out: list[tuple[Part, PartSpec]] = [(self.embedding, self.spec.embedding)]
+        if self.pass_input is not None:
+            out.append((self.pass_input, self.spec.pass_input))
         for block, ls in zip(self.layers, self.spec.layers):
             out.append((block.mixer, ls.mixer))
             if ls.feed_forward is not None:
@@ -123,8 +126,9 @@ class DecoderModel:
             h = self.embedding.forward(tokens, ctx, cache_views[len(schedule)] if own else None)
         else:
             h = self.embedding.forward(tokens)
-        # a pass of a loop that is given the input again adds the embedding's output to the stream
-        again = h.clone() if any(e.add_embedding for e in schedule) else None
+        # a pass of a loop that is given the input again adds the embedding's output to the stream, or begins with a
+        # part that reads both
+        again = h.clone() if any(e.add_embedding or e.begins_pass is not None for e in schedule) else None
         normed = None
         for i, entry in enumerate(schedule):
             block = self.layers[entry.layer]
@@ -133,8 +137,12 @@ class DecoderModel:
                     h = normed.settle()
                 ops.residual_add_norm(again, h)
                 normed = None
+            if entry.begins_pass is not None:
+                if isinstance(normed, PendingNorm):
+                    h = normed.settle()
+                h, normed = self.pass_input.forward(h, again, entry.begins_pass, ctx, block.first_norm())
             nxt = None
-            if i + 1 < len(schedule) and not schedule[i + 1].add_embedding:
+            if i + 1 < len(schedule) and not schedule[i + 1].add_embedding and schedule[i + 1].begins_pass is None:
                 nxt = self.layers[schedule[i + 1].layer].first_norm()
             h, normed = block.forward(h, ctx, cache_views[i], normed, nxt)
             if after_layer is not None:

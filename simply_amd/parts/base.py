@@ -9,10 +9,12 @@ feed-forwards take and return activations `[T, D]` in the activation dtype
 
 Parts, per kind, and what each must provide:
 
-* Norm:             forward(x, out_dtype) -> y;  add_into(residual, y, next_norm) (optional fusion)
+* Norm:             forward(x, out_dtype) -> y;  add_into(residual, y, next_norm) (optional fusion);
+                    after_sum(residual, y, mult, out_dtype) -> y if it sets `fuses_sum`
 * PositionEncoding: apply(x, positions, num_heads, head_dim, div); rotary_table() or None
 * Mixer:            cache_need(); forward(x, ctx, cache) -> y
 * FeedForward:      forward(x, ctx) -> y
+* PassInput:        forward(h, x0, number, ctx, next_norm) -> (h, next_norm(h) or None)
 * Block:            first_norm(); forward(h, ctx, cache, normed, next_norm) -> (h, normed_for_next)
 
 A mixer or feed-forward that sets `accepts_pending` may be handed a `PendingNorm` instead of x: the norm (and the
@@ -213,11 +215,12 @@ def pending_product(x: PendingNorm, run) -> torch.Tensor:
 
 
 def project(x, w, *, soft_cap: float | None = None, out_dtype: torch.dtype | None = None,
-            out: torch.Tensor | None = None, activation: int = 0, defer_sum: bool = False) -> torch.Tensor:
+            out: torch.Tensor | None = None, activation: int = 0, defer_sum: bool = False,
+            limit: float | None = None) -> torch.Tensor:
     """x . w^T (gated if w is a paired tiled weight) for activations x or a `PendingNorm`.  A pending norm is done
     inside the product's kernel when that kernel takes the sizes; otherwise it is materialized first.  `out`: where
     the result goes (a buffer of the caller's), else a new tensor.  `activation`: the gated product's (a code of
-    the ACTIVATIONS registry).  `defer_sum`: the result may be an `ops.PartialSums` (see `ops.gemm`)."""
+    the ACTIVATIONS registry), with `limit` where its rule has one.  `defer_sum`: the result may be an `ops.PartialSums` (see `ops.gemm`)."""
     import functools
 
     from ..kernels import ops
@@ -226,9 +229,9 @@ def project(x, w, *, soft_cap: float | None = None, out_dtype: torch.dtype | Non
         if pending_fits_product(x, w):
             return pending_product(x, functools.partial(ops.gemm_normed, w=w, soft_cap=soft_cap,
                                                         out_dtype=out_dtype or x.dtype, out=out,
-                                                        activation=activation))
+                                                        activation=activation, limit=limit))
         x = x.materialize()
-    return ops.gemm(x, w, soft_cap=soft_cap, out_dtype=out_dtype, out=out, activation=activation, defer_sum=defer_sum)
+    return ops.gemm(x, w, soft_cap=soft_cap, out_dtype=out_dtype, out=out, activation=activation, defer_sum=defer_sum, limit=limit)
 
 
 class Part:
@@ -244,6 +247,14 @@ class Part:
 
 
 class Norm(Part):
+    #: True if after_sum() exists: a residual sum and this norm of its result in one kernel
+    fuses_sum = False
+
+    def after_sum(self, residual: torch.Tensor, y: "torch.Tensor | None", mult: float,
+                  out_dtype: torch.dtype) -> torch.Tensor:
+        """residual += mult * y (y None: nothing is added; rows may be one row expanded); returns self(residual)."""
+        raise NotImplementedError
+
     def forward(self, x: torch.Tensor, out_dtype: torch.dtype) -> torch.Tensor:
         raise NotImplementedError
 
@@ -301,6 +312,16 @@ class StreamPart(Part):
     def forward(self, h: torch.Tensor, ctx: Any, x: "torch.Tensor | None" = None) -> None:
         """h: float32 [T, D] residual stream, updated in place.  x: the same stream in the activation type, if the
         caller has it already."""
+        raise NotImplementedError
+
+
+class PassInput(Part):
+    """What happens to the residual stream right before the first layer of every pass of a loop over layers."""
+
+    def forward(self, h: torch.Tensor, x0: torch.Tensor, number: int, ctx: Any,
+                next_norm: "Norm | None") -> "tuple[torch.Tensor, torch.Tensor | None]":
+        """h: float32 [T, D] residual stream; x0: the embedding's output [T, D] float32 (not to be written); number: of
+        the pass, from 0.  Returns (the new stream, next_norm of it or None without a norm)."""
         raise NotImplementedError
 
 

@@ -128,8 +128,8 @@ class PostNormBlock(Block):
 class PreNormBlock(Block):
     """h += mult * mixer(pre_mixer(h));  h += mult * ffn(pre_ffn(h)): the parts read normed input, what they return is
     added as it is, times a constant (`mult`, a residual multiplier).  A layer may have no feed-forward; then the
-    second step is left out.  Each sum runs in one kernel with the norm in front of the next part where that is an
-    RMSNorm."""
+    second step is left out.  Each sum runs in one kernel with the norm in front of the next part where that norm
+    has such a kernel (an RMSNorm, a layer norm)."""
 
     def __init__(self, mixer, feed_forward, norms, mult: float = 1.0):
         super().__init__(mixer, feed_forward, norms)
@@ -144,9 +144,8 @@ class PreNormBlock(Block):
 
     def _add(self, h, y, norm, dtype):
         """h += mult * y; returns norm(h), or None without a norm."""
-        if norm is not None and getattr(norm, "fusable_rms", False):
-            return ops.residual_add_next_norm(y, h, norm.scale, eps=norm.eps, plus_one=norm.scale_plus_one,
-                                              mult=self.mult, out_dtype=dtype)
+        if norm is not None and norm.fuses_sum:
+            return norm.after_sum(h, y, self.mult, dtype)
         ops.residual_add_norm(y, h, mult=self.mult)
         return norm.forward(h, dtype) if norm is not None else None
 

@@ -15,8 +15,11 @@ from .base import ParamSpec, Part, StateNeed, as_product_weight, project
 
 @EMBEDDINGS.register("scaled_embedding")
 class ScaledEmbedding(Part):
-    def __init__(self, vocab_size: int, dim: int, scale: float):
+    """The token's row times a constant (`round_scale`: the constant rounded to the table's type first)."""
+
+    def __init__(self, vocab_size: int, dim: int, scale: float, round_scale: bool = True):
         self.vocab_size, self.dim, self.scale = int(vocab_size), int(dim), float(scale)
+        self.round_scale = bool(round_scale)
         self.table: torch.Tensor | None = None
 
     def param_specs(self):
@@ -29,7 +32,7 @@ class ScaledEmbedding(Part):
     def forward(self, tokens: torch.Tensor) -> torch.Tensor:
         """tokens int32 [T] -> float32 residual stream [T, D]."""
         # the factor is rounded to the table's dtype (module.py:476-480), the product is kept in float32
-        scale = float(torch.tensor(self.scale, dtype=self.table.dtype))
+        scale = float(torch.tensor(self.scale, dtype=self.table.dtype)) if self.round_scale else self.scale
         return ops.embed(self.table, tokens, scale)
 
 

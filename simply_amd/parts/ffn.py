@@ -14,6 +14,16 @@ ACTIVATIONS.register("gelu_tanh", ops.ACT_GELU_TANH)
 ACTIVATIONS.register("silu", ops.ACT_SILU)
 ACTIVATIONS.register("squared_relu", ops.ACT_SQUARED_RELU)
 ACTIVATIONS.register("gelu_erf", ops.ACT_GELU_ERF)   # the exact GELU, x Phi(x)
+# a rule for the two factors of a gated feed-forward (both clamped to a limit), not an activation of one
+ACTIVATIONS.register("clamped_glu", ops.ACT_CLAMPED_GLU)
+
+
+def check_limit(activation: str, limit: float | None) -> float | None:
+    """The limit of the clamped gated rule: it comes with that rule and with no other activation."""
+    clamped = int(ACTIVATIONS.get(activation)) == ops.ACT_CLAMPED_GLU
+    if clamped != (limit is not None) or (limit is not None and not float(limit) > 0):
+        raise ValueError(f"activation {activation!r} with limit {limit!r}: a positive limit goes with 'clamped_glu' alone")
+    return None if limit is None else float(limit)
 
 
 @FEED_FORWARDS.register("dense")
@@ -26,6 +36,8 @@ class Dense(FeedForward):
         self.hidden_size, self.intermediate_size = int(hidden_size), int(intermediate_size)
         self.activation = activation
         self.activation_code = int(ACTIVATIONS.get(activation))
+        if self.activation_code == ops.ACT_CLAMPED_GLU:
+            raise ValueError(f"dense: {activation!r} joins two factors, and this feed-forward has one")
         self.up_proj = self.down_proj = None
 
     def param_specs(self):
@@ -43,13 +55,17 @@ class Dense(FeedForward):
 
 @FEED_FORWARDS.register("gated_dense")
 class GatedDense(FeedForward):
+    """With activation 'clamped_glu' and its `limit` the two factors g = gate(x), u = up(x) are joined as
+    g' sigmoid(1.702 g') (u' + 1) with g' = min(g, limit), u' = clamp(u, -limit, limit)."""
+
     accepts_pending = True
     defers_sum = True
 
-    def __init__(self, hidden_size: int, intermediate_size: int, activation: str = "gelu_tanh"):
+    def __init__(self, hidden_size: int, intermediate_size: int, activation: str = "gelu_tanh", limit: float | None = None):
         self.hidden_size, self.intermediate_size = int(hidden_size), int(intermediate_size)
         self.activation = activation
         self.activation_code = int(ACTIVATIONS.get(activation))   # an unknown name is refused with the known ones
+        self.limit = check_limit(activation, limit)
         self.gate_proj = self.up_proj = self.down_proj = self.gate_up = None
 
     def param_specs(self):
@@ -70,32 +86,35 @@ class GatedDense(FeedForward):
     def forward(self, x: torch.Tensor, ctx=None, defer_sum=False) -> torch.Tensor:
         # gelu(x.Wg^T) * (x.Wu^T), one kernel
         if self.gate_up is not None:
-            z = project(x, self.gate_up, activation=self.activation_code)
+            z = project(x, self.gate_up, activation=self.activation_code, limit=self.limit)
         else:
             if isinstance(x, PendingNorm):
                 x = x.materialize()
-            z = ops.gemm(x, self.gate_proj, w2=self.up_proj, activation=self.activation_code)
+            z = ops.gemm(x, self.gate_proj, w2=self.up_proj, activation=self.activation_code, limit=self.limit)
         return ops.gemm(z, self.down_proj, defer_sum=defer_sum)
 
 
 @FEED_FORWARDS.register("routed_experts")
 class RoutedExperts(FeedForward):
     """A mixture of experts: `num_experts` feed-forwards without biases, of which every token uses the `top` ones that
-    the router chooses; an expert's result is weighted by its score times `router_scale`, the weights are not
-    renormalized.
+    the router chooses; an expert's result is weighted by its score times `router_scale`.
 
       gated       True: an expert is down(act(gate x) * (up x)); False: down(act(up x)), and there are no gate tensors
-      router      'softmax': scores are the softmax of the router's logits over all experts (32-bit), the largest are
-                  chosen; 'sigmoid': scores are sigmoids of the logits, the choice goes by score + a stored correction
-                  per expert (`correction`) among the experts of the `keep_groups` best of `num_groups` equal groups of
-                  neighbours (a group's score: the sum of its two largest choice scores), and the weights are the
-                  scores without the correction
+      activation  of the gated form also 'clamped_glu', with `limit` (`shared_limit` for the shared feed-forward)
+      router      scores (32-bit) are the softmax of the router's logits over all experts ('softmax') or sigmoids of the
+                  logits ('sigmoid'); the choice goes by score + a stored correction per expert (`correction`), and the
+                  weights are the scores without the correction
+      num_groups  equal groups of neighbouring experts; only experts of the `keep_groups` best can be chosen.  A group's
+                  score: `group_score` 'two_largest', the sum of its two largest choice scores, or 'largest'
+      renormalize None, or a small constant e: the weights are the chosen scores divided by their sum + e
       shared_size one more feed-forward of the experts' form runs for every token and is added, times sigmoid(w . x)
                   (one number per token) if `shared_gate`."""
 
     def __init__(self, hidden_size: int, num_experts: int, top: int, expert_size: int, router_scale: float = 1.0,
                  activation: str = "silu", shared_size: int | None = None, shared_gate: bool = True, gated: bool = True,
-                 router: str = "softmax", correction: bool = False, num_groups: int = 1, keep_groups: int = 1):
+                 router: str = "softmax", correction: bool = False, num_groups: int = 1, keep_groups: int = 1,
+                 group_score: str = "two_largest", renormalize: float | None = None, limit: float | None = None,
+                 shared_limit: float | None = None):
         self.hidden_size, self.num_experts, self.top = int(hidden_size), int(num_experts), int(top)
         self.expert_size, self.router_scale = int(expert_size), float(router_scale)
         if not 1 <= self.top <= self.num_experts:
@@ -104,16 +123,22 @@ class RoutedExperts(FeedForward):
             raise ValueError(f"routed_experts: the router is 'softmax' or 'sigmoid', not {router!r}")
         self.router_kind, self.correction = router, bool(correction)
         self.num_groups, self.keep_groups = int(num_groups), int(keep_groups)
-        if router == "softmax" and (self.correction or self.num_groups != 1):
-            raise ValueError("routed_experts: a correction and groups go with the sigmoid router")
+        if group_score not in ("two_largest", "largest"):
+            raise ValueError(f"routed_experts: a group's score is its 'two_largest' or its 'largest', not {group_score!r}")
+        self.group_best = 1 if group_score == "largest" else 2
+        self.renormalize = None if renormalize is None else float(renormalize)
         if self.num_groups < 1 or self.num_experts % self.num_groups or not 1 <= self.keep_groups <= self.num_groups \
                 or self.top > self.keep_groups * (self.num_experts // self.num_groups):
             raise ValueError(f"routed_experts: {num_experts} experts in {num_groups} groups of which {keep_groups} stay "
                              f"do not give {top} choices")
         self.gated = bool(gated)
         self.activation_code = int(ACTIVATIONS.get(activation))
-        shared_cls = GatedDense if self.gated else Dense
-        self.shared = shared_cls(hidden_size, int(shared_size), activation) if shared_size else None
+        self.limit = check_limit(activation, limit)
+        self.shared = None
+        if shared_size and self.gated:
+            self.shared = GatedDense(hidden_size, int(shared_size), activation, shared_limit)
+        elif shared_size:
+            self.shared = Dense(hidden_size, int(shared_size), activation)
         self.shared_gate = bool(shared_gate) and self.shared is not None
         self.router = self.gate_w = self.up_w = self.down_w = self.correction_w = None
 
@@ -149,11 +174,14 @@ class RoutedExperts(FeedForward):
     def forward(self, x: torch.Tensor, ctx=None) -> torch.Tensor:
         E = self.num_experts
         logits = ops.gemm(x, self.router, out_dtype=torch.float32)
-        if self.router_kind == "sigmoid":
+        plain = self.router_kind == "softmax" and not self.correction and self.num_groups == 1 and self.renormalize is None
+        if not plain:
             experts, weights = ops.route_choice(logits[:, :E], self.top, self.router_scale, correction=self.correction_w,
-                                                groups=self.num_groups, keep=self.keep_groups)
+                                                groups=self.num_groups, keep=self.keep_groups,
+                                                softmax=self.router_kind == "softmax", group_best=self.group_best,
+                                                renorm=self.renormalize)
         else:
             experts, weights = ops.route(logits[:, :E], self.top, self.router_scale)
         shared = self.shared.forward(x, ctx) if self.shared is not None else None
         return ops.routed_experts(x, experts, weights, self.gate_w, self.up_w, self.down_w, self.activation_code,
-                                  shared=shared, shared_gate=logits[:, E:E + 1] if self.shared_gate else None)
+                                  shared=shared, shared_gate=logits[:, E:E + 1] if self.shared_gate else None, limit=self.limit)

@@ -1,5 +1,6 @@
-"""RMSNorm with an optional `(1 + scale)` gain (simply/model_lib.py:114-178, LayerNorm with
-use_bias=False).  Statistics and the multiplication are in float32."""
+"""Norms: RMSNorm with an optional `(1 + scale)` gain (simply/model_lib.py:114-178, LayerNorm with
+use_bias=False), and the layer norm with weight and bias.  Statistics and the
+multiplication are in float32."""
 from __future__ import annotations
 
 import torch
@@ -38,7 +39,7 @@ class RMSNorm(Norm):
         #: a constant that the norm's result is multiplied by (a residual multiplier of blocks that norm what a part
         #: returns); the kernels that fuse this norm into a product compute the norm without it
         self.mult = float(mult)
-        self.fusable_rms = self.mult == 1.0
+        self.fusable_rms = self.fuses_sum = self.mult == 1.0
         self.adds_partial_sums = self.mult == 1.0
         self.scale: torch.Tensor | None = None
 
@@ -49,6 +50,10 @@ class RMSNorm(Norm):
         if self.mult != 1.0:
             raise NotImplementedError("rmsnorm: a norm with a factor is applied through add_into only")
         return ops.rmsnorm(x, self.scale, self.eps, self.scale_plus_one, out_dtype)
+
+    def after_sum(self, residual, y, mult, out_dtype):
+        return ops.residual_add_next_norm(y, residual, self.scale, eps=self.eps, plus_one=self.scale_plus_one, mult=mult,
+                                          out_dtype=out_dtype)
 
     def add_into(self, residual, y, next_norm, out_dtype):
         """residual += self(y) and, fused when the next norm is an RMSNorm too, next_norm(residual)."""
@@ -68,3 +73,29 @@ class RMSNorm(Norm):
                 next_plus_one=True if next_norm is None else next_norm.scale_plus_one, out_dtype=out_dtype)
         ops.add_rmsnorm(y, residual, post_weight=self.scale, post_eps=self.eps, post_plus_one=self.scale_plus_one)
         return next_norm.forward(residual, out_dtype)
+
+
+@NORMS.register("layernorm")
+class LayerNorm(Norm):
+    """(x - mean) / sqrt(variance + eps) * weight + bias, the variance being the mean of the squared deviations."""
+
+    fuses_sum = True
+
+    def __init__(self, dim: int, eps: float):
+        self.dim, self.eps = int(dim), float(eps)
+        self.scale = self.bias = None
+
+    def param_specs(self):
+        return {"scale": ParamSpec((self.dim,), role="vector", init="norm"),
+                "bias": ParamSpec((self.dim,), role="vector", init="norm")}
+
+    def load(self, tensors):
+        self.scale, self.bias = tensors["scale"].contiguous(), tensors["bias"].to(tensors["scale"].dtype).contiguous()
+
+    def after_sum(self, residual, y, mult, out_dtype):
+        return ops.residual_add_next_norm(y, residual, self.scale, bias=self.bias, eps=self.eps, mult=mult,
+                                          out_dtype=out_dtype)
+
+    def forward(self, x, out_dtype):
+        # (the kernel reads 32-bit rows and, with nothing to add, leaves them as they are)
+        return self.after_sum(x if x.dtype == torch.float32 else x.to(torch.float32), None, 1.0, out_dtype)

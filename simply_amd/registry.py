@@ -91,5 +91,7 @@ EMBEDDINGS = Registry("embedding")
 HEADS = Registry("head")
 #: parts that read and update the residual stream themselves, behind a block's mixer and feed-forward
 STREAM_PARTS = Registry("stream part")
+#: what is done to the residual stream before every pass of a loop over layers
+PASS_INPUTS = Registry("pass input")
 #: activation name -> code of the gated product's epilogue (simply_amd/csrc/activations.h)
 ACTIVATIONS = Registry("activation")

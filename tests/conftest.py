@@ -36,7 +36,7 @@ def cpu_ops(monkeypatch):
                  "delta_prepare", "delta_inputs", "delta_rule", "embed_sum", "token_gate_", "bias_add_", "weighted_sum",
                  "exp_gates", "linear_state", "normalized_readout", "route", "routed_experts", "residual_add_next_norm",
                  "paged_attention_maps", "attention_maps_units_takes", "norm_rope_cache_write", "short_conv", "head_product", "rglru_scan",
-                 "attention_inputs", "route_choice"):
+                 "attention_inputs", "route_choice", "token_shift", "low_rank_decay", "concat_rows", "gemm_sections"):
         monkeypatch.setattr(ops, name, getattr(torch_ops, name))
     return torch_ops
 

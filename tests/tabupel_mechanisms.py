@@ -379,7 +379,7 @@ def latent_part(device, dtype, sizes=(40, 3, 12, 8, 10, 20, 24), window=13, page
     want = plain.latent_attention(x.double(), p, m, 1e-5)
     part = _load_part("latent_attention", {
         "hidden_size": D, "num_heads": H, "key_dim": dk, "rot_dim": dr, "value_dim": dv, "q_rank": Rq, "kv_rank": R,
-        "scale": 0.3, "norm_eps": 1e-5, "window": window, "output_gate": True,
+        "scale": 0.3, "norm_eps": 1e-5, "window": window, "output_gate": "head",
         "position_encoding": PartSpec("pair_rope", {"dims": dr, "base": 1000.0, "scaling": {"kind": "ramp", **sc}}),
     }, {"dq_proj": p["dq"], "dq_norm": p["dq.norm"], "uq_proj": p["uq"], "dkv_proj": p["dkv"], "dkv_norm": p["dkv.norm"],
         "uk_proj": p["uk"], "uv_proj": p["uv"], "gate_proj": p["g"], "o_proj": p["o"]}, dtype, device)

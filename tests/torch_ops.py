@@ -122,8 +122,19 @@ def gelu_erf(x):
 ACTIVATIONS = (gelu_tanh, silu, squared_relu, gelu_erf)   # by the kernels' activation codes
 
 
+CLAMPED_GLU = 4
+
+
+def gated(activation, gate, up, limit=None):
+    """The two factors of a gated product joined by the rule of that code."""
+    if activation == CLAMPED_GLU:
+        g, u = gate.clamp(max=limit), up.clamp(-limit, limit)
+        return g * torch.sigmoid(1.702 * g) * (u + 1.0)
+    return ACTIVATIONS[activation](gate) * up
+
+
 def gemm(a, w, *, w2=None, soft_cap=None, out_dtype=None, out=None, algo=0, shape=0, activation=0, defer_sum=False,
-         activate=None):
+         activate=None, limit=None):
     # (defer_sum: the kernels may leave a sum to the caller; this stand-in never cuts a product)
     out_dtype = out_dtype or a.dtype
     if getattr(w, "paired", False):
@@ -132,7 +143,7 @@ def gemm(a, w, *, w2=None, soft_cap=None, out_dtype=None, out=None, algo=0, shap
     c = _f(a) @ _f(w).T
     if w2 is not None:
         up = _f(a) @ _f(w2).T
-        c = ACTIVATIONS[activation](_f(c.to(out_dtype))) * _f(up.to(out_dtype))
+        c = gated(activation, _f(c.to(out_dtype)), _f(up.to(out_dtype)), limit)
     elif soft_cap:
         c = soft_cap * torch.tanh(c / soft_cap)
     elif activate is not None:
@@ -265,7 +276,7 @@ def gated_heads(x, gate, num_heads, size, *, kind, weight=None, eps=0.0, out_dty
     T = x.shape[0]
     v = _f(x).reshape(T, num_heads, size)
     if weight is not None:
-        v = v / torch.sqrt((v * v).mean(-1, keepdim=True) + eps) * _f(weight)
+        v = v / torch.sqrt((v * v).mean(-1, keepdim=True) + eps) * _f(weight).reshape(-1, size)
     g = _f(gate).reshape(T, num_heads, 1 if per_head else size)
     g = torch.sigmoid(g) if kind == GATE_SIGMOID else g * torch.sigmoid(g)
     r = (v * g).reshape(T, num_heads * size).to(out_dtype or (out.dtype if out is not None else x.dtype))
@@ -539,7 +550,7 @@ def exp_gates(raw, bias, cap, num_heads, m_state, seq_meta, num_seqs):
 
 
 def linear_state(proj, q_at, k_at, v_at, q_mult, gates, scalar, num_heads, key_dim, value_dim, ones, state, seq_meta,
-                 num_seqs, *, decay_bias=None, tau=None):
+                 num_seqs, *, decay_bias=None, tau=None, bonus=None):
     H, dk, dv = num_heads, key_dim, value_dim
     if tau is not None:   # the gates are z: a = sigmoid(z + bias)^(1 / tau)
         z = _f(gates) + (_f(decay_bias) if decay_bias is not None else 0.0)
@@ -560,8 +571,10 @@ def linear_state(proj, q_at, k_at, v_at, q_mult, gates, scalar, num_heads, key_d
                 a, c = g[t, :H].view(H, 1, 1), g[t, H:2 * H].view(H, 1)
             else:
                 a, c = g[t, :H * dk].view(H, 1, dk), 1.0
-            S = a * S + (c * v)[:, :, None] * k[:, None, :]
-            out[t] = torch.einsum("hcd,hd->hc", S, q).reshape(-1)
+            kv = (c * v)[:, :, None] * k[:, None, :]
+            read = S + _f(bonus).view(H, 1, dk) * kv if bonus is not None else a * S + kv
+            S = a * S + kv
+            out[t] = torch.einsum("hcd,hd->hc", read, q).reshape(-1)
         if count > 0:
             state[slot, :H * dk * CT] = S.reshape(-1).to(torch.float32)
     return out.to(torch.float32)
@@ -584,23 +597,26 @@ def route(logits, top, scale):
     return best.indices.to(torch.int32).contiguous(), (best.values * scale).to(torch.float32).contiguous()
 
 
-def route_choice(logits, top, scale, *, correction=None, groups=1, keep=1):
-    s = torch.sigmoid(_f(logits))
+def route_choice(logits, top, scale, *, correction=None, groups=1, keep=1, softmax=False, group_best=2, renorm=None):
+    s = torch.softmax(_f(logits), -1) if softmax else torch.sigmoid(_f(logits))
     T, E = s.shape
     c = s + _f(correction) if correction is not None else s.clone()
     if groups > 1:
         per = E // groups
         by_group = c.reshape(T, groups, per)
-        score = torch.topk(by_group, min(2, per), dim=-1).values.sum(-1)
+        score = torch.topk(by_group, min(group_best, per), dim=-1).values.sum(-1)
         stay = torch.zeros(T, groups, dtype=torch.bool, device=s.device)
         stay.scatter_(1, torch.topk(score, keep, dim=-1).indices, True)
         c = torch.where(stay[:, :, None].expand(T, groups, per).reshape(T, E), c, torch.full_like(c, float("-inf")))
     chosen = torch.topk(c, top, dim=-1).indices
-    return chosen.to(torch.int32).contiguous(), (torch.gather(s, 1, chosen) * scale).to(torch.float32).contiguous()
+    w = torch.gather(s, 1, chosen)
+    if renorm is not None:
+        w = w / (w.sum(-1, keepdim=True) + renorm)
+    return chosen.to(torch.int32).contiguous(), (w * scale).to(torch.float32).contiguous()
 
 
 def routed_experts(x, experts, weights, gate_w, up_w, down_w, activation, *, shared=None, shared_gate=None,
-                   out_dtype=None):
+                   out_dtype=None, limit=None):
     from simply_amd.kernels.packing import TiledWeight, unpack_tiles
 
     def matrix(stack, e):
@@ -617,8 +633,8 @@ def routed_experts(x, experts, weights, gate_w, up_w, down_w, activation, *, sha
             if gate_w is None:   # experts without a gate
                 h = _activation(activation, (xf[t] @ matrix(up_w, e).T).to(x.dtype).to(xf.dtype))
             else:
-                h = _activation(activation, (xf[t] @ matrix(gate_w, e).T).to(x.dtype).to(xf.dtype)) \
-                    * (xf[t] @ matrix(up_w, e).T).to(x.dtype).to(xf.dtype)
+                h = gated(activation, (xf[t] @ matrix(gate_w, e).T).to(x.dtype).to(xf.dtype),
+                          (xf[t] @ matrix(up_w, e).T).to(x.dtype).to(xf.dtype), limit)
             out[t] += _f(weights[t, k]) * (h.to(x.dtype).to(xf.dtype) @ matrix(down_w, e).T)
     if shared is not None:
         s = _f(shared)
@@ -629,13 +645,17 @@ def routed_experts(x, experts, weights, gate_w, up_w, down_w, activation, *, sha
 # --------------------------------------------------------------------------- attention with several maps, latents, rglru
 
 
-def residual_add_next_norm(y, residual, weight, *, eps, plus_one=False, mult=1.0, out_dtype=None):
+def residual_add_next_norm(y, residual, weight, *, eps, plus_one=False, mult=1.0, bias=None, out_dtype=None):
     if hasattr(y, "materialize"):
         y = y.materialize()
     if y is not None:
         residual.copy_((_f(residual) + mult * _f(y)).to(torch.float32))
     h = _f(residual)
+    if bias is not None:
+        h = h - h.mean(-1, keepdim=True)
     out = h / torch.sqrt((h * h).mean(-1, keepdim=True) + eps) * (_f(weight) + (1.0 if plus_one else 0.0))
+    if bias is not None:
+        out = out + _f(bias)
     return out.to(out_dtype or (y.dtype if y is not None else torch.float32))
 
 
@@ -748,7 +768,7 @@ def head_product(x, w, *, in_stride=None, tail=0, gate=None, out_dtype=None):
     heads = torch.stack([xf[:, h * hs:h * hs + I + tail] for h in range(H)], dim=1)       # [T, H, I + tail]
     o = torch.einsum("thi,hoi->tho", heads[..., :I], _f(w))
     if gate is not None:
-        o = o * torch.sigmoid(_f(gate))[:, :, None]
+        o = o * torch.sigmoid(_f(gate)).reshape(T, H, -1)
     return torch.cat([o, heads[..., I:]], dim=-1).reshape(T, H * (O + tail)).to(out_dtype or x.dtype)
 
 
@@ -832,3 +852,33 @@ def attention_inputs(proj, seq_meta, num_seqs, max_q_len, num_heads, num_kv_head
         k_pages.copy_(rows_as_stored_keys(rows))
         v_pages[page, :, :, off] = v[keep].to(v_pages.dtype)
     return (q * q_mult).reshape(T, H * dk).to(proj.dtype)
+
+
+# --------------------------------------------------------------------------- token shift, data-dependent decays, passes
+
+
+def token_shift(h, mu, tails, seq_meta, num_seqs, max_q_len):
+    T, D = h.shape
+    out = torch.empty((T, mu.shape[0] * D), dtype=h.dtype, device=h.device)
+    for slot, first, count, _ in seq_meta[:num_seqs].tolist():
+        if count == 0:
+            continue
+        now = _f(h[first:first + count])
+        before = torch.cat([_f(tails[slot, :D])[None], now[:-1]])
+        mixes = now[:, None, :] + (before - now)[:, None, :] * _f(mu)[None]
+        out[first:first + count] = mixes.reshape(count, -1).to(h.dtype)
+        tails[slot, :D] = now[-1].to(torch.float32)
+    return out
+
+
+def low_rank_decay(p, w, base):
+    return torch.exp(-torch.exp(torch.tanh(_f(p)) @ _f(w) + _f(base))).to(torch.float32)
+
+
+def concat_rows(x, y, out_dtype):
+    return torch.cat([x, y], dim=1).to(out_dtype)
+
+
+def gemm_sections(a, w):
+    S, N, K = len(w.parts), w.rows, w.cols
+    return torch.cat([gemm(a[:, s * K:(s + 1) * K], w.parts[s]) for s in range(S)], dim=1)
