@@ -612,6 +612,71 @@ def run_rudutar(args):
             torch.cuda.empty_cache()
 
 
+# --only kolorax: layer sizes that resemble a real model's, for the Kolorax design (three layers with the token-shift
+# recurrence to one with latent attention, routed clamped experts in every layer, layers 2 and 3 looped twice) and, beside
+# it, the closest model that the engine has, Nemidra, at equal width, depth, heads and head size: gated linear attention
+# in place of the recurrence, windowed attention beside a matrix memory in place of the latent attention, experts of the
+# same sizes in every layer, the same loop
+KOLORAX_LOOP = {"start": 2, "stop": 4, "times": 2}
+
+
+def kolorax_config(size: dict, layers: int) -> dict:
+    W, H, d, ff = size["width"], size["heads"], size["dim"], size["ff"] // 4
+    mlp = {"kind": "moe", "expert": {"ff": ff, "limit": 7.0}, "shared": {"ff": ff, "limit": 7.0},
+           "router": {"experts": 16, "top": 2, "groups": {"count": 4, "keep": 2}}}
+    out = []
+    for i in range(layers):
+        if i % 4 == 3:
+            out.append({"type": "latent_attention", "mlp": mlp,
+                        "mixer": {"heads": H, "dim": d, "rot_dim": 64, "vdim": d, "kv_rank": 512, "scale": (d + 64) ** -0.5,
+                                  "rot": {"dims": 64, "base": 50000.0}}})
+        else:
+            out.append({"type": "wkv", "mlp": mlp, "mixer": {"heads": H, "dim": d, "rank": 64}})
+    d = {"architecture": "Kolorax", "vocab": size["vocab"], "width": W, "residual_mult": 0.7, "norm": {"eps": 1e-5},
+         "embedding": {"scale": 1.0}, "layers": out}
+    if layers >= KOLORAX_LOOP["stop"]:
+        d["loop"] = dict(KOLORAX_LOOP)
+    return d
+
+
+def nemidra_of_kolorax_size(size: dict, layers: int, positions: int) -> dict:
+    d = nemidra_config(size, layers, positions)
+    for l in d["layers"]:
+        l["mlp"] = {"kind": "moe", "expert": {"ff": size["ff"] // 4}, "router": {"experts": 16, "top": 2, "scale": 1.0},
+                    "shared": {"ff": size["ff"] // 4}}
+    if layers >= KOLORAX_LOOP["stop"]:
+        d["loop"] = dict(KOLORAX_LOOP)
+    return d
+
+
+def run_kolorax(args):
+    import torch
+    from simply_amd.config import config_from_dict
+    from simply_amd.engine.loading import random_model
+
+    tdtype = torch.bfloat16 if args.dtype == "bfloat16" else torch.float32
+    layers = args.layers or 8
+    positions = max(args.prefill_tokens, args.context + args.steps + args.warmup) + 16
+    for name in args.sizes.split(","):
+        size = ZENUZEN_SIZES[name]
+        for label, d in (("kolorax", kolorax_config(size, layers)),
+                         ("nemidra-equal-size", nemidra_of_kolorax_size(size, layers, positions))):
+            if args.alone and label != args.alone_model:
+                continue
+            cfg = config_from_dict(d)
+            model = random_model(cfg, 0, tdtype, torch.device("cuda:0"), std=0.02)
+            pt, dt = run_executor_bench(model, size["vocab"], args.prefill_tokens, args.batch, args.context, args.steps,
+                                        args.warmup, args.page_size, args.dtype)
+            print(json.dumps({"metric": "prefill and decode tokens/s through the step function", "model": label,
+                              "size": name, "width": size["width"], "layers": layers, "layer_runs": len(model.spec.schedule),
+                              "prefill_tokens": args.prefill_tokens, "prefill_tokens_per_s": round(args.prefill_tokens / pt, 1),
+                              "prefill_ms": round(pt * 1e3, 3), "batch": args.batch, "context": args.context,
+                              "decode_tokens_per_s": round(args.batch / dt, 1), "decode_ms_per_step": round(dt * 1e3, 3),
+                              "dtype": args.dtype, "data": "synthetic"}), flush=True)
+            del model
+            torch.cuda.empty_cache()
+
+
 def main():
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -628,7 +693,7 @@ def main():
     ap.add_argument("--contexts", default="1024,4096,8192", help="--only decode-grid: the context lengths")
     ap.add_argument("--only", default="all", choices=["all", "decode", "decode-grid", "prefill", "prefill-chunked", "products",
                                                       "gated-products", "ceilings", "zenuzen", "nemidra", "tabupel",
-                                                      "rudutar"],
+                                                      "rudutar", "kolorax"],
                     help="measure one part alone (for profiles); the line then holds that part only.  products / "
                          "gated-products: the sweep of the product kernels over rows and weight sizes; ceilings: "
                          "what the GPU itself reaches in reading HBM and in bfloat16 MFMA instructions")
@@ -636,8 +701,10 @@ def main():
                     help="decode steps run one at a time after the timed ones, for the p50 and p99 of a step's latency")
     ap.add_argument("--shape", default="2b", choices=sorted(SHAPES), help="layer sizes: Gemma 2 2B (the default), 9B, 27B")
     ap.add_argument("--sizes", default="small,medium,large",
-                    help="--only zenuzen / nemidra / tabupel / rudutar: which of the layer sizes small, medium, large (8 layers each, or --layers)")
-    ap.add_argument("--alone", action="store_true", help="--only nemidra / tabupel / rudutar: without the closest model beside it (for profiles)")
+                    help="--only zenuzen / nemidra / tabupel / rudutar / kolorax: which of the layer sizes small, medium, large (8 layers each, or --layers)")
+    ap.add_argument("--alone", action="store_true", help="--only nemidra / tabupel / rudutar / kolorax: without the closest model beside it (for profiles)")
+    ap.add_argument("--alone-model", default="kolorax", choices=["kolorax", "nemidra-equal-size"],
+                    help="--only kolorax --alone: which of the two models runs")
     ap.add_argument("--requests", type=int, default=0,
                     help="instead of timed decode steps: a workload of this many requests through the scheduler")
     ap.add_argument("--prompt-min", type=int, default=128)
@@ -672,6 +739,9 @@ def main():
         return
     if args.only == "rudutar":
         run_rudutar(args)
+        return
+    if args.only == "kolorax":
+        run_kolorax(args)
         return
     d = dict(GEMMA2_2B, **SHAPES[args.shape])
     full_layers = d["num_hidden_layers"]

@@ -108,10 +108,14 @@ int sa_gemm(const void* A, int a_dtype, int64_t lda, const void* W, const void* 
 // == 1: C holds the product as after sa_gemm.
 // C = the sum of `count` planes [M][N] float32 in their order, rounded to C's type: the kernel that sa_gemm_planes
 // leaves out.
+// sa_gemm (bfloat16, tiled weights, no epilogue) for several products at once: rows s n_step .. of W, n_step a multiple
+// of 16 (the last section may be shorter), times the columns s a_step .. s a_step + K of A; C [M, N].
+int sa_gemm_sections(const void* A, int64_t lda, const void* W, void* C, int c_dtype, int64_t ldc, int M, int N, int K,
+                     int n_step, int a_step, void* workspace, int64_t workspace_bytes, hipStream_t stream);
 // Which kernel sa_gemm would run for bfloat16 operands of these sizes with tiled weights and 16-byte aligned
 // operands (2: few-rows, 3: tiled, 4: wide), and, in us[0..2] if it is not null, the microseconds that the library
 // expects of the three (negative: not eligible).  c_dtype is the output's element type (the wide kernel writes
-// bfloat16 only).  A host function: nothing is launched.
+// 32-bit results of large products without an epilogue only).  A host function: nothing is launched.
 int sa_gemm_plan(int M, int N, int K, int epilogue, int c_dtype, int64_t workspace_bytes, double* us);
 int sa_sum_planes(const float* planes, int count, void* C, int c_dtype, int64_t ldc, int M, int N, hipStream_t stream);
 int sa_gemm_planes(const void* A, int a_dtype, int64_t lda, const void* W, const void* W2, int w_dtype, void* C,
@@ -227,6 +231,12 @@ int sa_probe_mfma(const void* operands, int iters, int workgroups, void* sink, h
 }
 
 namespace sa {
+// Several products run as one: rows s n_step .. of W (a multiple of 16; the last section may be shorter) are multiplied
+// with the columns s a_step .. s a_step + K of A.  n_step 0: one product.
+struct Sections {
+  int n_step = 0;
+  int a_step = 0;
+};
 int gemm_generic(const void* A, int a_dtype, int64_t lda, const void* W, const void* W2, int w_dtype, void* C,
                  int c_dtype, int64_t ldc, int M, int N, int K, int epi, int act, float cap, int packed,
                  hipStream_t stream);
@@ -240,7 +250,7 @@ double gemm_skinny_predict_us(int M, int N, int K, int epi);
 double gemm_tiled_predict_us(int M, int N, int K, int epi);
 double gemm_wide_predict_us(int M, int N, int K, int epi, bool have_workspace, size_t workspace_bytes);
 int gemm_skinny(const void* A, int64_t lda, const void* W, const void* W2, void* C, int c_dtype, int64_t ldc, int M,
-                int N, int K, int epi, int act, float cap, int packed, int shape, hipStream_t stream);
+                int N, int K, int epi, int act, float cap, int packed, int shape, hipStream_t stream, Sections sec = {});
 bool paged_attention_decode_takes(int H, int Kh, int hd, int page_size, int max_q_len, int64_t q_stride, const void* q);
 int paged_attention_decode(const void* q, int64_t q_stride, const void* k_pages, const void* v_pages,
                            const int* block_table, int table_stride, const int* seq_meta, int seq_begin, int seq_count,
@@ -258,14 +268,15 @@ int paged_attention_prefill(const void* q, int64_t q_stride, const void* k_pages
 bool gemm_wide_takes(int M, int N, int K, int64_t lda, int64_t ldc, const void* A, const void* W, const void* W2,
                      const void* C, int c_dtype, int epi, int packed);
 int gemm_wide(const void* A, int64_t lda, const void* W, void* C, int64_t ldc, int M, int N, int K, int epi, int act,
-              float limit, int shape, int ks, void* workspace, size_t workspace_bytes, hipStream_t stream, int* planes_left = nullptr);
+              float limit, int shape, int ks, void* workspace, size_t workspace_bytes, hipStream_t stream, int* planes_left = nullptr,
+              int c_dtype = 1 /* bfloat16 */, Sections sec = {});
 // C = epilogue(sum over z of partials[z][M][NW]): the second kernel of every product that cuts K over workgroups
 int gemm_sum_partials(const float* partials, int ks, void* C, int c_dtype, int64_t ldc, int M, int N, int NW, int epi,
                       int act, float cap, hipStream_t stream);
 bool gemm_streams_weights(int M, int NW, int K);
 bool gemm_tiled_takes(int M, int N, int K, int64_t lda, const void* A, const void* W, const void* W2, int packed);
 int gemm_tiled(const void* A, int64_t lda, const void* W, void* C, int c_dtype, int64_t ldc, int M, int N, int K,
-               int epi, int act, float cap, int ksplit, void* workspace, size_t workspace_bytes, hipStream_t stream);
+               int epi, int act, float cap, int ksplit, void* workspace, size_t workspace_bytes, hipStream_t stream, Sections sec = {});
 int paged_attention_generic(const void* q, int dtype, int64_t q_stride, const void* k_pages, const void* v_pages,
                             const int* block_table, int table_stride, const int* token_seq, const int* positions,
                             void* out, int64_t out_stride, int T, int H, int Kh, int hd, int page_size, int window,
@@ -519,9 +530,10 @@ int sa_expert_combine(const float* y, const float* weights, int top, const void*
 int sa_token_shift(const void* h, int dtype, int64_t h_stride, const void* mu, int mu_dtype, int streams, float* tails,
                    int64_t tail_stride, const int* seq_meta, int num_seqs, int max_q_len, void* out, int D,
                    hipStream_t stream);
-// out[t, c] = exp(-exp(sum_r w[r, c] tanh(p[t, r]) + w0[c])), 32-bit; w [rank, C].
-int sa_low_rank_decay(const void* p, int p_dtype, int64_t p_stride, const void* w, int w_dtype, const void* w0, int w0_dtype,
-                      float* out, int T, int C, int rank, hipStream_t stream);
+// out[t, c] = exp(-exp(sum_r w[c, r] tanh(p[t, r]) + w0[c])), 32-bit; w [C, rank], row-major or (tiled) in the operand
+// tiles of the product kernels.
+int sa_low_rank_decay(const void* p, int p_dtype, int64_t p_stride, const void* w, int w_dtype, int tiled, const void* w0,
+                      int w0_dtype, float* out, int T, int C, int rank, hipStream_t stream);
 // out[t] = [x[t] (D) | y[t] (E)] in out's type.
 int sa_concat_rows(const float* x, const float* y, void* out, int out_dtype, int T, int D, int E, hipStream_t stream);
 }

@@ -101,60 +101,93 @@ static bool launch_residual_add_norm_typed(const void* y, int64_t y_stride, cons
 // with the norm in front of the next part: out = h / sqrt(mean(h^2) + eps) * (w + plus_one) over the updated row h,
 // which is held in registers between the two.  y null: nothing is added.  CENTERED: a layer norm instead, out =
 // (h - mean) / sqrt(mean((h - mean)^2) + eps) * (w + plus_one) + b.  A y_stride of 0 adds the same row to every row.
-template <typename YT, typename OT, int NP, bool CENTERED>
+// The layer norm's mean and sum of squared deviations come from every wave's own, merged by the counts (one exchange
+// through LDS, no cancellation).
+template <typename YT, typename WT, typename OT, int NP, bool CENTERED>
 __global__ __launch_bounds__(256) void residual_add_next_norm_kernel(
-    const YT* __restrict__ y, int64_t y_stride, float mult, float* __restrict__ residual, const void* __restrict__ w,
-    const void* __restrict__ b, int w_dtype, float eps, float plus_one, OT* __restrict__ out, int D) {
+    const YT* __restrict__ y, int64_t y_stride, float mult, float* __restrict__ residual, const WT* __restrict__ w,
+    const WT* __restrict__ b, float eps, float plus_one, OT* __restrict__ out, int D) {
   __shared__ float scratch[16];
   const size_t yb = static_cast<size_t>(blockIdx.x) * y_stride, rb = static_cast<size_t>(blockIdx.x) * D;
-  float hv[NP], wv[NP], bv[CENTERED ? NP : 1];
-  float ss = 0.f;
+  float yv[NP], hv[NP], wv[NP], bv[CENTERED ? NP : 1];
 #pragma unroll
   for (int p = 0; p < NP; ++p) {
     const int d = threadIdx.x + p * 256;
     const bool ok = d < D;
-    const float yv = (ok && y != nullptr) ? to_float(y[yb + d]) : 0.f;
-    const float h = ok ? residual[rb + d] : 0.f;
-    wv[p] = ok ? load_f(w, w_dtype, d) + plus_one : 0.f;
-    if constexpr (CENTERED) bv[p] = ok ? load_f(b, w_dtype, d) : 0.f;
-    hv[p] = y != nullptr ? h + mult * yv : h;
-    if (ok && y != nullptr) residual[rb + d] = hv[p];
+    yv[p] = (ok && y != nullptr) ? to_float(y[yb + d]) : 0.f;
+    hv[p] = ok ? residual[rb + d] : 0.f;
+    wv[p] = ok ? to_float(w[d]) + plus_one : 0.f;
+    if constexpr (CENTERED) bv[p] = ok ? to_float(b[d]) : 0.f;
+  }
+  float ss = 0.f;
+#pragma unroll
+  for (int p = 0; p < NP; ++p) {
+    const int d = threadIdx.x + p * 256;
+    if (y != nullptr) {
+      hv[p] = hv[p] + mult * yv[p];
+      if (d < D) residual[rb + d] = hv[p];
+    }
     if constexpr (CENTERED) ss += hv[p];   // (entries beyond the row are zero)
     else ss = fmaf(hv[p], hv[p], ss);
   }
-  ss = block_sum(ss, scratch);
   if constexpr (CENTERED) {
-    const float mean = ss / static_cast<float>(D);
-    ss = 0.f;
+    const int wave = threadIdx.x / kWave;
+    int mine = 0;   // entries of the row that this wave holds
 #pragma unroll
     for (int p = 0; p < NP; ++p) {
-      hv[p] -= mean;
-      if (threadIdx.x + p * 256 < D) ss = fmaf(hv[p], hv[p], ss);
+      const int left = D - p * 256 - wave * kWave;
+      mine += left < 0 ? 0 : left > kWave ? kWave : left;
     }
+    const float part = mine > 0 ? wave_sum(ss) / static_cast<float>(mine) : 0.f;
+    float sq = 0.f;
+#pragma unroll
+    for (int p = 0; p < NP; ++p) {
+      const float e = hv[p] - part;
+      if (threadIdx.x + p * 256 < D) sq = fmaf(e, e, sq);
+    }
+    sq = wave_sum(sq);
+    if (threadIdx.x % kWave == 0) {
+      scratch[wave] = part;
+      scratch[4 + wave] = sq;
+      scratch[8 + wave] = static_cast<float>(mine);
+    }
+    __syncthreads();
+    float mean = 0.f;
+#pragma unroll
+    for (int v = 0; v < 4; ++v) mean = fmaf(scratch[v], scratch[8 + v], mean);
+    mean /= static_cast<float>(D);
+    ss = 0.f;
+#pragma unroll
+    for (int v = 0; v < 4; ++v) {
+      const float e = scratch[v] - mean;
+      ss += fmaf(e * e, scratch[8 + v], scratch[4 + v]);
+    }
+#pragma unroll
+    for (int p = 0; p < NP; ++p) hv[p] -= mean;
+  } else {
     ss = block_sum(ss, scratch);
   }
   const float r = 1.f / sqrtf(ss / static_cast<float>(D) + eps);
 #pragma unroll
   for (int p = 0; p < NP; ++p) {
     const int d = threadIdx.x + p * 256;
-    if (d < D) out[rb + d] = from_float<OT>(CENTERED ? fmaf(hv[p] * r, wv[p], bv[p]) : hv[p] * r * wv[p]);
+    if (d < D) out[rb + d] = from_float<OT>(CENTERED ? fmaf(hv[p] * r, wv[p], bv[CENTERED ? p : 0]) : hv[p] * r * wv[p]);
   }
 }
 
-template <typename YT, typename OT, bool CENTERED>
-static void launch_residual_add_next_norm(const void* y, int64_t y_stride, float mult, float* residual, const void* w, const void* b,
-                                          int w_dtype, float eps, float plus_one, void* out, int T, int D,
+template <typename YT, typename WT, typename OT, bool CENTERED>
+static void launch_residual_add_next_norm(const void* y, int64_t y_stride, float mult, float* residual, const void* w,
+                                          const void* b, float eps, float plus_one, void* out, int T, int D,
                                           hipStream_t stream) {
-  const YT* yp = static_cast<const YT*>(y);
-  OT* op = static_cast<OT*>(out);
-  if (D <= 1024)
-    residual_add_next_norm_kernel<YT, OT, 4, CENTERED><<<T, 256, 0, stream>>>(yp, y_stride, mult, residual, w, b, w_dtype, eps, plus_one, op, D);
-  else if (D <= 2048)
-    residual_add_next_norm_kernel<YT, OT, 8, CENTERED><<<T, 256, 0, stream>>>(yp, y_stride, mult, residual, w, b, w_dtype, eps, plus_one, op, D);
-  else if (D <= 4096)
-    residual_add_next_norm_kernel<YT, OT, 16, CENTERED><<<T, 256, 0, stream>>>(yp, y_stride, mult, residual, w, b, w_dtype, eps, plus_one, op, D);
-  else
-    residual_add_next_norm_kernel<YT, OT, 32, CENTERED><<<T, 256, 0, stream>>>(yp, y_stride, mult, residual, w, b, w_dtype, eps, plus_one, op, D);
+#define SA_NEXT_NORM_NP(NP)                                                                                        \
+  residual_add_next_norm_kernel<YT, WT, OT, NP, CENTERED><<<T, 256, 0, stream>>>(                                    \
+      static_cast<const YT*>(y), y_stride, mult, residual, static_cast<const WT*>(w), static_cast<const WT*>(b), eps, \
+      plus_one, static_cast<OT*>(out), D)
+  if (D <= 1024) SA_NEXT_NORM_NP(4);
+  else if (D <= 2048) SA_NEXT_NORM_NP(8);
+  else if (D <= 4096) SA_NEXT_NORM_NP(16);
+  else SA_NEXT_NORM_NP(32);
+#undef SA_NEXT_NORM_NP
 }
 
 // ------------------------------------------------------------------ heads normed and gated
@@ -421,18 +454,25 @@ extern "C" int sa_residual_add_next_norm(const void* y, int y_dtype, int64_t y_s
   const bool yb = y == nullptr ? out_dtype == kBF16 : y_dtype == kBF16;
   SA_REQUIRE((y == nullptr || y_dtype == kBF16 || y_dtype == kF32) && (out_dtype == kBF16 || out_dtype == kF32),
              "residual_add_next_norm: rows are bfloat16 or float32");
-#define SA_NEXT_NORM(YT, OT)                                                                                            \
-  do {                                                                                                                  \
-    if (b != nullptr)                                                                                                   \
-      launch_residual_add_next_norm<YT, OT, true>(y, y_stride, mult, residual, w, b, w_dtype, eps, plus, out, T, D, stream); \
-    else                                                                                                                \
-      launch_residual_add_next_norm<YT, OT, false>(y, y_stride, mult, residual, w, b, w_dtype, eps, plus, out, T, D, stream); \
+  SA_REQUIRE(w_dtype == kBF16 || w_dtype == kF32, "residual_add_next_norm: weights are bfloat16 or float32");
+#define SA_NEXT_NORM_C(YT, WT, OT)                                                                                        \
+  do {                                                                                                                    \
+    if (b != nullptr)                                                                                                     \
+      launch_residual_add_next_norm<YT, WT, OT, true>(y, y_stride, mult, residual, w, b, eps, plus, out, T, D, stream);   \
+    else                                                                                                                  \
+      launch_residual_add_next_norm<YT, WT, OT, false>(y, y_stride, mult, residual, w, b, eps, plus, out, T, D, stream);  \
+  } while (0)
+#define SA_NEXT_NORM(YT, OT)                               \
+  do {                                                     \
+    if (w_dtype == kBF16) SA_NEXT_NORM_C(YT, bf16, OT);    \
+    else SA_NEXT_NORM_C(YT, float, OT);                    \
   } while (0)
   if (yb && out_dtype == kBF16) SA_NEXT_NORM(bf16, bf16);
   else if (yb) SA_NEXT_NORM(bf16, float);
   else if (out_dtype == kBF16) SA_NEXT_NORM(float, bf16);
   else SA_NEXT_NORM(float, float);
 #undef SA_NEXT_NORM
+#undef SA_NEXT_NORM_C
   return check_launch("residual_add_next_norm");
 }
 

@@ -38,7 +38,8 @@ template <int MB, int EPI, bool PACKED, int kUnroll, int G>
 __global__ __launch_bounds__(1024) void gemm_skinny_kernel(const bf16* __restrict__ A, int64_t lda,
                                                            const bf16* __restrict__ W, const bf16* __restrict__ W2,
                                                            void* __restrict__ C, int c_dtype, int64_t ldc, int M, int N,
-                                                           int K, int chunks, int tile_rows, float cap, int act) {
+                                                           int K, int chunks, int tile_rows, float cap, int act,
+                                                           Sections sec) {
   constexpr int NP = EPI == 1 ? 2 : 1;  // planes: gate and up for the gated epilogue
   extern __shared__ float red[];        // [NW][NP][MB][16 * 17]
   const int tid = threadIdx.x, lane = tid % kWave;
@@ -46,6 +47,7 @@ __global__ __launch_bounds__(1024) void gemm_skinny_kernel(const bf16* __restric
   const int NW = blockDim.x / kWave;
   const int r = lane % 16, kq = lane / 16;
   const int n0 = blockIdx.x * tile_rows;
+  if (sec.n_step > 0) A += static_cast<size_t>(n0 / sec.n_step) * sec.a_step;   // (a tile lies within one section)
   const int c0 = static_cast<int>(static_cast<int64_t>(chunks) * wave / NW);
   const int c1 = static_cast<int>(static_cast<int64_t>(chunks) * (wave + 1) / NW);
 
@@ -241,7 +243,7 @@ static void choose_shape(int N, int chunks, int planes, int MB, int* tile_rows, 
 
 template <int MB, bool PACKED, int U, int G = 1>
 static void launch_skinny(const bf16* A, int64_t lda, const bf16* W, const bf16* W2, void* C, int c_dtype, int64_t ldc,
-                          int M, int N, int K, int epi, int act, float cap, int tile_rows, int waves,
+                          int M, int N, int K, int epi, int act, float cap, int tile_rows, int waves, Sections sec,
                           hipStream_t stream) {
   const int chunks = (K + 31) / 32;
   const dim3 grid((N + tile_rows - 1) / tile_rows);
@@ -249,13 +251,13 @@ static void launch_skinny(const bf16* A, int64_t lda, const bf16* W, const bf16*
   const size_t lds = static_cast<size_t>(waves) * (epi == 1 ? 2 : 1) * MB * 16 * 17 * sizeof(float);
   if (epi == 0)
     gemm_skinny_kernel<MB, 0, PACKED, U, G><<<grid, threads, lds, stream>>>(A, lda, W, W2, C, c_dtype, ldc, M, N, K, chunks,
-                                                                      tile_rows, cap, act);
+                                                                      tile_rows, cap, act, sec);
   else if (epi == 1)
     gemm_skinny_kernel<MB, 1, PACKED, U, G><<<grid, threads, lds, stream>>>(A, lda, W, W2, C, c_dtype, ldc, M, N, K, chunks,
-                                                                      tile_rows, cap, act);
+                                                                      tile_rows, cap, act, sec);
   else
     gemm_skinny_kernel<MB, 2, PACKED, U, G><<<grid, threads, lds, stream>>>(A, lda, W, W2, C, c_dtype, ldc, M, N, K, chunks,
-                                                                      tile_rows, cap, act);
+                                                                      tile_rows, cap, act, sec);
 }
 
 bool gemm_skinny_takes(int M, int N, int K, int64_t lda, const void* A, const void* W, const void* W2) {
@@ -286,7 +288,7 @@ double gemm_skinny_predict_us(int M, int N, int K, int epi) {
 
 // shape > 0 fixes the cut: tile_rows * 100 + waves (for instance 816: 8 rows, 16 waves)
 int gemm_skinny(const void* A, int64_t lda, const void* W, const void* W2, void* C, int c_dtype, int64_t ldc, int M,
-                int N, int K, int epi, int act, float cap, int packed, int shape, hipStream_t stream) {
+                int N, int K, int epi, int act, float cap, int packed, int shape, hipStream_t stream, Sections sec) {
   const int chunks = (K + 31) / 32, planes = epi == 1 ? 2 : 1;
   const int MB = M <= 16 ? 1 : (M <= 32 ? 2 : 4);
   int tile_rows, waves;
@@ -306,15 +308,15 @@ int gemm_skinny(const void* A, int64_t lda, const void* W, const void* W2, void*
 #define SA_SKINNY(MBV)                                                                                              \
   do {                                                                                                              \
     if (packed)                                                                                                     \
-      launch_skinny<MBV, true, 4>(a, lda, w, w2, C, c_dtype, ldc, M, N, K, epi, act, cap, tile_rows, waves, stream); \
+      launch_skinny<MBV, true, 4>(a, lda, w, w2, C, c_dtype, ldc, M, N, K, epi, act, cap, tile_rows, waves, sec, stream); \
     else                                                                                                            \
-      launch_skinny<MBV, false, 4>(a, lda, w, w2, C, c_dtype, ldc, M, N, K, epi, act, cap, tile_rows, waves, stream); \
+      launch_skinny<MBV, false, 4>(a, lda, w, w2, C, c_dtype, ldc, M, N, K, epi, act, cap, tile_rows, waves, sec, stream); \
   } while (0)
   // up to 8 rows against tiled weights: two or four chunks of K to a load of activations
   if (packed && K % 32 == 0 && tile_rows == 16 && M <= 4)
-    launch_skinny<1, true, 4, 4>(a, lda, w, w2, C, c_dtype, ldc, M, N, K, epi, act, cap, tile_rows, waves, stream);
+    launch_skinny<1, true, 4, 4>(a, lda, w, w2, C, c_dtype, ldc, M, N, K, epi, act, cap, tile_rows, waves, sec, stream);
   else if (packed && K % 32 == 0 && tile_rows == 16 && M <= 8)
-    launch_skinny<1, true, 4, 2>(a, lda, w, w2, C, c_dtype, ldc, M, N, K, epi, act, cap, tile_rows, waves, stream);
+    launch_skinny<1, true, 4, 2>(a, lda, w, w2, C, c_dtype, ldc, M, N, K, epi, act, cap, tile_rows, waves, sec, stream);
   else if (MB == 1) SA_SKINNY(1);
   else if (MB == 2) SA_SKINNY(2);
   else SA_SKINNY(4);

@@ -40,7 +40,7 @@ template <int WM, int EPI, int WAVES_N, bool TAIL>
 __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2)))
 void gemm_tiled_kernel(const bf16* __restrict__ A, int64_t lda, const bf16* __restrict__ W, void* __restrict__ C,
                        int c_dtype, int64_t ldc, int M, int N, int K, int chunks, float cap, int act,
-                       float* __restrict__ partials) {
+                       float* __restrict__ partials, Sections sec) {
   constexpr int WAVES_M = 4 / WAVES_N;
   constexpr int BM = WAVES_M * WM * 16;
   constexpr int BNW = WAVES_N * 64;  // weight rows per workgroup
@@ -75,8 +75,17 @@ void gemm_tiled_kernel(const bf16* __restrict__ A, int64_t lda, const bf16* __re
   }
   const int m_base = by * BM;
   const int NW = EPI == 1 ? 2 * ((N + 15) / 16) * 16 : N;
-  const int ntiles = (NW + 15) / 16;
-  const int nt0 = bx * (BNW / 16) + wn * 4;  // this wave's first 16-row tile of W
+  // several products at once: which section this workgroup is in, its columns of A, its rows of W
+  int first_tile = 0, NL = NW;   // the section's first 16-row tile of W and the end of its rows
+  if (sec.n_step > 0) {
+    const int per = (sec.n_step + BNW - 1) / BNW, s = bx / per;
+    bx -= s * per;
+    first_tile = s * (sec.n_step / 16);
+    A += static_cast<size_t>(s) * sec.a_step;
+    NL = (s + 1) * sec.n_step < NW ? (s + 1) * sec.n_step : NW;
+  }
+  const int ntiles = (NL + 15) / 16;
+  const int nt0 = first_tile + bx * (BNW / 16) + wn * 4;  // this wave's first 16-row tile of W
 
   floatx4 acc[WM][4];
 #pragma unroll
@@ -185,7 +194,7 @@ void gemm_tiled_kernel(const bf16* __restrict__ A, int64_t lda, const bf16* __re
 #pragma unroll
         for (int j = 0; j < 4; ++j) {
           const int n = (nt0 + j) * 16 + r;
-          if (n < NW) partials[(static_cast<size_t>(blockIdx.z) * M + m) * NW + n] = acc[i][j][v];
+          if (n < NL) partials[(static_cast<size_t>(blockIdx.z) * M + m) * NW + n] = acc[i][j][v];
         }
       }
     return;
@@ -199,7 +208,7 @@ void gemm_tiled_kernel(const bf16* __restrict__ A, int64_t lda, const bf16* __re
 #pragma unroll
       for (int j = 0; j < OUT_TILES; ++j) {
         const int n = EPI == 1 ? (nt0 / 2 + j) * 16 + r : (nt0 + j) * 16 + r;
-        if (n >= N) continue;
+        if (n >= (EPI == 1 ? N : NL)) continue;
         float x;
         if (EPI == 1)
           x = gated_product(act, cap, to_float(float_to_bf16(acc[i][2 * j][v])), to_float(float_to_bf16(acc[i][2 * j + 1][v])));
@@ -290,16 +299,17 @@ __global__ __launch_bounds__(256) void gemm_reduce4_kernel(const float* __restri
 
 template <int WM, int EPI, int WAVES_N>
 static void launch(const bf16* A, int64_t lda, const bf16* W, void* C, int c_dtype, int64_t ldc, int M, int N, int K,
-                   float cap, int act, int ks, float* partials, hipStream_t stream) {
+                   float cap, int act, int ks, float* partials, Sections sec, hipStream_t stream) {
   constexpr int BM = (4 / WAVES_N) * WM * 16, BNW = WAVES_N * 64;
   const int NW = EPI == 1 ? 2 * ((N + 15) / 16) * 16 : N;
-  const dim3 grid((NW + BNW - 1) / BNW, (M + BM - 1) / BM, ks);
+  const int whole = sec.n_step > 0 ? (NW - 1) / sec.n_step : 0;   // sections before the last one
+  const dim3 grid(whole * ((sec.n_step + BNW - 1) / BNW) + (NW - whole * sec.n_step + BNW - 1) / BNW, (M + BM - 1) / BM, ks);
   if (K % BK == 0)
     gemm_tiled_kernel<WM, EPI, WAVES_N, false><<<grid, 256, 0, stream>>>(A, lda, W, C, c_dtype, ldc, M, N, K, (K + 31) / 32,
-                                                                         cap, act, partials);
+                                                                         cap, act, partials, sec);
   else
     gemm_tiled_kernel<WM, EPI, WAVES_N, true><<<grid, 256, 0, stream>>>(A, lda, W, C, c_dtype, ldc, M, N, K, (K + 31) / 32,
-                                                                        cap, act, partials);
+                                                                        cap, act, partials, sec);
   if (ks > 1) gemm_sum_partials(partials, ks, C, c_dtype, ldc, M, N, NW, EPI, act, cap, stream);
 }
 
@@ -350,7 +360,7 @@ bool gemm_tiled_takes(int M, int N, int K, int64_t lda, const void* A, const voi
 
 // ksplit > 0 fixes the number of cuts of K.
 int gemm_tiled(const void* A, int64_t lda, const void* W, void* C, int c_dtype, int64_t ldc, int M, int N, int K,
-               int epi, int act, float cap, int ksplit, void* workspace, size_t workspace_bytes, hipStream_t stream) {
+               int epi, int act, float cap, int ksplit, void* workspace, size_t workspace_bytes, hipStream_t stream, Sections sec) {
   const bf16* a = static_cast<const bf16*>(A);
   const bf16* w = static_cast<const bf16*>(W);
   float* ws = static_cast<float*>(workspace);
@@ -379,9 +389,9 @@ int gemm_tiled(const void* A, int64_t lda, const void* W, void* C, int c_dtype, 
   while (ks > 1 && (ws == nullptr || static_cast<size_t>(ks) * M * NW * sizeof(float) > workspace_bytes)) --ks;
 #define SA_TILED(WM, WN)                                                                                      \
   do {                                                                                                        \
-    if (epi == 1) tiled::launch<WM, 1, WN>(a, lda, w, C, c_dtype, ldc, M, N, K, cap, act, ks, ws, stream);      \
-    else if (epi == 2) tiled::launch<WM, 2, WN>(a, lda, w, C, c_dtype, ldc, M, N, K, cap, act, ks, ws, stream); \
-    else tiled::launch<WM, 0, WN>(a, lda, w, C, c_dtype, ldc, M, N, K, cap, act, ks, ws, stream);               \
+    if (epi == 1) tiled::launch<WM, 1, WN>(a, lda, w, C, c_dtype, ldc, M, N, K, cap, act, ks, ws, sec, stream);      \
+    else if (epi == 2) tiled::launch<WM, 2, WN>(a, lda, w, C, c_dtype, ldc, M, N, K, cap, act, ks, ws, sec, stream); \
+    else tiled::launch<WM, 0, WN>(a, lda, w, C, c_dtype, ldc, M, N, K, cap, act, ks, ws, sec, stream);               \
   } while (0)
   if (few) SA_TILED(4, 4);
   else SA_TILED(4, 2);

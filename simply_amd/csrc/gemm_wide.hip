@@ -68,7 +68,7 @@ template <int WM, int WN, int WAVES_M, int EPI, int NSTAGE, int WAVES>
 __global__ __launch_bounds__(WAVES * 64) void gemm_wide_kernel(const bf16* __restrict__ A, int64_t lda,
                                                         const bf16* __restrict__ W, bf16* __restrict__ C, int64_t ldc,
                                                         int M, int N, int K, int chunks, int act, float limit,
-                                                        float* __restrict__ partials) {
+                                                        float* __restrict__ partials, Sections sec) {
   constexpr int WAVES_N = WAVES / WAVES_M;
   constexpr int MT = WAVES_M * WM, NT = WAVES_N * WN;  // 16-row tiles of A and of W per workgroup
   constexpr int BM = MT * 16;
@@ -110,8 +110,18 @@ __global__ __launch_bounds__(WAVES * 64) void gemm_wide_kernel(const bf16* __res
   A += static_cast<size_t>(slab0) * BK;
   const int m_base = by * BM;
   const int NW = EPI == 1 ? 2 * ((N + 15) / 16) * 16 : N;
-  const int ntiles = (NW + 15) / 16;
-  const int nt_base = bx * NT;
+  // several products at once: which section this workgroup is in, its columns of A, its rows of W
+  int first_tile = 0, NL = NW;   // the section's first 16-row tile of W and the end of its rows
+  if (sec.n_step > 0) {
+    constexpr int BNW = NT * 16;
+    const int per = (sec.n_step + BNW - 1) / BNW, s = bx / per;
+    bx -= s * per;
+    first_tile = s * (sec.n_step / 16);
+    A += static_cast<size_t>(s) * sec.a_step;
+    NL = (s + 1) * sec.n_step < NW ? (s + 1) * sec.n_step : NW;
+  }
+  const int ntiles = (NL + 15) / 16;
+  const int nt_base = first_tile + bx * NT;
 
   // ---- what this wave copies of every slab: KiB blocks wave + WAVES i of A and of W.
   // A block b is rows 8 (b % 2) .. + 8 of tile b / 2, all 64 columns of the slab: eight lanes per row read its 128
@@ -268,7 +278,7 @@ __global__ __launch_bounds__(WAVES * 64) void gemm_wide_kernel(const bf16* __res
 #pragma unroll
       for (int j = 0; j < WN; ++j) {
         const int n = (nt_base + wn * WN + j) * 16 + quad * 4;
-        if (n < N) *reinterpret_cast<floatx4*>(p_row + n) = acc[i][j];
+        if (n < NL) *reinterpret_cast<floatx4*>(p_row + n) = acc[i][j];
       }
       continue;
     }
@@ -278,7 +288,7 @@ __global__ __launch_bounds__(WAVES * 64) void gemm_wide_kernel(const bf16* __res
     for (int j = 0; j < OUT; ++j) {
       const int tile = EPI == 1 ? (nt_base + wn * WN) / 2 + j : nt_base + wn * WN + j;
       const int n = tile * 16 + quad * 4;
-      if (n >= N) continue;
+      if (n >= (EPI == 1 ? N : NL)) continue;
       float x[4];
 #pragma unroll
       for (int v = 0; v < 4; ++v) {
@@ -300,19 +310,20 @@ __global__ __launch_bounds__(WAVES * 64) void gemm_wide_kernel(const bf16* __res
 
 template <int WM, int WN, int WAVES_M, int NSTAGE, int WAVES = 8>
 static void launch(const bf16* A, int64_t lda, const bf16* W, bf16* C, int64_t ldc, int M, int N, int K, int epi,
-                   int act, float limit, int ks, float* partials, hipStream_t stream) {
+                   int act, float limit, int ks, float* partials, bool raw, Sections sec, hipStream_t stream) {
   constexpr int BM = WAVES_M * WM * 16, BNW = (WAVES / WAVES_M) * WN * 16;
   const int NW = epi == 1 ? 2 * ((N + 15) / 16) * 16 : N;
-  const dim3 grid((NW + BNW - 1) / BNW, (M + BM - 1) / BM, ks);
+  const int whole = sec.n_step > 0 ? (NW - 1) / sec.n_step : 0;   // sections before the last one
+  const dim3 grid(whole * ((sec.n_step + BNW - 1) / BNW) + (NW - whole * sec.n_step + BNW - 1) / BNW, (M + BM - 1) / BM, ks);
   if (epi == 1)
     gemm_wide_kernel<WM, WN, WAVES_M, 1, NSTAGE, WAVES><<<grid, WAVES * 64, 0, stream>>>(A, lda, W, C, ldc, M, N, K, K / 32,
-                                                                                         act, limit, nullptr);
-  else if (ks > 1)
+                                                                                         act, limit, nullptr, sec);
+  else if (raw)
     gemm_wide_kernel<WM, WN, WAVES_M, 3, NSTAGE, WAVES><<<grid, WAVES * 64, 0, stream>>>(A, lda, W, C, ldc, M, N, K, K / 32,
-                                                                                         act, limit, partials);
+                                                                                         act, limit, partials, sec);
   else
     gemm_wide_kernel<WM, WN, WAVES_M, 0, NSTAGE, WAVES><<<grid, WAVES * 64, 0, stream>>>(A, lda, W, C, ldc, M, N, K, K / 32,
-                                                                                         act, limit, nullptr);
+                                                                                         act, limit, nullptr, sec);
 }
 
 }  // namespace wide
@@ -320,7 +331,8 @@ static void launch(const bf16* A, int64_t lda, const bf16* W, bf16* C, int64_t l
 bool gemm_wide_takes(int M, int N, int K, int64_t lda, int64_t ldc, const void* A, const void* W, const void* W2,
                      const void* C, int c_dtype, int epi, int packed) {
   auto aligned = [](const void* p, uintptr_t a) { return (reinterpret_cast<uintptr_t>(p) & (a - 1)) == 0; };
-  return packed && W2 == nullptr && (epi == 0 || epi == 1) && c_dtype == kBF16 && M >= 1 && K % wide::BK == 0 &&
+  return packed && W2 == nullptr && (epi == 0 || epi == 1) && M >= 1 &&
+         (c_dtype == kBF16 || (c_dtype == kF32 && epi == 0 && ldc == N && M > 64 && N >= 512 && aligned(C, 16))) && K % wide::BK == 0 &&
          N % 4 == 0 && lda % 8 == 0 && ldc % 4 == 0 && aligned(A, 16) && aligned(W, 16) && aligned(C, 8) &&
          static_cast<int64_t>(M) * lda < (int64_t{1} << 31);  // byte offsets of rows are kept in 32 bits
 }
@@ -405,7 +417,8 @@ static double plan_shape(int M, int N, int K, int epi, bool have_workspace, size
 // ks > 1 cuts K over that many workgroups per tile (no epilogue only; the partial tiles go through `workspace`,
 // which must hold ks * M * N floats).
 int gemm_wide(const void* A, int64_t lda, const void* W, void* C, int64_t ldc, int M, int N, int K, int epi, int act,
-              float limit, int shape, int ks, void* workspace, size_t workspace_bytes, hipStream_t stream, int* planes_left) {
+              float limit, int shape, int ks, void* workspace, size_t workspace_bytes, hipStream_t stream, int* planes_left, int c_dtype,
+              Sections sec) {
   if (ks < 1) ks = 1;
   if (ks > K / wide::BK) ks = K / wide::BK;
   if (ks > 1 && (epi != 0 || workspace == nullptr || static_cast<size_t>(ks) * M * N * sizeof(float) > workspace_bytes)) {
@@ -417,22 +430,25 @@ int gemm_wide(const void* A, int64_t lda, const void* W, void* C, int64_t ldc, i
   const bf16* w = static_cast<const bf16*>(W);
   bf16* c = static_cast<bf16*>(C);
   if (shape == 0) plan_shape(M, N, K, epi, ws != nullptr, workspace_bytes, shape, ks);
+  // 32-bit results: the cuts' partial sums as they are, of one cut straight into C (whose rows are contiguous)
+  const bool raw = ks > 1 || c_dtype == kF32;
+  float* to = ks > 1 ? ws : static_cast<float*>(C);
   switch (shape) {
-    case 2256192: wide::launch<4, 6, 4, 2>(a, lda, w, c, ldc, M, N, K, epi, act, limit, ks, ws, stream); break;
-    case 3256128: wide::launch<4, 4, 4, 3>(a, lda, w, c, ldc, M, N, K, epi, act, limit, ks, ws, stream); break;
-    case 3128256: wide::launch<4, 4, 2, 3>(a, lda, w, c, ldc, M, N, K, epi, act, limit, ks, ws, stream); break;
-    case 3192128: wide::launch<3, 4, 4, 3>(a, lda, w, c, ldc, M, N, K, epi, act, limit, ks, ws, stream); break;
-    case 2128192: wide::launch<4, 6, 2, 2, 4>(a, lda, w, c, ldc, M, N, K, epi, act, limit, ks, ws, stream); break;  // two workgroups per CU
+    case 2256192: wide::launch<4, 6, 4, 2>(a, lda, w, c, ldc, M, N, K, epi, act, limit, ks, to, raw, sec, stream); break;
+    case 3256128: wide::launch<4, 4, 4, 3>(a, lda, w, c, ldc, M, N, K, epi, act, limit, ks, to, raw, sec, stream); break;
+    case 3128256: wide::launch<4, 4, 2, 3>(a, lda, w, c, ldc, M, N, K, epi, act, limit, ks, to, raw, sec, stream); break;
+    case 3192128: wide::launch<3, 4, 4, 3>(a, lda, w, c, ldc, M, N, K, epi, act, limit, ks, to, raw, sec, stream); break;
+    case 2128192: wide::launch<4, 6, 2, 2, 4>(a, lda, w, c, ldc, M, N, K, epi, act, limit, ks, to, raw, sec, stream); break;  // two workgroups per CU
     // small tiles, for products of a few hundred rows whose large tiles would leave most CUs idle (two or more
     // workgroups per CU fit: 36 to 72 KiB of LDS each)
-    case 3128128: wide::launch<2, 4, 4, 3>(a, lda, w, c, ldc, M, N, K, epi, act, limit, ks, ws, stream); break;
-    case 3128064: wide::launch<2, 2, 4, 3>(a, lda, w, c, ldc, M, N, K, epi, act, limit, ks, ws, stream); break;
-    case 3064128: wide::launch<1, 4, 4, 3>(a, lda, w, c, ldc, M, N, K, epi, act, limit, ks, ws, stream); break;
-    case 3064064: wide::launch<1, 2, 4, 3>(a, lda, w, c, ldc, M, N, K, epi, act, limit, ks, ws, stream); break;
-    case 6064064: wide::launch<1, 2, 4, 6>(a, lda, w, c, ldc, M, N, K, epi, act, limit, ks, ws, stream); break;
-    case 5128064: wide::launch<2, 2, 4, 5>(a, lda, w, c, ldc, M, N, K, epi, act, limit, ks, ws, stream); break;
-    case 4128128: wide::launch<2, 4, 4, 4>(a, lda, w, c, ldc, M, N, K, epi, act, limit, ks, ws, stream); break;
-    case 6064128: wide::launch<1, 4, 4, 6>(a, lda, w, c, ldc, M, N, K, epi, act, limit, ks, ws, stream); break;
+    case 3128128: wide::launch<2, 4, 4, 3>(a, lda, w, c, ldc, M, N, K, epi, act, limit, ks, to, raw, sec, stream); break;
+    case 3128064: wide::launch<2, 2, 4, 3>(a, lda, w, c, ldc, M, N, K, epi, act, limit, ks, to, raw, sec, stream); break;
+    case 3064128: wide::launch<1, 4, 4, 3>(a, lda, w, c, ldc, M, N, K, epi, act, limit, ks, to, raw, sec, stream); break;
+    case 3064064: wide::launch<1, 2, 4, 3>(a, lda, w, c, ldc, M, N, K, epi, act, limit, ks, to, raw, sec, stream); break;
+    case 6064064: wide::launch<1, 2, 4, 6>(a, lda, w, c, ldc, M, N, K, epi, act, limit, ks, to, raw, sec, stream); break;
+    case 5128064: wide::launch<2, 2, 4, 5>(a, lda, w, c, ldc, M, N, K, epi, act, limit, ks, to, raw, sec, stream); break;
+    case 4128128: wide::launch<2, 4, 4, 4>(a, lda, w, c, ldc, M, N, K, epi, act, limit, ks, to, raw, sec, stream); break;
+    case 6064128: wide::launch<1, 4, 4, 6>(a, lda, w, c, ldc, M, N, K, epi, act, limit, ks, to, raw, sec, stream); break;
     default:
       set_error("gemm: unknown wide tile %d", shape);
       return 1;
@@ -443,7 +459,7 @@ int gemm_wide(const void* A, int64_t lda, const void* W, void* C, int64_t ldc, i
     return 0;
   }
   if (ks > 1) {
-    if (gemm_sum_partials(ws, ks, C, kBF16, ldc, M, N, N, 0, 0, 0.f, stream)) return 1;
+    if (gemm_sum_partials(ws, ks, C, c_dtype, ldc, M, N, N, 0, 0, 0.f, stream)) return 1;
     if (epi == 0 && act > 0) return apply_activation(C, kBF16, ldc, M, N, act - 1, stream);   // (the kernels with K cut have no such epilogue)
   }
   return 0;

@@ -35,7 +35,7 @@ extern "C" int sa_version() { return 1; }
 static int gemm_routed(const void* A, int a_dtype, int64_t lda, const void* W, const void* W2, int w_dtype, void* C,
                        int c_dtype, int64_t ldc, int M, int N, int K, int epilogue, float cap, int algo,
                        int packed, int shape, void* workspace, int64_t workspace_bytes, int* planes_left,
-                       hipStream_t stream) {
+                       hipStream_t stream, Sections sec = {}) {
   if (planes_left != nullptr) *planes_left = 1;
   if (M == 0 || N == 0) return 0;
   SA_REQUIRE(M > 0 && N > 0 && K > 0, "gemm: bad sizes M=%d N=%d K=%d", M, N, K);
@@ -63,7 +63,8 @@ static int gemm_routed(const void* A, int a_dtype, int64_t lda, const void* W, c
   const size_t ws_bytes = static_cast<size_t>(workspace_bytes < 0 ? 0 : workspace_bytes);
   // Which of the three bfloat16 kernels take these arguments; a kernel that the caller names must take them.
   const bool skinny_ok = bf16_in && gemm_skinny_takes(M, N, K, lda, A, W, W2);
-  const bool wide_ok = bf16_in && gemm_wide_takes(M, N, K, lda, ldc, A, W, W2, C, c_dtype, epilogue, packed);
+  const bool wide_ok = bf16_in && gemm_wide_takes(M, N, K, lda, ldc, A, W, W2, C, c_dtype, epilogue, packed) &&
+                       (c_dtype == kBF16 || activated == 0);
   const bool tiled_ok = bf16_in && gemm_tiled_takes(M, N, K, lda, A, W, W2, packed);
   SA_REQUIRE(algo != 2 || skinny_ok,
              "gemm: the few-rows kernel takes bfloat16 with M <= 64, K and lda multiples of 8 and 16-byte aligned "
@@ -94,15 +95,17 @@ static int gemm_routed(const void* A, int a_dtype, int64_t lda, const void* W, c
   // (a shape given by the caller for the wide kernel may carry a cut of K in front: cuts * 10000000 + shape)
   if (kernel == 4)
     return gemm_wide(A, lda, W, C, ldc, M, N, K, epilogue, activated ? activated : act, cap, algo == 4 ? shape % 10000000 : 0,
-                     algo == 4 ? shape / 10000000 : 1, workspace, ws_bytes, stream, planes_left);
+                     algo == 4 ? shape / 10000000 : 1, workspace, ws_bytes, stream, planes_left, c_dtype, sec);
   // (the few-rows kernel has the activation in its epilogue too, for bfloat16 results)
   if (kernel == 2 && activated && c_dtype == kBF16)
     return gemm_skinny(A, lda, W, W2, C, c_dtype, ldc, M, N, K, epilogue, activated, cap, packed, shape, stream);
+  SA_REQUIRE(sec.n_step == 0 || kernel == 2 || kernel == 3,
+             "gemm_sections: none of the bfloat16 kernels takes K=%d lda=%lld and these operands", K, (long long)lda);
   int rc;
   if (kernel == 2)
-    rc = gemm_skinny(A, lda, W, W2, C, c_dtype, ldc, M, N, K, epilogue, act, cap, packed, shape, stream);
+    rc = gemm_skinny(A, lda, W, W2, C, c_dtype, ldc, M, N, K, epilogue, act, cap, packed, shape, stream, sec);
   else if (kernel == 3)
-    rc = gemm_tiled(A, lda, W, C, c_dtype, ldc, M, N, K, epilogue, act, cap, shape, workspace, ws_bytes, stream);
+    rc = gemm_tiled(A, lda, W, C, c_dtype, ldc, M, N, K, epilogue, act, cap, shape, workspace, ws_bytes, stream, sec);
   else
     rc = gemm_generic(A, a_dtype, lda, W, W2, w_dtype, C, c_dtype, ldc, M, N, K, epilogue, act, cap, packed, stream);
   if (rc == 0 && activated) rc = apply_activation(C, c_dtype, ldc, M, N, activated - 1, stream);
@@ -114,6 +117,21 @@ extern "C" int sa_gemm(const void* A, int a_dtype, int64_t lda, const void* W, c
                        int packed, int shape, void* workspace, int64_t workspace_bytes, hipStream_t stream) {
   return gemm_routed(A, a_dtype, lda, W, W2, w_dtype, C, c_dtype, ldc, M, N, K, epilogue, cap, algo, packed, shape,
                      workspace, workspace_bytes, nullptr, stream);
+}
+
+extern "C" int sa_gemm_sections(const void* A, int64_t lda, const void* W, void* C, int c_dtype, int64_t ldc, int M, int N,
+                                int K, int n_step, int a_step, void* workspace, int64_t workspace_bytes,
+                                hipStream_t stream) {
+  SA_REQUIRE(n_step > 0 && n_step % 16 == 0 && N > 0, "gemm_sections: sections of %d rows (a multiple of 16)", n_step);
+  const int sections = (N + n_step - 1) / n_step;
+  SA_REQUIRE(a_step >= 0 && lda >= static_cast<int64_t>(sections - 1) * a_step + K,
+             "gemm_sections: rows of %lld do not hold %d sections %d apart", (long long)lda, sections, a_step);
+  SA_REQUIRE(a_step % 8 == 0, "gemm_sections: sections lie a multiple of 8 columns apart");
+  Sections sec;
+  sec.n_step = n_step;
+  sec.a_step = a_step;
+  return gemm_routed(A, kBF16, lda, W, nullptr, kBF16, C, c_dtype, ldc, M, N, K, kEpilogueNone, 0.f, 0, 1, 0, workspace,
+                     workspace_bytes, nullptr, stream, sec);
 }
 
 extern "C" int sa_gemm_plan(int M, int N, int K, int epilogue, int c_dtype, int64_t workspace_bytes, double* us_out) {

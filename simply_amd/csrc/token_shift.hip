@@ -1,7 +1,7 @@
 // What a mixer with a token shift and data-dependent decays reads, and the rows of a looped pass:
 //
 //   token_shift_kernel     out[t, s, :] = h[t] + (h[t - 1] - h[t]) * mu[s, :]   for every stream s of a mixer's input
-//   low_rank_decay_kernel  a[t, c] = exp(-exp(sum_r w[r, c] tanh(p[t, r]) + w0[c]))
+//   low_rank_decay_kernel  a[t, c] = exp(-exp(sum_r w[c, r] tanh(p[t, r]) + w0[c]))
 //   concat_rows_kernel     out[t] = [x[t] | y[t]]
 //
 // A request's tokens of this step are rows first .. first + count - 1 (seq_meta [S, 4]: state slot, first row, count,
@@ -92,9 +92,8 @@ __global__ __launch_bounds__(kShiftThreads) void token_shift_kernel(const T* __r
   }
 }
 
-// A wave takes 64 channels of kDecayTokens tokens: tanh(p) of the tokens goes through LDS, kDecayRank factors at a
-// time, a lane sums its channel for all the tokens in the factors' order.  w is [rank, C]: a wave's loads of a factor
-// are contiguous.
+// 32-bit weights [C, rank], or bfloat16 ones as rows: a wave takes 64 channels of kDecayTokens tokens; tanh(p) of the
+// tokens goes through LDS, kDecayRank factors at a time, a lane sums its channel for all the tokens in the factors' order.
 constexpr int kDecayTokens = 16;
 constexpr int kDecayRank = 64;
 template <typename WT>
@@ -104,7 +103,7 @@ __global__ __launch_bounds__(kWave) void low_rank_decay_kernel(const void* __res
                                                                int rank) {
   __shared__ __align__(16) float ts[kDecayTokens][kDecayRank];
   const int lane = threadIdx.x, c = blockIdx.x * kWave + lane, t0 = blockIdx.y * kDecayTokens;
-  const int cc = c < C ? c : C - 1;
+  const WT* row = w + static_cast<size_t>(c < C ? c : C - 1) * rank;
   float acc[kDecayTokens];
 #pragma unroll
   for (int k = 0; k < kDecayTokens; ++k) acc[k] = 0.f;
@@ -116,18 +115,10 @@ __global__ __launch_bounds__(kWave) void low_rank_decay_kernel(const void* __res
     }
     __syncthreads();
     const int rn = rank - r0 < kDecayRank ? rank - r0 : kDecayRank;
-    for (int r = 0; r < rn; r += 4) {
-      float wv[4];
+    for (int r = 0; r < rn; ++r) {
+      const float wv = to_float(row[r0 + r]);
 #pragma unroll
-      for (int i = 0; i < 4; ++i) wv[i] = r + i < rn ? to_float(w[static_cast<size_t>(r0 + r + i) * C + cc]) : 0.f;
-#pragma unroll
-      for (int k = 0; k < kDecayTokens; ++k) {
-        const float4 x = *reinterpret_cast<const float4*>(&ts[k][r]);
-        acc[k] = fmaf(x.x, wv[0], acc[k]);
-        acc[k] = fmaf(x.y, wv[1], acc[k]);
-        acc[k] = fmaf(x.z, wv[2], acc[k]);
-        acc[k] = fmaf(x.w, wv[3], acc[k]);
-      }
+      for (int k = 0; k < kDecayTokens; ++k) acc[k] = fmaf(ts[k][r], wv, acc[k]);
     }
   }
   if (c >= C) return;
@@ -135,6 +126,82 @@ __global__ __launch_bounds__(kWave) void low_rank_decay_kernel(const void* __res
 #pragma unroll
   for (int k = 0; k < kDecayTokens; ++k)
     if (t0 + k < T) out[static_cast<size_t>(t0 + k) * C + c] = expf(-expf(acc[k] + base));
+}
+
+// bfloat16 weights in MFMA operand tiles ([C / 16][rank / 32][64][8], zeros beyond C and rank): a wave takes 16 tokens and
+// `tiles` tiles of 16 channels.  tanh(p) goes in as three bfloat16 numbers (its rounding, the rounding of what that leaves,
+// and the rest: all 24 bits), so that the sum is that of 32-bit factors; a lane computes the eight entries of every 32
+// that its operand holds.
+typedef __attribute__((__vector_size__(8 * sizeof(__bf16)))) __bf16 bf16x8;
+typedef __attribute__((__vector_size__(4 * sizeof(float)))) float floatx4;
+constexpr int kDecayChunks = 2;   // chunks of 32 factors whose tanh a wave holds at a time
+__global__ __launch_bounds__(256) void low_rank_decay_tiled_kernel(const void* __restrict__ p, int p_dtype, int64_t p_stride,
+                                                                   const bf16* __restrict__ w, const void* __restrict__ w0,
+                                                                   int w0_dtype, float* __restrict__ out, int T, int C,
+                                                                   int rank, int tiles) {
+  const int lane = threadIdx.x % kWave, wave = threadIdx.x / kWave;
+  const int r = lane % 16, kq = lane / 16;
+  const int t = blockIdx.y * 16 + r, tc = t < T ? t : T - 1;
+  const int chunks = (rank + 31) / 32, all = (C + 15) / 16;
+  const int n0 = (blockIdx.x * 4 + wave) * tiles, n1 = n0 + tiles < all ? n0 + tiles : all;
+  if (n0 >= all) return;   // (a whole wave; there are no barriers)
+  // one pass holds the sums of up to 4 channel tiles
+  for (int nb = n0; nb < n1; nb += 4) {
+    floatx4 acc[4];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) acc[i] = floatx4{0.f, 0.f, 0.f, 0.f};
+    for (int c0 = 0; c0 < chunks; c0 += kDecayChunks) {
+      bf16x8 wv[4][kDecayChunks];
+#pragma unroll
+      for (int i = 0; i < 4; ++i)
+#pragma unroll
+        for (int u = 0; u < kDecayChunks; ++u) {
+          const int tile = nb + i < n1 ? nb + i : n1 - 1, ch = c0 + u < chunks ? c0 + u : chunks - 1;
+          wv[i][u] = *reinterpret_cast<const bf16x8*>(w + (static_cast<size_t>(tile) * chunks + ch) * 512 + lane * 8);
+        }
+#pragma unroll
+      for (int u = 0; u < kDecayChunks; ++u) {
+        if (c0 + u >= chunks) break;   // (uniform)
+        bf16x8 hi, mid, lo;
+#pragma unroll
+        for (int j = 0; j < 8; ++j) {
+          const int k = (c0 + u) * 32 + kq * 8 + j;
+          const float x = k < rank ? load_f(p, p_dtype, static_cast<size_t>(tc) * p_stride + k) : 0.f;
+          // tanh by the hardware's exponential: 1 - 2 / (e^(2x) + 1), and x (1 - x^2 / 3) where that cancels
+          const float y = 1.f - 2.f * __builtin_amdgcn_rcpf(__expf(2.f * x) + 1.f);
+          const float th = fabsf(x) < 0.02f ? x * fmaf(x * x, -1.f / 3.f, 1.f) : y;
+          hi[j] = static_cast<__bf16>(th);
+          const float rest = th - static_cast<float>(hi[j]);
+          mid[j] = static_cast<__bf16>(rest);
+          lo[j] = static_cast<__bf16>(rest - static_cast<float>(mid[j]));
+        }
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          acc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wv[i][u], hi, acc[i], 0, 0, 0);
+          acc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wv[i][u], mid, acc[i], 0, 0, 0);
+          acc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wv[i][u], lo, acc[i], 0, 0, 0);
+        }
+      }
+    }
+    // lane: token r, channels 4 kq .. of every tile
+    if (t >= T) continue;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      if (nb + i >= n1) break;
+      const int c = (nb + i) * 16 + kq * 4;
+      float* dst = out + static_cast<size_t>(t) * C + c;
+      float a[4];
+#pragma unroll
+      for (int v = 0; v < 4; ++v) a[v] = c + v < C ? __expf(-__expf(acc[i][v] + load_f(w0, w0_dtype, c + v))) : 0.f;
+      if (c + 4 <= C && C % 4 == 0) {
+        *reinterpret_cast<float4*>(dst) = float4{a[0], a[1], a[2], a[3]};
+      } else {
+#pragma unroll
+        for (int v = 0; v < 4; ++v)
+          if (c + v < C) dst[v] = a[v];
+      }
+    }
+  }
 }
 
 __global__ __launch_bounds__(256) void concat_rows_kernel(const float* __restrict__ x, const float* __restrict__ y,
@@ -183,14 +250,25 @@ extern "C" int sa_token_shift(const void* h, int dtype, int64_t h_stride, const 
   return check_launch("token_shift");
 }
 
-extern "C" int sa_low_rank_decay(const void* p, int p_dtype, int64_t p_stride, const void* w, int w_dtype, const void* w0,
-                                 int w0_dtype, float* out, int T, int C, int rank, hipStream_t stream) {
+extern "C" int sa_low_rank_decay(const void* p, int p_dtype, int64_t p_stride, const void* w, int w_dtype, int tiled,
+                                 const void* w0, int w0_dtype, float* out, int T, int C, int rank, hipStream_t stream) {
   if (T == 0) return 0;
   SA_REQUIRE(T > 0 && C > 0 && rank > 0 && p_stride >= rank, "low_rank_decay: bad sizes T=%d C=%d rank=%d", T, C, rank);
   SA_REQUIRE(p != nullptr && w != nullptr && w0 != nullptr && out != nullptr, "low_rank_decay: a null pointer");
   SA_REQUIRE((w_dtype == kF32 || w_dtype == kBF16) && (p_dtype == kF32 || p_dtype == kBF16) &&
                  (w0_dtype == kF32 || w0_dtype == kBF16),
              "low_rank_decay: unknown dtype");
+  if (tiled) {
+    SA_REQUIRE(w_dtype == kBF16, "low_rank_decay: tiled weights are bfloat16");
+    // a wave takes one tile of channels while there are few tokens, four when there are many (their tanh is shared)
+    const int tt = (T + 15) / 16, all = (C + 15) / 16;
+    const int tiles = static_cast<int64_t>(tt) * all >= 4096 ? 4 : 1;
+    const dim3 grid((all + 4 * tiles - 1) / (4 * tiles), tt);
+    SA_REQUIRE(grid.y <= 65535, "low_rank_decay: too many tokens");
+    low_rank_decay_tiled_kernel<<<grid, 256, 0, stream>>>(p, p_dtype, p_stride, static_cast<const bf16*>(w), w0, w0_dtype, out,
+                                                          T, C, rank, tiles);
+    return check_launch("low_rank_decay");
+  }
   const dim3 grid((C + kWave - 1) / kWave, (T + kDecayTokens - 1) / kDecayTokens);
   SA_REQUIRE(grid.y <= 65535, "low_rank_decay: too many tokens");
   if (w_dtype == kBF16)

@@ -478,32 +478,46 @@ def gemm(a: torch.Tensor, w: "torch.Tensor | TiledWeight", *, w2: "torch.Tensor 
 
 
 class SectionedWeight:
-    """Weights [N, K] of several products that are run as one: section s of the result, columns s N .. (s + 1) N, is
-    section s of the input rows, columns s K .. (s + 1) K, times the s-th weight."""
+    """Weights of several products that are run as one: section s of the result, columns s N .. (s + 1) N, is section s of
+    the input rows, columns s K .. (s + 1) K, times the s-th weight [N, K]; the last weight may have fewer rows.
+    bfloat16 weights on the GPU whose N is a multiple of 16 lie in one tiled weight (`fused`), of which `parts` are views."""
 
-    def __init__(self, parts: list, rows: int, cols: int):
-        self.parts, self.rows, self.cols = parts, rows, cols   # (parts: one product weight per section)
-
-    @classmethod
-    def of(cls, ws) -> "SectionedWeight":
+    def __init__(self, ws):
         from .packing import pack_tiles
 
         ws = list(ws)
-        N, K = ws[0].shape
-        if any(tuple(w.shape) != (N, K) or w.dtype != ws[0].dtype for w in ws):
+        self.step, self.cols = ws[0].shape
+        self.rows = sum(w.shape[0] for w in ws)
+        if any(w.dim() != 2 or w.shape[1] != self.cols or w.dtype != ws[0].dtype for w in ws) \
+                or any(w.shape[0] != self.step for w in ws[:-1]) or not 0 < ws[-1].shape[0] <= self.step:
             raise KernelError("SectionedWeight: the sections' weights differ in shape or type")
         tiled = ws[0].dtype == torch.bfloat16 and ws[0].is_cuda
-        return cls([pack_tiles(w.contiguous()) if tiled else w.contiguous() for w in ws], N, K)
+        self.fused = None
+        if tiled and self.step % 16 == 0:
+            self.fused = pack_tiles(torch.cat(ws).contiguous())
+            t = self.step // 16
+            self.parts = [TiledWeight(self.fused.data[s * t:s * t + -(-w.shape[0] // 16)], w.shape[0], self.cols)
+                          for s, w in enumerate(ws)]
+        else:
+            self.parts = [pack_tiles(w.contiguous()) if tiled else w.contiguous() for w in ws]
 
 
 def gemm_sections(a: torch.Tensor, w: SectionedWeight) -> torch.Tensor:
-    """[T, S * N] from rows a [T, S * K] (a view is fine): every section's columns times its own weight."""
-    S, N, K = len(w.parts), w.rows, w.cols
+    """[T, w.rows] from rows a [T, sections * K] (a view is fine): every section's columns times its own weight."""
+    S, N, K = len(w.parts), w.step, w.cols
     if a.dim() != 2 or a.shape[1] != S * K:
         raise KernelError(f"gemm_sections: rows {tuple(a.shape)} for {S} sections of {K}")
-    out = torch.empty((a.shape[0], S * N), dtype=a.dtype, device=a.device)
+    out = torch.empty((a.shape[0], w.rows), dtype=a.dtype, device=a.device)
+    lda = _rows(a, "gemm_sections: a")
+    if w.fused is not None and a.dtype == torch.bfloat16 and K % 8 == 0 and lda % 8 == 0 and a.data_ptr() % 16 == 0 \
+            and a.shape[0] * lda < 1 << 30:
+        _dev(a, w.fused.data)
+        ws = _workspace(a.device)
+        _lib.call("sa_gemm_sections", _ptr(a), lda, _ptr(w.fused.data), _ptr(out), _code(out), out.stride(0), a.shape[0],
+                  w.rows, K, N, K, _ptr(ws), ws.numel(), _stream())
+        return out
     for s, part in enumerate(w.parts):
-        gemm(a[:, s * K:(s + 1) * K], part, out=out[:, s * N:(s + 1) * N])
+        gemm(a[:, s * K:(s + 1) * K], part, out=out[:, s * N:s * N + part.shape[0]])
     return out
 
 
@@ -1627,17 +1641,20 @@ def token_shift(h: torch.Tensor, mu: torch.Tensor, tails: torch.Tensor, seq_meta
     return out
 
 
-def low_rank_decay(p: torch.Tensor, w: torch.Tensor, base: torch.Tensor) -> torch.Tensor:
-    """float32 [T, C]: exp(-exp(tanh(p) w + base)) with p [T, rank], w [rank, C], base [C]; all of it 32-bit."""
-    _dev(p, w, base)
+def low_rank_decay(p: torch.Tensor, w: "torch.Tensor | TiledWeight", base: torch.Tensor) -> torch.Tensor:
+    """float32 [T, C]: exp(-exp(w tanh(p) + base)) with p [T, rank], w [C, rank] (tiled if bfloat16 on the GPU), base [C].
+    All of it is 32-bit: where the matrix cores take bfloat16 operands, tanh is three of them."""
+    tiled = isinstance(w, TiledWeight)
+    data = w.data if tiled else w
+    _dev(p, data, base)
     stride = _rows(p, "low_rank_decay: p")
     T, rank = p.shape
-    if w.dim() != 2 or w.shape[0] != rank or not w.is_contiguous() or base.numel() != w.shape[1] or not base.is_contiguous():
+    C = w.shape[0]
+    if w.shape[1] != rank or not data.is_contiguous() or base.numel() != C or not base.is_contiguous():
         raise KernelError(f"low_rank_decay: w {tuple(w.shape)} and base {tuple(base.shape)} for {rank} factors")
-    C = w.shape[1]
     out = torch.empty((T, C), dtype=torch.float32, device=p.device)
-    _lib.call("sa_low_rank_decay", _ptr(p), _code(p), stride, _ptr(w), _code(w), _ptr(base), _code(base), _ptr(out), T, C,
-              rank, _stream())
+    _lib.call("sa_low_rank_decay", _ptr(p), _code(p), stride, _ptr(data), _code(data), int(tiled), _ptr(base), _code(base),
+              _ptr(out), T, C, rank, _stream())
     return out
 
 

@@ -26,7 +26,7 @@ class WKV(Mixer):
         self.hidden_size, self.num_heads, self.head_dim = int(hidden_size), int(num_heads), int(head_dim)
         self.decay_rank, self.norm_eps = int(decay_rank), float(norm_eps)
         self.state_words = self.num_heads * self.head_dim * self.head_dim
-        self.mu = self.in_proj = self.decay_in = self.decay_out = self.decay_base = self.bonus = self.norm = self.o_proj = None
+        self.mu = self.in_proj = self.decay_out = self.decay_base = self.bonus = self.norm = self.o_proj = None
 
     def param_specs(self):
         D, H, d, R = self.hidden_size, self.num_heads, self.head_dim, self.decay_rank
@@ -40,10 +40,12 @@ class WKV(Mixer):
     def load(self, tensors):
         t = tensors
         self.mu = torch.stack([t["mu_" + s].to(t["mu_r"].dtype) for s in self.STREAMS]).contiguous()
-        # r, k, v and the gate: one product whose blocks of outputs read blocks of the mixes
-        self.in_proj = ops.SectionedWeight.of([t[s + "_proj"] for s in "rkvg"])
-        self.decay_in = as_product_weight(t["decay_in"])
-        self.decay_out = t["decay_out"].t().contiguous()          # [rank, channels]: what the decay's kernel reads
+        # r, k, v, the gate and the decay's first factor: products whose blocks of outputs read blocks of the mixes, run
+        # as one where the decay's rank is not larger than the heads
+        rkvg = [t[s + "_proj"] for s in "rkvg"]
+        self.decay_in = None if self.decay_rank <= rkvg[0].shape[0] else as_product_weight(t["decay_in"])
+        self.in_proj = ops.SectionedWeight(rkvg + ([t["decay_in"]] if self.decay_in is None else []))
+        self.decay_out = as_product_weight(t["decay_out"])
         self.decay_base, self.norm = t["decay_base"].contiguous(), t["norm"].contiguous()
         self.bonus = t["bonus"].reshape(-1).contiguous()
         self.o_proj = as_product_weight(t["o_proj"])
@@ -57,10 +59,14 @@ class WKV(Mixer):
         D, H, d = self.hidden_size, self.num_heads, self.head_dim
         C = H * d
         mixes = ops.token_shift(x, self.mu, cache.state[:, self.state_words:], ctx.seq_meta, ctx.num_seqs, ctx.max_q_len)
-        proj = ops.gemm_sections(mixes[:, :4 * D], self.in_proj)                      # [T, r | k | v | gate]
-        decay = ops.low_rank_decay(ops.gemm(mixes[:, 4 * D:], self.decay_in), self.decay_out, self.decay_base)
+        if self.decay_in is None:
+            proj = ops.gemm_sections(mixes, self.in_proj)                             # [T, r | k | v | gate | decay's factor]
+            low = proj[:, 4 * C:]
+        else:
+            proj, low = ops.gemm_sections(mixes[:, :4 * D], self.in_proj), ops.gemm(mixes[:, 4 * D:], self.decay_in)
+        decay = ops.low_rank_decay(low, self.decay_out, self.decay_base)
         o = ops.linear_state(proj, 0, C, 2 * C, 1.0, decay, False, H, d, d, False, cache.state, ctx.seq_meta, ctx.num_seqs,
                              bonus=self.bonus)
-        z = ops.gated_heads(o, proj[:, 3 * C:], H, d, kind=ops.GATE_SILU, weight=self.norm, eps=self.norm_eps,
+        z = ops.gated_heads(o, proj[:, 3 * C:4 * C], H, d, kind=ops.GATE_SILU, weight=self.norm, eps=self.norm_eps,
                             out_dtype=ctx.dtype)
         return ops.gemm(z, self.o_proj)

@@ -872,7 +872,7 @@ def token_shift(h, mu, tails, seq_meta, num_seqs, max_q_len):
 
 
 def low_rank_decay(p, w, base):
-    return torch.exp(-torch.exp(torch.tanh(_f(p)) @ _f(w) + _f(base))).to(torch.float32)
+    return torch.exp(-torch.exp(torch.tanh(_f(p)) @ _f(w).T + _f(base))).to(torch.float32)
 
 
 def concat_rows(x, y, out_dtype):
@@ -880,5 +880,5 @@ def concat_rows(x, y, out_dtype):
 
 
 def gemm_sections(a, w):
-    S, N, K = len(w.parts), w.rows, w.cols
+    S, K = len(w.parts), w.cols
     return torch.cat([gemm(a[:, s * K:(s + 1) * K], w.parts[s]) for s in range(S)], dim=1)
