@@ -30,13 +30,7 @@ def cpu_ops(monkeypatch):
     import torch_ops
     from simply_amd.kernels import ops
 
-    for name in ("embed", "rmsnorm", "add_rmsnorm", "rope_cache_write", "rope", "gather_rows", "fill_", "gemm",
-                 "paged_attention", "sample", "score", "decode_attention_takes", "paged_attention_sink",
-                 "residual_add_norm", "gated_heads", "activation_", "qk_norm_rope_cache_write", "short_conv_silu",
-                 "delta_prepare", "delta_inputs", "delta_rule", "embed_sum", "token_gate_", "bias_add_", "weighted_sum",
-                 "exp_gates", "linear_state", "normalized_readout", "route", "routed_experts", "residual_add_next_norm",
-                 "paged_attention_maps", "attention_maps_units_takes", "norm_rope_cache_write", "short_conv", "head_product", "rglru_scan",
-                 "attention_inputs", "route_choice", "token_shift", "low_rank_decay", "concat_rows", "gemm_sections"):
+    for name in torch_ops.STAND_INS:
         monkeypatch.setattr(ops, name, getattr(torch_ops, name))
     return torch_ops
 
