@@ -723,44 +723,45 @@ def test_gemm_dispatch_of_few_rows_against_a_long_k(M, N, K):
     assert not out[:, N:].any()
 
 
-@pytest.mark.parametrize("activation", [0, 1, 2, 3])
+@pytest.mark.parametrize("activation", [0, 1, 2, 3, 4])
 @pytest.mark.parametrize("M", [5, 16, 40, 300])
 def test_gated_activations_in_every_product_kernel(M, activation):
     """act(a.Wg^T) * (a.Wu^T) for the three activations that the reference registers (tanh-gelu, silu, squared relu:
-    simply/model_lib.py:93-104) and for the exact GELU, in each kernel that has the gated epilogue: the 32-bit one, the few-rows one, the
-    one with the norms in front, the tiled one with and without its sum kernel, the wide one."""
+    simply/model_lib.py:93-104) and for the exact GELU, and the rule that clamps both factors, in each kernel that has the gated epilogue: the
+    32-bit one, the few-rows one, the one with the norms in front, the tiled one with and without its sum kernel, the wide one."""
     from simply_amd.kernels import ops
     from simply_amd.kernels.packing import pack_gate_up
     N, K = 200, 256
     a = rand((M, K), torch.bfloat16, 130, 1.5)
     w, w2 = rand((N, K), torch.bfloat16, 131, 0.08), rand((N, K), torch.bfloat16, 132, 0.08)
     tg = pack_gate_up(w, w2)
-    want = ref.gemm(a, w, w2=w2, activation=activation).float()
+    kw = {"activation": activation, **({"limit": 0.9} if activation == 4 else {})}
+    want = ref.gemm(a, w, w2=w2, **kw).float()
     assert want.abs().max() > 0.5
     if activation in (1, 2):   # (the exact GELU is within a bfloat16 step of the tanh form)
         assert not torch.allclose(want, ref.gemm(a, w, w2=w2).float(), rtol=2e-2, atol=2e-2)   # the activations differ
     # (the squared relu doubles the relative error of its argument: one step more than gelu and silu)
     t = dict(bf16_steps=4.0 if activation == 2 else 3.0)
     a32, w32, w232 = a.float(), w.float(), w2.float()
-    check(ops.gemm(a32, w32, w2=w232, activation=activation),
-                               ref.gemm(a32, w32, w2=w232, activation=activation), rtol=1e-4, atol=1e-4)
-    check(ops.gemm(a, w, w2=w2, activation=activation, algo=ops.ALGO_GENERIC).float(), want, **t)
-    check(ops.gemm(a, tg, activation=activation).float(), want, **t)      # the dispatcher's choice
+    check(ops.gemm(a32, w32, w2=w232, **kw),
+                               ref.gemm(a32, w32, w2=w232, **kw), rtol=1e-4, atol=1e-4)
+    check(ops.gemm(a, w, w2=w2, **kw, algo=ops.ALGO_GENERIC).float(), want, **t)
+    check(ops.gemm(a, tg, **kw).float(), want, **t)      # the dispatcher's choice
     if M <= 16:
-        check(ops.gemm(a, tg, activation=activation, algo=ops.ALGO_SKINNY).float(), want, **t)
+        check(ops.gemm(a, tg, **kw, algo=ops.ALGO_SKINNY).float(), want, **t)
         h = a.float() * 3.0
         wn = rand((K,), torch.bfloat16, 133, 0.3)
         normed = ref.rmsnorm(h, wn, 1e-6, True, torch.bfloat16)
         got = ops.gemm_normed(None, h, None, tg, post_weight=None, post_eps=0.0, post_plus_one=True, next_weight=wn,
-                              next_eps=1e-6, next_plus_one=True, activation=activation)
-        check(got.float(), ref.gemm(normed, w, w2=w2, activation=activation).float(), **t)
+                              next_eps=1e-6, next_plus_one=True, **kw)
+        check(got.float(), ref.gemm(normed, w, w2=w2, **kw).float(), **t)
     for cuts in (1, 2):
-        got = ops.gemm(a, tg, activation=activation, algo=ops.ALGO_TILED, shape=cuts)
+        got = ops.gemm(a, tg, **kw, algo=ops.ALGO_TILED, shape=cuts)
         check(got.float(), want, **t)
-    check(ops.gemm(a, tg, activation=activation, algo=ops.ALGO_WIDE).float(), want, **t)
+    check(ops.gemm(a, tg, **kw, algo=ops.ALGO_WIDE).float(), want, **t)
     from simply_amd.kernels.lib import KernelError
     with pytest.raises(KernelError, match="activation"):
-        ops.gemm(a, tg, activation=4)
+        ops.gemm(a, tg, activation=9)
 
 
 @pytest.mark.parametrize("M", [1, 3, 8, 9, 13, 16])
