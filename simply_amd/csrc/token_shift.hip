@@ -135,21 +135,54 @@ __global__ __launch_bounds__(kWave) void low_rank_decay_kernel(const void* __res
 typedef __attribute__((__vector_size__(8 * sizeof(__bf16)))) __bf16 bf16x8;
 typedef __attribute__((__vector_size__(4 * sizeof(float)))) float floatx4;
 constexpr int kDecayChunks = 2;   // chunks of 32 factors whose tanh a wave holds at a time
-__global__ __launch_bounds__(256) void low_rank_decay_tiled_kernel(const void* __restrict__ p, int p_dtype, int64_t p_stride,
-                                                                   const bf16* __restrict__ w, const void* __restrict__ w0,
-                                                                   int w0_dtype, float* __restrict__ out, int T, int C,
-                                                                   int rank, int tiles) {
+template <typename PT, typename BT, bool VEC>
+__global__ __launch_bounds__(256) void low_rank_decay_tiled_kernel(const PT* __restrict__ p, int64_t p_stride,
+                                                                   const bf16* __restrict__ w, const BT* __restrict__ w0,
+                                                                   float* __restrict__ out, int T, int C, int rank,
+                                                                   int tiles) {
   const int lane = threadIdx.x % kWave, wave = threadIdx.x / kWave;
   const int r = lane % 16, kq = lane / 16;
   const int t = blockIdx.y * 16 + r, tc = t < T ? t : T - 1;
   const int chunks = (rank + 31) / 32, all = (C + 15) / 16;
   const int n0 = (blockIdx.x * 4 + wave) * tiles, n1 = n0 + tiles < all ? n0 + tiles : all;
   if (n0 >= all) return;   // (a whole wave; there are no barriers)
+  bf16x8 hi[kDecayChunks], mid[kDecayChunks], lo[kDecayChunks];
+  auto factors = [&](int c0) __attribute__((always_inline)) {
+#pragma unroll
+    for (int u = 0; u < kDecayChunks; ++u) {
+      const int k0 = (c0 + u) * 32 + kq * 8;
+      const PT* src = p + static_cast<size_t>(tc) * p_stride + k0;
+      float xs[8];
+      if (VEC && k0 + 8 <= rank) {
+        load8f(src, xs);
+      } else {
+#pragma unroll
+        for (int j = 0; j < 8; ++j) xs[j] = k0 + j < rank ? to_float(src[j]) : 0.f;
+      }
+#pragma unroll
+      for (int j = 0; j < 8; ++j) {
+        const float x = xs[j];
+        // tanh by the hardware's exponential: 1 - 2 / (e^(2x) + 1), and x (1 - x^2 / 3) where that cancels
+        const float y = 1.f - 2.f * __builtin_amdgcn_rcpf(__expf(2.f * x) + 1.f);
+        const float th = fabsf(x) < 0.02f ? x * fmaf(x * x, -1.f / 3.f, 1.f) : y;
+        hi[u][j] = static_cast<__bf16>(th);
+        const float rest = th - static_cast<float>(hi[u][j]);
+        mid[u][j] = static_cast<__bf16>(rest);
+        lo[u][j] = static_cast<__bf16>(rest - static_cast<float>(mid[u][j]));
+      }
+    }
+  };
+  if (chunks <= kDecayChunks) factors(0);   // (held for all of the wave's channels)
   // one pass holds the sums of up to 4 channel tiles
   for (int nb = n0; nb < n1; nb += 4) {
-    floatx4 acc[4];
+    floatx4 acc[4];   // (from the channels' constants)
 #pragma unroll
-    for (int i = 0; i < 4; ++i) acc[i] = floatx4{0.f, 0.f, 0.f, 0.f};
+    for (int i = 0; i < 4; ++i)
+#pragma unroll
+      for (int v = 0; v < 4; ++v) {
+        const int c = (nb + i < n1 ? nb + i : n1 - 1) * 16 + kq * 4 + v;
+        acc[i][v] = to_float(w0[c < C ? c : C - 1]);
+      }
     for (int c0 = 0; c0 < chunks; c0 += kDecayChunks) {
       bf16x8 wv[4][kDecayChunks];
 #pragma unroll
@@ -159,27 +192,15 @@ __global__ __launch_bounds__(256) void low_rank_decay_tiled_kernel(const void* _
           const int tile = nb + i < n1 ? nb + i : n1 - 1, ch = c0 + u < chunks ? c0 + u : chunks - 1;
           wv[i][u] = *reinterpret_cast<const bf16x8*>(w + (static_cast<size_t>(tile) * chunks + ch) * 512 + lane * 8);
         }
+      if (chunks > kDecayChunks) factors(c0);
 #pragma unroll
       for (int u = 0; u < kDecayChunks; ++u) {
         if (c0 + u >= chunks) break;   // (uniform)
-        bf16x8 hi, mid, lo;
-#pragma unroll
-        for (int j = 0; j < 8; ++j) {
-          const int k = (c0 + u) * 32 + kq * 8 + j;
-          const float x = k < rank ? load_f(p, p_dtype, static_cast<size_t>(tc) * p_stride + k) : 0.f;
-          // tanh by the hardware's exponential: 1 - 2 / (e^(2x) + 1), and x (1 - x^2 / 3) where that cancels
-          const float y = 1.f - 2.f * __builtin_amdgcn_rcpf(__expf(2.f * x) + 1.f);
-          const float th = fabsf(x) < 0.02f ? x * fmaf(x * x, -1.f / 3.f, 1.f) : y;
-          hi[j] = static_cast<__bf16>(th);
-          const float rest = th - static_cast<float>(hi[j]);
-          mid[j] = static_cast<__bf16>(rest);
-          lo[j] = static_cast<__bf16>(rest - static_cast<float>(mid[j]));
-        }
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
-          acc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wv[i][u], hi, acc[i], 0, 0, 0);
-          acc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wv[i][u], mid, acc[i], 0, 0, 0);
-          acc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wv[i][u], lo, acc[i], 0, 0, 0);
+          acc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wv[i][u], hi[u], acc[i], 0, 0, 0);
+          acc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wv[i][u], mid[u], acc[i], 0, 0, 0);
+          acc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wv[i][u], lo[u], acc[i], 0, 0, 0);
         }
       }
     }
@@ -192,7 +213,7 @@ __global__ __launch_bounds__(256) void low_rank_decay_tiled_kernel(const void* _
       float* dst = out + static_cast<size_t>(t) * C + c;
       float a[4];
 #pragma unroll
-      for (int v = 0; v < 4; ++v) a[v] = c + v < C ? __expf(-__expf(acc[i][v] + load_f(w0, w0_dtype, c + v))) : 0.f;
+      for (int v = 0; v < 4; ++v) a[v] = c + v < C ? __expf(-__expf(acc[i][v])) : 0.f;
       if (c + 4 <= C && C % 4 == 0) {
         *reinterpret_cast<float4*>(dst) = float4{a[0], a[1], a[2], a[3]};
       } else {
@@ -260,13 +281,27 @@ extern "C" int sa_low_rank_decay(const void* p, int p_dtype, int64_t p_stride, c
              "low_rank_decay: unknown dtype");
   if (tiled) {
     SA_REQUIRE(w_dtype == kBF16, "low_rank_decay: tiled weights are bfloat16");
-    // a wave takes one tile of channels while there are few tokens, four when there are many (their tanh is shared)
+    // a wave takes one tile of channels while there are few tokens, up to eight when there are many (their tanh is shared)
     const int tt = (T + 15) / 16, all = (C + 15) / 16;
-    const int tiles = static_cast<int64_t>(tt) * all >= 4096 ? 4 : 1;
+    const int64_t units = static_cast<int64_t>(tt) * all;
+    const int tiles = units >= 8192 ? 8 : units >= 4096 ? 4 : 1;
     const dim3 grid((all + 4 * tiles - 1) / (4 * tiles), tt);
     SA_REQUIRE(grid.y <= 65535, "low_rank_decay: too many tokens");
-    low_rank_decay_tiled_kernel<<<grid, 256, 0, stream>>>(p, p_dtype, p_stride, static_cast<const bf16*>(w), w0, w0_dtype, out,
-                                                          T, C, rank, tiles);
+    const bool vec = (reinterpret_cast<uintptr_t>(p) & 15u) == 0 && p_stride % 8 == 0;
+#define SA_DECAY(PT, BT, V)                                                                                               \
+  low_rank_decay_tiled_kernel<PT, BT, V><<<grid, 256, 0, stream>>>(static_cast<const PT*>(p), p_stride,                    \
+                                                                   static_cast<const bf16*>(w), static_cast<const BT*>(w0), \
+                                                                   out, T, C, rank, tiles)
+#define SA_DECAY_B(PT, V)                      \
+  do {                                         \
+    if (w0_dtype == kBF16) SA_DECAY(PT, bf16, V); \
+    else SA_DECAY(PT, float, V);               \
+  } while (0)
+    if (p_dtype == kBF16 && vec) SA_DECAY_B(bf16, true);
+    else if (p_dtype == kBF16) SA_DECAY_B(bf16, false);
+    else SA_DECAY_B(float, false);
+#undef SA_DECAY_B
+#undef SA_DECAY
     return check_launch("low_rank_decay");
   }
   const dim3 grid((C + kWave - 1) / kWave, (T + kDecayTokens - 1) / kDecayTokens);
