@@ -8,7 +8,8 @@
 //
 //   exp_gates_kernel          i, f from their projections, the running maximum m, a = exp(f + m' - m), c = exp(i - m)
 //   linear_state_kernel       the recurrence, prefill and decode; a decay per channel may come as z with
-//                             a = sigmoid(z + b)^(1/tau), computed as the tile is staged
+//                             a = sigmoid(z + b)^(1/tau), computed as the tile is staged; with a bonus a token reads
+//                             the state before it and its own k v^T through a factor per key channel
 //   normalized_readout_kernel o / (max(|n.q|, exp(-m)) + 1e-6), each head to unit RMS, times a weight and sigmoid(gate)
 //
 // A request's tokens of this step are rows first .. first + count - 1 (seq_meta [S, 4]: state slot, first row, count,
@@ -82,7 +83,8 @@ template <int DK, int LPC, bool SCALAR, bool BONUS, typename XT>
 __global__ __launch_bounds__(256) void linear_state_kernel(
     const XT* __restrict__ proj, int64_t proj_stride, int q_at, int k_at, int v_at, float q_mult,
     const float* __restrict__ gates, int64_t gates_stride, const void* __restrict__ gate_bias, int bias_dtype,
-    float inv_tau, const void* __restrict__ bonus, int bonus_dtype, int H, int dk, int dv, int ones, float* __restrict__ state, int64_t state_stride,
+    float inv_tau, const void* __restrict__ bonus, int bonus_dtype, int H, int dk, int dv, int ones,
+    float* __restrict__ state, int64_t state_stride,
     const int* __restrict__ seq_meta, float* __restrict__ out) {
   constexpr int R = DK / LPC, COLS = 256 / LPC;
   constexpr int AD = SCALAR ? 1 : DK;
@@ -258,8 +260,8 @@ extern "C" int sa_exp_gates(const float* raw, int64_t raw_stride, const void* bi
 
 extern "C" int sa_linear_state(const void* proj, int dtype, int64_t proj_stride, int q_at, int k_at, int v_at,
                                float q_mult, const float* gates, int64_t gates_stride, const void* gate_bias,
-                               int bias_dtype, float tau, int scalar, const void* bonus, int bonus_dtype, int H, int dk, int dv, int ones, float* state,
-                               int64_t state_stride, const int* seq_meta, int num_seqs, float* out, hipStream_t stream) {
+                               int bias_dtype, float tau, int scalar, const void* bonus, int bonus_dtype, int H,
+                               int dk, int dv, int ones, float* state, int64_t state_stride, const int* seq_meta, int num_seqs, float* out, hipStream_t stream) {
   if (num_seqs == 0) return 0;
   SA_REQUIRE(num_seqs > 0 && num_seqs <= 65535 && H > 0 && H <= 65535 && dk > 0 && dv > 0 && (ones == 0 || ones == 1),
              "linear_state: bad sizes S=%d H=%d dk=%d dv=%d", num_seqs, H, dk, dv);

@@ -44,7 +44,8 @@ static int gemm_routed(const void* A, int a_dtype, int64_t lda, const void* W, c
   int act = epilogue_activation(epilogue);
   epilogue = epilogue_kind(epilogue);
   SA_REQUIRE(epilogue >= 0 && epilogue <= 3, "gemm: unknown epilogue %d", epilogue);
-  SA_REQUIRE(act >= 0 && act < (epilogue == 1 ? kNumGatedRules : kNumActivations) && (epilogue == 1 || epilogue == 3 || act == 0),
+  SA_REQUIRE(act >= 0 && act < (epilogue == 1 ? kNumGatedRules : kNumActivations) &&
+                 (epilogue == 1 || epilogue == 3 || act == 0),
              "gemm: unknown activation %d", act);
   SA_REQUIRE(act != kActClampedGlu || cap > 0.f, "gemm: the clamped gated product needs a positive limit");
   // an activation without a gate: the product as without an epilogue, the activation in the wide kernel's epilogue

@@ -220,7 +220,8 @@ def project(x, w, *, soft_cap: float | None = None, out_dtype: torch.dtype | Non
     """x . w^T (gated if w is a paired tiled weight) for activations x or a `PendingNorm`.  A pending norm is done
     inside the product's kernel when that kernel takes the sizes; otherwise it is materialized first.  `out`: where
     the result goes (a buffer of the caller's), else a new tensor.  `activation`: the gated product's (a code of
-    the ACTIVATIONS registry), with `limit` where its rule has one.  `defer_sum`: the result may be an `ops.PartialSums` (see `ops.gemm`)."""
+    the ACTIVATIONS registry), with `limit` where its rule has one.  `defer_sum`: the result may be an `ops.PartialSums`
+    (see `ops.gemm`)."""
     import functools
 
     from ..kernels import ops

@@ -13,6 +13,8 @@ n_t = a n_(t-1) + c k_t runs beside S (stored as one more column of it, whose va
 o = S^T q / (max(|n . q|, exp(-m)) + 1e-6); each head's o is then divided by its root mean square, multiplied by a
 weight (one entry per head and channel) and by sigmoid(gate x), then projected.
 
+(The kernel of the recurrence also runs 'wkv', parts/wkv.py, whose tokens read the state before them.)
+
 Queries are multiplied by key size^(-1/2).  The state (and m) lives in one float32 row of a state slot per request;
 gates, decays and the recurrence are 32-bit, q, k, v and the gate come out of one product in the activation type.
 """
