@@ -16,6 +16,7 @@ from .nemidra import NemidraConfig
 from .tabupel import TabupelConfig
 from .rudutar import RudutarConfig
 from .kolorax import KoloraxConfig
+from .nozizen import NozizenConfig
 
 
 def architecture_name(d: Mapping[str, Any]) -> str:
@@ -53,4 +54,4 @@ def load_config(model_dir: str):
 
 __all__ = ["EngineConfig", "parse_dtype", "LayerSpec", "ModelSpec", "PartSpec", "ScheduleEntry",
            "ConfigError", "Gemma2Config", "ZenuzenConfig", "NemidraConfig", "TabupelConfig", "RudutarConfig", "KoloraxConfig",
-           "architecture_name", "config_from_dict", "load_config"]
+           "NozizenConfig", "architecture_name", "config_from_dict", "load_config"]

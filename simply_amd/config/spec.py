@@ -74,6 +74,9 @@ class ModelSpec:
     ignorable: tuple[str, ...] = ()
     #: what is done to the stream before every pass of a loop (registry PASS_INPUTS), for entries with `begins_pass`
     pass_input: "PartSpec | None" = None
+    #: None: the residual is one row per token; n: every token has n parallel streams, all equal to the embedding's output
+    #: at the start and summed at the end (every layer's block arrangement is then one of streams)
+    streams: "int | None" = None
 
     def validate(self) -> None:
         n = len(self.layers)
@@ -89,6 +92,13 @@ class ModelSpec:
                         f"schedule entry {i} reads the cache of entry {e.cache_from}, which itself has none")
         if self.pass_input is None and any(e.begins_pass is not None for e in self.schedule):
             raise ValueError("a schedule entry begins a pass, but the model has no pass input")
+        if self.streams is not None:
+            if self.streams < 1 or any(l.block.params.get("streams") != self.streams for l in self.layers):
+                raise ValueError(f"a residual of {self.streams} streams: every layer's block arrangement takes as many")
+            if any(e.begins_pass is not None or e.add_embedding for e in self.schedule):
+                raise ValueError("a residual of several streams has no passes that are given the embedding again")
+        elif any("streams" in l.block.params for l in self.layers):
+            raise ValueError("a block arrangement of streams needs a model with streams")
         for name, of in self.copies.items():
             if name == of:
                 raise ValueError(f"tensor {name!r} is declared a copy of itself")

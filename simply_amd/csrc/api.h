@@ -469,10 +469,13 @@ int sa_exp_gates(const float* raw, int64_t raw_stride, const void* bias, int bia
 // c = 1; with tau > 0 these gates are z and a = sigmoid(z + gate_bias)^(1 / tau) (gate_bias [H dk] or null).  ones: the
 // state has a column dv whose value is always 1.  bonus [H dk] (null: none; with decays per key channel): out_t =
 // (S_(t-1) + diag(bonus) k v^T)^T q, the state before the token.  state [slot][H][dv + ones][dk]; out [T, H (dv + ones)].
+// key_heads: heads of queries and keys, each shared by H / key_heads neighbouring heads (fewer than H with scalar only);
+// skip [H] (null: none; with scalar, ones 0): out += skip[h] v.
 int sa_linear_state(const void* proj, int dtype, int64_t proj_stride, int q_at, int k_at, int v_at, float q_mult,
                     const float* gates, int64_t gates_stride, const void* gate_bias, int bias_dtype, float tau, int scalar,
-                    const void* bonus, int bonus_dtype, int H, int dk, int dv, int ones, float* state, int64_t state_stride, const int* seq_meta, int num_seqs,
-                    float* out, hipStream_t stream);
+                    const void* bonus, int bonus_dtype, const void* skip, int skip_dtype, int H, int key_heads, int dk, int dv,
+                    int ones, float* state, int64_t state_stride, const int* seq_meta, int num_seqs, float* out,
+                    hipStream_t stream);
 // x [T, H, size + 1] -> out[t, h, :] = unit_rms(x[t, h, :size] / (max(|x[t, h, size]|, floor[t, h]) + 1e-6)) * w[h, :]
 // * sigmoid(g[t, h, :]).
 int sa_normalized_readout(const float* x, const float* floor, int64_t floor_stride, const void* g, int g_dtype,
@@ -485,28 +488,51 @@ int sa_normalized_readout(const float* x, const float* floor, int64_t floor_stri
 // convolution (taps [channels, num_taps] oldest first; tails float32 [slots, (num_taps - 1) * channels], updated).  norm
 // 0: none; 1: queries and keys head by head with weights [dk]; 2: over the whole row with weights [H * dk] and
 // [K * dk].  Then the first rot_dims entries of every head turn in pairs (i, i + rot_dims / 2) by position *
-// inv_freq[i], and queries are multiplied by 1 + temp_coef * ln(floor((position + 1) / temp_every) + 1) (temp_every 0:
+// inv_freq[i] and are multiplied by rot_mult, and queries are multiplied by 1 + temp_coef * ln(floor((position + 1) / temp_every) + 1) (temp_every 0:
 // not) and by q_mult.  Queries go to q_out [T, H * dk], keys and values into their pages.  taps_by_tap (or null): the
 // taps once more as [num_taps, channels] in their type, which the kernel for aligned bfloat16 rows reads in pieces.
 // in_bias (or null; only with num_taps 0): a bias per channel that the projection has not had added yet.
 int sa_attention_inputs(const void* proj, int dtype, int64_t row_stride, int H, int K, int dk, int dv, int k_at, int v_at,
                         int values_are_keys, const void* taps, int taps_dtype, int num_taps, float* tails,
                         int64_t tail_stride, int norm, const void* q_w, const void* k_w, int w_dtype, float eps,
-                        const float* inv_freq, int rot_dims, float temp_coef, int temp_every, float q_mult,
+                        const float* inv_freq, int rot_dims, float rot_mult, float temp_coef, int temp_every, float q_mult,
                         const int* seq_meta, int num_seqs, int max_q_len, const int64_t* slot_mapping, void* q_out, int64_t q_stride,
                         void* k_pages, void* v_pages, int page_size, const void* taps_by_tap, const void* in_bias,
                         int bias_dtype, hipStream_t stream);
+
+// ---- a residual of several streams (streams.hip)
+// S streams of a token: entries x[t * x_row + s * x_stream + d] (x_stream 0: all are the same row).  With y (type of out,
+// or `planes` > 0 partial results [planes][T][D] of a bfloat16 product): h[t, q, :] = sum_s mix[s, q] x_s + out_w[q] y
+// (h [T, S, D], may be x).  With in_w: out[t, :] = u / sqrt(mean(u^2) + eps) * w over u = sum_s in_w[s] (new) stream s
+// (w null: u itself).  rows (or null, only without y): token t is read at row rows[t].  mix, out_w, in_w: float32.
+int sa_streams(const float* x, int64_t x_row, int64_t x_stream, float* h, int S, const void* y, int y_dtype, int64_t y_stride,
+               int planes, const float* mix, const float* out_w, const float* in_w, const void* w, int w_dtype, float eps,
+               const int* rows, void* out, int out_dtype, int T, int D, hipStream_t stream);
+
+// ---- around a state-space mixer's recurrence (ssm.hip)
+// Columns x_at .. x_at + C of proj's rows through a causal convolution (taps [num_taps, C], oldest first, bias [C]) and
+// silu into y [T, C] (proj's type); tails float32 [slots, (num_taps - 1) * C] are read and moved on.  Columns dt_at ..
+// dt_at + H: dt = softplus(. + dt_bias[h]), l = -exp(a_log[h]) dt; gates [T, 3 H] = exp(l), dt, l.
+int sa_ssm_inputs(const void* proj, int dtype, int64_t row_stride, int x_at, int dt_at, int C, const void* taps,
+                  const void* bias, int taps_dtype, int num_taps, const void* dt_bias, const void* a_log, int vec_dtype,
+                  float* tails, int64_t tail_stride, const int* seq_meta, int num_seqs, int max_q_len, void* y, float* gates,
+                  int H, hipStream_t stream);
+// out[t, :] = v / sqrt(mean(v^2) + eps) * w, v = y silu(z), in `groups` equal parts of the width, each by its own mean.
+int sa_gated_group_norm(const float* y, int64_t y_stride, const void* z, int dtype, int64_t z_stride, const void* w,
+                        int w_dtype, float eps, void* out, int groups, int64_t out_stride, int T, int width,
+                        hipStream_t stream);
 
 // ---- routed experts (routed.hip)
 // softmax over E logits, the top largest: experts [T, top], weights [T, top] = score * scale.
 int sa_route(const float* logits, int64_t stride, int T, int E, int top, float scale, int* experts, float* weights,
              hipStream_t stream);
-// Scores are sigmoids of the logits, or their softmax.  The choice goes by score + correction[e] (null: by the score);
+// bias [E] (or null) is added to the logits.  Scores are sigmoids of the logits (softmax 0), their softmax (1), or the
+// logits themselves with the softmax among the chosen ones as weights (2; renorm < 0).  The choice goes by score + correction[e] (null: by the score);
 // the experts form `groups` equal groups of neighbours, a group's score is the sum of its two largest choice scores
 // (group_best 2) or its largest one (1), and only experts of the `keep` best groups can be chosen.  weights = score *
 // scale (without the correction), with renorm >= 0 divided by the chosen scores' sum + renorm.
-int sa_route_choice(const float* logits, int64_t stride, int T, int E, int top, float scale, const void* correction,
-                    int corr_dtype, int groups, int keep, int softmax, int group_best, float renorm, int* experts,
+int sa_route_choice(const float* logits, int64_t stride, int T, int E, int top, float scale, const void* bias,
+                    int bias_dtype, const void* correction, int corr_dtype, int groups, int keep, int softmax, int group_best, float renorm, int* experts,
                     float* weights, hipStream_t stream);
 // The most tiles of tile_rows (16 or 64) rows of one expert that P pairs over E experts make.
 int sa_expert_tiles_max(int P, int E, int tile_rows);

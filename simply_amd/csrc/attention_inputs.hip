@@ -8,7 +8,7 @@
 //   norm          of queries and of keys: none; head by head, x / sqrt(mean(x^2) + eps) * w[d] with w shared by the
 //                 heads; or over the whole row (all heads at once) with a weight per entry.
 //   rotation      the first rot_dims entries of every head turn, entry i with entry i + rot_dims / 2, by the angle
-//                 position * inv_freq[i]; after the norm.
+//                 position * inv_freq[i] and are multiplied by rot_mult (on sines and cosines); after the norm.
 //   temperature   queries at position p times 1 + coef * ln(floor((p + 1) / every) + 1)  (every == 0: none), and times
 //                 q_mult (the scores' factor, for an attention kernel that has none of its own).
 //   bias          (without a convolution) a bias per column of the projection, added as the row is read.
@@ -36,7 +36,7 @@ struct AttentionInputs {
   int norm;                // 0 none, 1 head by head, 2 over the whole row
   int rot_dims;
   int temp_every;
-  float temp_coef, eps;
+  float temp_coef, eps, rot_mult;
   const void* in_bias;      // (or null) added to the projection's columns as they are read; without a convolution only
   int bias_dtype;
   int own_tails;            // every request brings one token: the thread that reads a channel's tail also moves it on
@@ -88,8 +88,12 @@ __global__ __launch_bounds__(kInputThreads) void attention_inputs_kernel(
     stage[i] = v;
   }
   // the token's angles once for all heads (every head turns by the same ones)
-  for (int i = tid; i < p.rot_dims / 2; i += kInputThreads)
-    sincosf(static_cast<float>(pos) * inv_freq[i], &rot_s[p.rot_dims / 2 + i], &rot_s[i]);
+  for (int i = tid; i < p.rot_dims / 2; i += kInputThreads) {
+    float sn, cs;
+    sincosf(static_cast<float>(pos) * inv_freq[i], &sn, &cs);
+    rot_s[i] = cs * p.rot_mult;
+    rot_s[p.rot_dims / 2 + i] = sn * p.rot_mult;
+  }
   __syncthreads();
 
   const int64_t kv_slot = sec > 0 ? slot_mapping[t] : -1;
@@ -230,8 +234,12 @@ __global__ __launch_bounds__(kInputThreads) void attention_inputs_rows_kernel(
     if (c < q_len) ss_q += ss;
     else if (c < k_end) ss_k += ss;
   }
-  for (int i = tid; i < p.rot_dims / 2; i += kInputThreads)
-    sincosf(static_cast<float>(pos) * inv_freq[i], &rot_s[p.rot_dims / 2 + i], &rot_s[i]);
+  for (int i = tid; i < p.rot_dims / 2; i += kInputThreads) {
+    float sn, cs;
+    sincosf(static_cast<float>(pos) * inv_freq[i], &sn, &cs);
+    rot_s[i] = cs * p.rot_mult;
+    rot_s[p.rot_dims / 2 + i] = sn * p.rot_mult;
+  }
   float r_q = 1.f, r_k = 1.f;
   if (p.norm == 2) {
     r_q = 1.f / sqrtf(block_sum(ss_q, red_s) / static_cast<float>(q_len) + p.eps);
@@ -328,7 +336,7 @@ extern "C" int sa_attention_inputs(const void* proj, int dtype, int64_t row_stri
                                    int k_at, int v_at, int values_are_keys, const void* taps, int taps_dtype,
                                    int num_taps, float* tails, int64_t tail_stride, int norm, const void* q_w,
                                    const void* k_w, int w_dtype, float eps, const float* inv_freq, int rot_dims,
-                                   float temp_coef, int temp_every, float q_mult, const int* seq_meta, int num_seqs,
+                                   float rot_mult, float temp_coef, int temp_every, float q_mult, const int* seq_meta, int num_seqs,
                                    int max_q_len,
                                    const int64_t* slot_mapping, void* q_out, int64_t q_stride, void* k_pages,
                                    void* v_pages, int page_size, const void* taps_by_tap, const void* in_bias,
@@ -371,7 +379,7 @@ extern "C" int sa_attention_inputs(const void* proj, int dtype, int64_t row_stri
   AttentionInputs p;
   p.H = H, p.K = K, p.dk = dk, p.dv = dv, p.k_at = k_at, p.v_at = v_at, p.values_are_keys = values_are_keys;
   p.taps = num_taps, p.conv_channels = C, p.norm = norm, p.rot_dims = rot_dims, p.temp_every = temp_every;
-  p.temp_coef = temp_coef, p.eps = eps, p.page_size = page_size, p.q_mult = q_mult;
+  p.temp_coef = temp_coef, p.eps = eps, p.rot_mult = rot_mult, p.page_size = page_size, p.q_mult = q_mult;
   p.in_bias = in_bias, p.bias_dtype = bias_dtype;
   // with one token a request a channel's tail has one reader, who moves it on; else a second launch does, behind all readers
   p.own_tails = max_q_len == 1 && num_taps > 1;

@@ -9,7 +9,8 @@
 //   exp_gates_kernel          i, f from their projections, the running maximum m, a = exp(f + m' - m), c = exp(i - m)
 //   linear_state_kernel       the recurrence, prefill and decode; a decay per channel may come as z with
 //                             a = sigmoid(z + b)^(1/tau), computed as the tile is staged; with a bonus a token reads
-//                             the state before it and its own k v^T through a factor per key channel
+//                             the state before it and its own k v^T through a factor per key channel; queries and keys
+//                             may be shared by groups of heads; a skip adds a head's factor times v to its result
 //   normalized_readout_kernel o / (max(|n.q|, exp(-m)) + 1e-6), each head to unit RMS, times a weight and sigmoid(gate)
 //
 // A request's tokens of this step are rows first .. first + count - 1 (seq_meta [S, 4]: state slot, first row, count,
@@ -83,8 +84,8 @@ template <int DK, int LPC, bool SCALAR, bool BONUS, typename XT>
 __global__ __launch_bounds__(256) void linear_state_kernel(
     const XT* __restrict__ proj, int64_t proj_stride, int q_at, int k_at, int v_at, float q_mult,
     const float* __restrict__ gates, int64_t gates_stride, const void* __restrict__ gate_bias, int bias_dtype,
-    float inv_tau, const void* __restrict__ bonus, int bonus_dtype, int H, int dk, int dv, int ones,
-    float* __restrict__ state, int64_t state_stride,
+    float inv_tau, const void* __restrict__ bonus, int bonus_dtype, const void* __restrict__ skip, int skip_dtype, int H,
+    int heads_per_key, int dk, int dv, int ones, float* __restrict__ state, int64_t state_stride,
     const int* __restrict__ seq_meta, float* __restrict__ out) {
   constexpr int R = DK / LPC, COLS = 256 / LPC;
   constexpr int AD = SCALAR ? 1 : DK;
@@ -93,6 +94,7 @@ __global__ __launch_bounds__(256) void linear_state_kernel(
   const int* meta = seq_meta + 4 * blockIdx.x;
   const int slot = meta[0], first = meta[1], count = meta[2];
   const int h = blockIdx.y, tid = threadIdx.x;
+  const int kh = heads_per_key > 1 ? h / heads_per_key : h;   // whose queries and keys this head reads
   const int CT = dv + ones;
   const int col = blockIdx.z * COLS + tid / LPC, part = tid % LPC;
   const bool live = col < CT;
@@ -104,6 +106,8 @@ __global__ __launch_bounds__(256) void linear_state_kernel(
     if constexpr (BONUS) bo[r] = i < dk ? load_f(bonus, bonus_dtype, static_cast<size_t>(h) * dk + i) : 0.f;
     s[r] = (live && i < dk) ? S[static_cast<size_t>(col) * dk + i] : 0.f;
   }
+  float sk = 0.f;
+  if constexpr (SCALAR) sk = skip != nullptr ? load_f(skip, skip_dtype, h) : 0.f;
   constexpr int PQ = kStateTokens * DK / 256, PV = (kStateTokens * COLS + 255) / 256;
   float pq[PQ], pk[PQ], pa[SCALAR ? 1 : PQ], pb[SCALAR ? 1 : PQ], pv[PV], pc = 0.f;
   bool pok[SCALAR ? 1 : PQ];
@@ -115,8 +119,8 @@ __global__ __launch_bounds__(256) void linear_state_kernel(
       const bool ok = j < tn && d < dk;
       const size_t t = static_cast<size_t>(first + t0 + (ok ? j : 0));
       const XT* row = proj + t * proj_stride;
-      pq[i] = ok ? to_float(row[q_at + h * dk + d]) * q_mult : 0.f;
-      pk[i] = ok ? to_float(row[k_at + h * dk + d]) : 0.f;
+      pq[i] = ok ? to_float(row[q_at + kh * dk + d]) * q_mult : 0.f;
+      pk[i] = ok ? to_float(row[k_at + kh * dk + d]) : 0.f;
       if constexpr (!SCALAR) {
         // (with inv_tau > 0 the gates are z and the bias rides along: the decay is computed when the tile is put into
         // LDS, a tile later, so that nothing waits for these loads here)
@@ -196,6 +200,12 @@ __global__ __launch_bounds__(256) void linear_state_kernel(
       }
       lanes_sum4<LPC>(o);
       if (live && part == 0) {
+        if constexpr (SCALAR) {
+          if (skip != nullptr) {
+#pragma unroll
+            for (int i = 0; i < 4; ++i) o[i] = fmaf(sk, vs[j0 + i][tid / LPC], o[i]);
+          }
+        }
 #pragma unroll
         for (int i = 0; i < 4; ++i)
           if (WHOLE || j0 + i < tn)
@@ -260,16 +270,21 @@ extern "C" int sa_exp_gates(const float* raw, int64_t raw_stride, const void* bi
 
 extern "C" int sa_linear_state(const void* proj, int dtype, int64_t proj_stride, int q_at, int k_at, int v_at,
                                float q_mult, const float* gates, int64_t gates_stride, const void* gate_bias,
-                               int bias_dtype, float tau, int scalar, const void* bonus, int bonus_dtype, int H,
-                               int dk, int dv, int ones, float* state, int64_t state_stride, const int* seq_meta, int num_seqs, float* out, hipStream_t stream) {
+                               int bias_dtype, float tau, int scalar, const void* bonus, int bonus_dtype,
+                               const void* skip, int skip_dtype, int H, int key_heads, int dk, int dv, int ones, float* state,
+                               int64_t state_stride, const int* seq_meta, int num_seqs, float* out, hipStream_t stream) {
   if (num_seqs == 0) return 0;
   SA_REQUIRE(num_seqs > 0 && num_seqs <= 65535 && H > 0 && H <= 65535 && dk > 0 && dv > 0 && (ones == 0 || ones == 1),
              "linear_state: bad sizes S=%d H=%d dk=%d dv=%d", num_seqs, H, dk, dv);
   SA_REQUIRE(dk <= 256, "linear_state: key size %d is above 256", dk);
   const int CT = dv + ones;
   SA_REQUIRE(state_stride >= static_cast<int64_t>(H) * dk * CT, "linear_state: the state rows are too short");
-  SA_REQUIRE(q_at >= 0 && k_at >= 0 && v_at >= 0 && proj_stride >= q_at + static_cast<int64_t>(H) * dk &&
-                 proj_stride >= k_at + static_cast<int64_t>(H) * dk && proj_stride >= v_at + static_cast<int64_t>(H) * dv,
+  SA_REQUIRE(key_heads > 0 && H % key_heads == 0 && (key_heads == H || scalar != 0),
+             "linear_state: %d heads over %d heads of queries and keys (fewer than heads only with decays per head)", H, key_heads);
+  SA_REQUIRE(skip == nullptr || (scalar != 0 && ones == 0 && (skip_dtype == kF32 || skip_dtype == kBF16)),
+             "linear_state: a skip goes with decays per head and without a normalizer");
+  SA_REQUIRE(q_at >= 0 && k_at >= 0 && v_at >= 0 && proj_stride >= q_at + static_cast<int64_t>(key_heads) * dk &&
+                 proj_stride >= k_at + static_cast<int64_t>(key_heads) * dk && proj_stride >= v_at + static_cast<int64_t>(H) * dv,
              "linear_state: the projection rows are too short");
   SA_REQUIRE(gates_stride >= (scalar ? 2 * H : H * dk), "linear_state: the gate rows are too short");
   SA_REQUIRE(proj != nullptr && gates != nullptr && state != nullptr && seq_meta != nullptr && out != nullptr,
@@ -283,7 +298,7 @@ extern "C" int sa_linear_state(const void* proj, int dtype, int64_t proj_stride,
 #define SA_STATE_LAUNCH(DK, LPC, SC, BO, XT)                                                                             \
   linear_state_kernel<DK, LPC, SC, BO, XT><<<dim3(num_seqs, H, (CT + 256 / LPC - 1) / (256 / LPC)), 256, 0, stream>>>(   \
       static_cast<const XT*>(proj), proj_stride, q_at, k_at, v_at, q_mult, gates, gates_stride, gate_bias, bias_dtype, \
-      inv_tau, bonus, bonus_dtype, H, dk, dv, ones, state, state_stride, seq_meta, out)
+      inv_tau, bonus, bonus_dtype, skip, skip_dtype, H, H / key_heads, dk, dv, ones, state, state_stride, seq_meta, out)
 #define SA_STATE_SIZES(SC, BO, XT)                       \
   do {                                               \
     if (dk <= 16) SA_STATE_LAUNCH(16, 4, SC, BO, XT);    \

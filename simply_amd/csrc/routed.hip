@@ -61,15 +61,17 @@ __global__ __launch_bounds__(kWave) void route_kernel(const float* __restrict__ 
   }
 }
 
-// A wave per token, for routers with options.  Scores are sigmoids of the logits or (`softmax`) their softmax over all
-// experts.  The choice is made by score + correction[e] (correction null: by the score); the experts form `groups`
+// A wave per token, for routers with options.  bias[e] (or null) is added to the logits first.  Scores are sigmoids of the
+// logits, (softmax 1) their softmax over all experts, or (softmax 2) the logits themselves, and the weights are then the
+// chosen ones' softmax among themselves (times scale; no renorm).  The choice is made by score + correction[e] (correction null: by the score); the experts form `groups`
 // equal groups of neighbours, a group's score is the sum of its two largest choice scores (group_best 2; of its only
 // one, in groups of one) or the largest one (group_best 1), and only experts of the `keep` groups with the largest
 // scores can be chosen (of equal ones the lowest index, for groups and for experts).  weight = score * scale without
 // the correction, with renorm >= 0 divided by the chosen scores' sum + renorm.  Choice scores can be negative: what is
 // taken or shut out is -inf.
 __global__ __launch_bounds__(kWave) void route_choice_kernel(const float* __restrict__ logits, int64_t stride, int E,
-                                                             int top, float scale, const void* __restrict__ correction,
+                                                             int top, float scale, const void* __restrict__ bias,
+                                                             int bias_dtype, const void* __restrict__ correction,
                                                              int corr_dtype, int groups, int keep, int softmax,
                                                              int group_best, float renorm, int* __restrict__ experts,
                                                              float* __restrict__ weights) {
@@ -82,9 +84,10 @@ __global__ __launch_bounds__(kWave) void route_choice_kernel(const float* __rest
   for (int i = 0; i < kRouteSlots; ++i) {
     const int e = lane + i * kWave;
     s[i] = e < E ? logits[static_cast<size_t>(t) * stride + e] : -INFINITY;
+    if (bias != nullptr && e < E) s[i] += load_f(bias, bias_dtype, e);
     mx = fmaxf(mx, s[i]);
   }
-  if (softmax) {
+  if (softmax == 1) {
     mx = wave_max(mx);
 #pragma unroll
     for (int i = 0; i < kRouteSlots; ++i) {
@@ -98,7 +101,7 @@ __global__ __launch_bounds__(kWave) void route_choice_kernel(const float* __rest
     const int e = lane + i * kWave;
     c[i] = -INFINITY;
     if (e < E) {
-      s[i] = softmax ? s[i] / sum : 1.f / (1.f + expf(-s[i]));
+      if (softmax != 2) s[i] = softmax ? s[i] / sum : 1.f / (1.f + expf(-s[i]));
       c[i] = correction != nullptr ? s[i] + load_f(correction, corr_dtype, e) : s[i];
       choice_s[e] = c[i];
     } else {
@@ -169,6 +172,14 @@ __global__ __launch_bounds__(kWave) void route_choice_kernel(const float* __rest
     }
   }
   __syncthreads();
+  if (softmax == 2) {
+    float best = -INFINITY, among = 0.f;
+    for (int r = 0; r < top; ++r) best = fmaxf(best, choice_s[r]);
+    for (int r = 0; r < top; ++r) among += expf(choice_s[r] - best);
+    for (int r = lane; r < top; r += kWave)
+      weights[static_cast<size_t>(t) * top + r] = expf(choice_s[r] - best) / among * scale;
+    return;
+  }
   const float by = renorm >= 0.f ? total + renorm : 1.f;
   for (int r = lane; r < top; r += kWave) weights[static_cast<size_t>(t) * top + r] = choice_s[r] / by * scale;
 }
@@ -491,7 +502,7 @@ extern "C" int sa_route(const float* logits, int64_t stride, int T, int E, int t
 }
 
 extern "C" int sa_route_choice(const float* logits, int64_t stride, int T, int E, int top, float scale,
-                               const void* correction, int corr_dtype, int groups, int keep, int softmax,
+                               const void* bias, int bias_dtype, const void* correction, int corr_dtype, int groups, int keep, int softmax,
                                int group_best, float renorm, int* experts, float* weights, hipStream_t stream) {
   if (T == 0) return 0;
   SA_REQUIRE(T > 0 && E > 0 && E <= kRouteSlots * kWave && top > 0 && stride >= E,
@@ -503,7 +514,10 @@ extern "C" int sa_route_choice(const float* logits, int64_t stride, int T, int E
              E / groups);
   SA_REQUIRE(correction == nullptr || corr_dtype == kF32 || corr_dtype == kBF16, "route_choice: unknown dtype %d",
              corr_dtype);
-  route_choice_kernel<<<T, kWave, 0, stream>>>(logits, stride, E, top, scale, correction, corr_dtype, groups, keep,
+  SA_REQUIRE(bias == nullptr || bias_dtype == kF32 || bias_dtype == kBF16, "route_choice: unknown dtype %d", bias_dtype);
+  SA_REQUIRE(softmax >= 0 && softmax <= 2 && (softmax != 2 || renorm < 0.f),
+             "route_choice: scores %d (0 sigmoid, 1 softmax, 2 the chosen logits' softmax, which sums to 1 by itself)", softmax);
+  route_choice_kernel<<<T, kWave, 0, stream>>>(logits, stride, E, top, scale, bias, bias_dtype, correction, corr_dtype, groups, keep,
                                                softmax, group_best, renorm, experts, weights);
   return check_launch("route_choice");
 }

@@ -87,17 +87,21 @@ _SIGNATURES = {
     "sa_bias_add": [_P, _I, _L, _P, _I, _I, _I, _P],
     "sa_weighted_sum": [_P, _L, _F, _P, _L, _F, _I, _P, _L, _I, _I, _P],
     "sa_exp_gates": [_P, _L, _P, _I, _F, _I, _P, _L, _P, _I, _P, _P],
-    "sa_linear_state": [_P, _I, _L, _I, _I, _I, _F, _P, _L, _P, _I, _F, _I, _P, _I, _I, _I, _I, _I, _P, _L, _P, _I, _P, _P],
+    "sa_linear_state": [_P, _I, _L, _I, _I, _I, _F, _P, _L, _P, _I, _F, _I, _P, _I, _P, _I, _I, _I, _I, _I, _I, _P, _L, _P, _I,
+                        _P, _P],
     "sa_normalized_readout": [_P, _P, _L, _P, _I, _L, _P, _I, _F, _P, _I, _L, _I, _I, _I, _P],
     "sa_route": [_P, _L, _I, _I, _I, _F, _P, _P, _P],
     "sa_expert_sort": [_P, _I, _I, _I, _P, _P, _I, _P],
     "sa_expert_product": [_P, _I, _L, _I, _I, _P, _P, _I, _I, _P, _P, _I, _I, _I, _I, _F, _P, _L, _I, _I, _P],
-    "sa_route_choice": [_P, _L, _I, _I, _I, _F, _P, _I, _I, _I, _I, _I, _F, _P, _P, _P],
+    "sa_route_choice": [_P, _L, _I, _I, _I, _F, _P, _I, _P, _I, _I, _I, _I, _I, _F, _P, _P, _P],
     "sa_token_shift": [_P, _I, _L, _P, _I, _I, _P, _L, _P, _I, _I, _P, _I, _P],
     "sa_low_rank_decay": [_P, _I, _L, _P, _I, _I, _P, _I, _P, _I, _I, _I, _P],
     "sa_gemm_sections": [_P, _L, _P, _P, _I, _L, _I, _I, _I, _I, _I, _P, _L, _P],
+    "sa_streams": [_P, _L, _L, _P, _I, _P, _I, _L, _I, _P, _P, _P, _P, _I, _F, _P, _P, _I, _I, _I, _P],
+    "sa_ssm_inputs": [_P, _I, _L, _I, _I, _I, _P, _P, _I, _I, _P, _P, _I, _P, _L, _P, _I, _I, _P, _P, _I, _P],
+    "sa_gated_group_norm": [_P, _L, _P, _I, _L, _P, _I, _F, _P, _I, _L, _I, _I, _P],
     "sa_concat_rows": [_P, _P, _P, _I, _I, _I, _I, _P],
-    "sa_attention_inputs": [_P, _I, _L, _I, _I, _I, _I, _I, _I, _I, _P, _I, _I, _P, _L, _I, _P, _P, _I, _F, _P, _I, _F, _I,
+    "sa_attention_inputs": [_P, _I, _L, _I, _I, _I, _I, _I, _I, _I, _P, _I, _I, _P, _L, _I, _P, _P, _I, _F, _P, _I, _F, _F, _I,
                             _F, _P, _I, _I, _P, _P, _L, _P, _P, _I, _P, _P, _I, _P],
     "sa_expert_combine": [_P, _P, _I, _P, _I, _L, _P, _L, _P, _I, _L, _I, _I, _P],
     "sa_sample": [_P, _L, _I, _I, _P, _P, _P, _P, _P, _P, _P, _I, _P, _L, _P],

@@ -1051,8 +1051,8 @@ def attention_inputs(proj: torch.Tensor, seq_meta: torch.Tensor, num_seqs: int, 
                      num_kv_heads: int, key_dim: int, value_dim: int, *, values_are_keys: bool = False,
                      taps: torch.Tensor | None = None, tails: torch.Tensor | None = None, norm: str | None = None,
                      q_weight: torch.Tensor | None = None, k_weight: torch.Tensor | None = None, eps: float = 0.0,
-                     inv_freq: torch.Tensor | None = None, rot_dims: int = 0, temp_coef: float = 0.0, temp_every: int = 0,
-                     q_mult: float = 1.0, taps_by_tap: torch.Tensor | None = None, in_bias: torch.Tensor | None = None,
+                     inv_freq: torch.Tensor | None = None, rot_dims: int = 0, rot_mult: float = 1.0,
+                     temp_coef: float = 0.0, temp_every: int = 0, q_mult: float = 1.0, taps_by_tap: torch.Tensor | None = None, in_bias: torch.Tensor | None = None,
                      slot_mapping: torch.Tensor | None = None, k_pages: torch.Tensor | None = None,
                      v_pages: torch.Tensor | None = None) -> torch.Tensor:
     """From fused projection rows [H * dk queries | K * dk keys | K * dv values | ...] of a ragged step (seq_meta) to
@@ -1060,7 +1060,7 @@ def attention_inputs(proj: torch.Tensor, seq_meta: torch.Tensor, num_seqs: int, 
     passes a causal convolution first (taps oldest first; the tails are the rows that earlier steps projected last and
     are brought up to date).  norm 'head': queries and keys divided by each head's root mean square, times q_weight /
     k_weight [dk]; 'row': by the whole row's, times weights [H * dk] / [K * dk].  Then the first rot_dims entries of
-    every head turn in pairs (i, i + rot_dims / 2) by position * inv_freq[i]; queries are multiplied by
+    every head turn in pairs (i, i + rot_dims / 2) by position * inv_freq[i], times rot_mult; queries are multiplied by
     1 + temp_coef * ln(floor((position + 1) / temp_every) + 1) (temp_every 0: not) and by q_mult.  Keys go into k_pages, values
     (values_are_keys: the keys' columns as projected, and there are no value columns) into v_pages; without pages the
     rows hold queries only.  taps_by_tap: the taps once more as [n, channels] (what the kernel for aligned bfloat16 rows
@@ -1120,7 +1120,7 @@ def attention_inputs(proj: torch.Tensor, seq_meta: torch.Tensor, num_seqs: int, 
               int(bool(values_are_keys)), _ptr(taps), _code(taps) if taps is not None else 0, int(n_taps),
               _ptr(tails) if n_taps > 1 else None, tails.stride(0) if n_taps > 1 else 0, code, _ptr(q_weight),
               _ptr(k_weight) if own else None, _CODES[w_dtype] if w_dtype is not None else 0, float(eps), _ptr(inv_freq),
-              int(rot_dims), float(temp_coef), int(temp_every), float(q_mult), _ptr(seq_meta), int(num_seqs), int(max_q_len),
+              int(rot_dims), float(rot_mult), float(temp_coef), int(temp_every), float(q_mult), _ptr(seq_meta), int(num_seqs), int(max_q_len),
               _ptr(slot_mapping) if own else None, _ptr(q_out), q_out.stride(0), _ptr(k_pages), _ptr(v_pages) if own else None,
               int(page_size), _ptr(taps_by_tap), _ptr(in_bias), _code(in_bias) if in_bias is not None else 0, _stream())
     return q_out
@@ -1570,14 +1570,17 @@ def exp_gates(raw: torch.Tensor, bias: torch.Tensor | None, cap: float, num_head
 def linear_state(proj: torch.Tensor, q_at: int, k_at: int, v_at: int, q_mult: float, gates: torch.Tensor, scalar: bool,
                  num_heads: int, key_dim: int, value_dim: int, ones: bool, state: torch.Tensor, seq_meta: torch.Tensor,
                  num_seqs: int, *, decay_bias: torch.Tensor | None = None, tau: float | None = None,
-                 bonus: torch.Tensor | None = None) -> torch.Tensor:
+                 bonus: torch.Tensor | None = None, key_heads: int | None = None,
+                 skip: torch.Tensor | None = None) -> torch.Tensor:
     """S <- diag(a) S + c k v^T, o = S^T (q * q_mult) along each request's tokens, from and into state float32 [slots,
     >= H * dk * (dv + ones)] (per head [dv + ones][dk]).  q, k, v: columns q_at, k_at, v_at of proj's rows, H heads
     each.  scalar: gates float32 [T, >= 2 H] hold a and c per head; else [T, H * dk] hold a per key channel, c = 1;
     with `tau` these hold z instead, and a = sigmoid(z + decay_bias)^(1 / tau) (decay_bias [H * dk] or None).
     bonus [H * dk] (decays per key channel): o = (S_before + diag(bonus) k v^T)^T q, the state before the token.
-    ones: one more column whose value is always 1 (a normalizer).  Returns float32 [T, H * (dv + ones)]."""
-    _dev(proj, gates, state, seq_meta)
+    ones: one more column whose value is always 1 (a normalizer).  key_heads (with scalar): q and k have that many heads,
+    each shared by H / key_heads neighbouring ones; skip [H] (with scalar, without ones): o += skip * v.  Returns float32
+    [T, H * (dv + ones)]."""
+    _dev(proj, gates, state, seq_meta, skip)
     T = proj.shape[0]
     H, dk, dv, CT = int(num_heads), int(key_dim), int(value_dim), int(value_dim) + int(bool(ones))
     if gates.dtype != torch.float32 or gates.shape[0] != T:
@@ -1591,12 +1594,15 @@ def linear_state(proj: torch.Tensor, q_at: int, k_at: int, v_at: int, q_mult: fl
         raise KernelError("linear_state: one bias per key channel")
     if bonus is not None and (scalar or bonus.numel() != H * dk or not bonus.is_contiguous()):
         raise KernelError("linear_state: a bonus has one entry per head and key channel and goes with decays per channel")
+    key_heads = H if key_heads is None else int(key_heads)
+    if skip is not None and (not scalar or ones or skip.numel() != H or not skip.is_contiguous()):
+        raise KernelError("linear_state: a skip has one entry per head and goes with decays per head, without a normalizer")
     _dev(decay_bias, bonus)
     out = torch.empty((T, H * CT), dtype=torch.float32, device=proj.device)
     _lib.call("sa_linear_state", _ptr(proj), _code(proj), _rows(proj, "linear_state: proj"), int(q_at), int(k_at), int(v_at),
               float(q_mult), _ptr(gates), _rows(gates, "linear_state: gates"), _ptr(decay_bias),
               _code(decay_bias) if decay_bias is not None else 0, float(tau or 0.0), int(bool(scalar)), _ptr(bonus),
-              _code(bonus) if bonus is not None else 0, H, dk, dv,
+              _code(bonus) if bonus is not None else 0, _ptr(skip), _code(skip) if skip is not None else 0, H, key_heads, dk, dv,
               int(bool(ones)), _ptr(state), state.stride(0), _ptr(seq_meta), int(num_seqs), _ptr(out), _stream())
     return out
 
@@ -1672,6 +1678,98 @@ def concat_rows(x: torch.Tensor, y: torch.Tensor, out_dtype: torch.dtype) -> tor
 
 # --------------------------------------------------------------------------- routed experts
 
+def streams(x: torch.Tensor, *, y: "torch.Tensor | PartialSums | None" = None, mix: torch.Tensor | None = None,
+            out_weights: torch.Tensor | None = None, in_weights: torch.Tensor | None = None,
+            weight: torch.Tensor | None = None, eps: float = 0.0, rows: torch.Tensor | None = None,
+            out_dtype: torch.dtype = torch.float32) -> "tuple[torch.Tensor, torch.Tensor | None]":
+    """A residual of S parallel streams, x float32 [T, S, D] (a row expanded over the streams is fine).  With y [T, D] (the
+    activation type): stream q <- sum_s mix[s, q] x_s + out_weights[q] y, all at once from the old ones, in place (into
+    new memory where x is an expanded row).  With in_weights: z = u / sqrt(mean(u^2) + eps) * weight (weight None: z = u)
+    over u = sum_s in_weights[s] x_s of the updated streams, in out_dtype.  rows (int32, without y): of these tokens only.
+    mix [S, S], out_weights [S], in_weights [S]: float32.  Returns (streams, z or None)."""
+    if x.dim() != 3 or x.dtype != torch.float32 or (x.shape[2] > 1 and x.stride(2) != 1):
+        raise KernelError("streams: the streams are float32 [T, S, D] with contiguous rows")
+    T, S, D = x.shape
+    planes, yt = 0, y
+    if isinstance(y, PartialSums):
+        if y.planes is not None:
+            y.check_fresh()
+            planes, yt = y.planes.shape[0], y.planes
+        else:
+            yt = y.out
+    _dev(x, yt, mix, out_weights, in_weights, weight, rows)
+    for t, n in ((mix, S * S), (out_weights, S), (in_weights, S)):
+        if t is not None and (t.dtype != torch.float32 or t.numel() != n or not t.is_contiguous()):
+            raise KernelError(f"streams: weights of {S} streams are contiguous float32, [S, S] from stream to stream or [S]")
+    h, ys = x, 0
+    if y is not None:
+        if mix is None or out_weights is None or rows is not None or tuple(y.shape) != (T, D) or y.dtype != out_dtype:
+            raise KernelError("streams: an update takes y [T, D] in the activation type, mix and out weights, and all rows")
+        ys = D if planes else _rows(yt, "streams: y")
+        if planes and not yt.is_contiguous():
+            raise KernelError("streams: partial sums are contiguous")
+        if x.stride(1) == 0 or not x.is_contiguous():
+            h = torch.empty((T, S, D), dtype=torch.float32, device=x.device)
+    if weight is not None and (weight.numel() != D or not weight.is_contiguous()):
+        raise KernelError("streams: the norm weight does not match the width")
+    R, z = T, None
+    if rows is not None:
+        _i32(rows, "streams: rows")
+        R = rows.numel()
+    if in_weights is not None:
+        z = torch.empty((R, D), dtype=out_dtype, device=x.device)
+    x_row = x.stride(0) if T > 1 else max(x.stride(0), D)
+    _lib.call("sa_streams", _ptr(x), x_row, x.stride(1) if S > 1 else 0, _ptr(h) if y is not None else None, S, _ptr(yt),
+              _CODES[out_dtype], ys, planes, _ptr(mix), _ptr(out_weights), _ptr(in_weights), _ptr(weight),
+              _code(weight) if weight is not None else 0, float(eps), _ptr(rows), _ptr(z), _CODES[out_dtype], R, D, _stream())
+    return h, z
+
+
+def ssm_inputs(proj: torch.Tensor, x_at: int, dt_at: int, channels: int, num_heads: int, taps_by_tap: torch.Tensor,
+               bias: torch.Tensor, dt_bias: torch.Tensor, a_log: torch.Tensor, tails: torch.Tensor, seq_meta: torch.Tensor,
+               num_seqs: int, max_q_len: int) -> tuple[torch.Tensor, torch.Tensor]:
+    """What a state-space recurrence reads, from projection rows of a ragged step: columns x_at .. x_at + channels through a
+    causal convolution (taps_by_tap [taps, channels], oldest first; bias [channels]) and silu -> [T, channels] in proj's
+    type; tails float32 [slots, >= (taps - 1) * channels] are what earlier steps left, and are moved on.  Columns dt_at ..
+    dt_at + num_heads: dt = softplus(. + dt_bias), l = -exp(a_log) dt -> gates float32 [T, 3 H] = exp(l), dt, l."""
+    _dev(proj, taps_by_tap, bias, dt_bias, a_log, tails, seq_meta)
+    T, H, C = proj.shape[0], int(num_heads), int(channels)
+    stride = _rows(proj, "ssm_inputs: proj")
+    n = taps_by_tap.shape[0]
+    if tuple(taps_by_tap.shape) != (n, C) or not taps_by_tap.is_contiguous() or bias.numel() != C or not bias.is_contiguous() \
+            or bias.dtype != taps_by_tap.dtype:
+        raise KernelError(f"ssm_inputs: taps [taps, {C}] and a bias of their type expected")
+    if dt_bias.numel() != H or a_log.numel() != H or dt_bias.dtype != a_log.dtype or not dt_bias.is_contiguous() \
+            or not a_log.is_contiguous():
+        raise KernelError("ssm_inputs: dt_bias and a_log are of one type, one entry per head")
+    if proj.shape[1] < max(x_at + C, dt_at + H):
+        raise KernelError("ssm_inputs: the projection rows are too short")
+    if tails.dtype != torch.float32 or tails.dim() != 2 or tails.stride(1) != 1 or tails.shape[1] < (n - 1) * C:
+        raise KernelError("ssm_inputs: tails must be float32 [slots, >= (taps - 1) * channels]")
+    _seq_meta(seq_meta, num_seqs, "ssm_inputs")
+    y = torch.empty((T, C), dtype=proj.dtype, device=proj.device)
+    gates = torch.empty((T, 3 * H), dtype=torch.float32, device=proj.device)
+    _lib.call("sa_ssm_inputs", _ptr(proj), _code(proj), stride, int(x_at), int(dt_at), C, _ptr(taps_by_tap), _ptr(bias),
+              _code(bias), n, _ptr(dt_bias), _ptr(a_log), _code(a_log), _ptr(tails), tails.stride(0), _ptr(seq_meta),
+              int(num_seqs), int(max_q_len), _ptr(y), _ptr(gates), H, _stream())
+    return y, gates
+
+
+def gated_group_norm(y: torch.Tensor, z: torch.Tensor, groups: int, weight: torch.Tensor, eps: float) -> torch.Tensor:
+    """v = y * silu(z), then v / sqrt(mean(v^2) + eps) * weight in `groups` equal parts of the width, each by its own mean.
+    y float32 [T, width], z [T, width] in the activation type, which the result has."""
+    _dev(y, z, weight)
+    T, width = y.shape
+    if y.dtype != torch.float32 or tuple(z.shape) != (T, width) or width % groups or weight.numel() != width \
+            or not weight.is_contiguous():
+        raise KernelError(f"gated_group_norm: y float32 and z [T, width] with a weight per channel, {groups} equal groups")
+    out = torch.empty((T, width), dtype=z.dtype, device=y.device)
+    _lib.call("sa_gated_group_norm", _ptr(y), _rows(y, "gated_group_norm: y"), _ptr(z), _code(z),
+              _rows(z, "gated_group_norm: z"), _ptr(weight), _code(weight), float(eps), _ptr(out), int(groups), out.stride(0),
+              T, width, _stream())
+    return out
+
+
 def route(logits: torch.Tensor, top: int, scale: float) -> tuple[torch.Tensor, torch.Tensor]:
     """softmax over the experts' logits (float32 [T, E]); returns (experts int32 [T, top], weights float32 [T, top] =
     score * scale) of the `top` largest scores, largest first."""
@@ -1687,24 +1785,30 @@ def route(logits: torch.Tensor, top: int, scale: float) -> tuple[torch.Tensor, t
 
 
 def route_choice(logits: torch.Tensor, top: int, scale: float, *, correction: torch.Tensor | None = None,
-                 groups: int = 1, keep: int = 1, softmax: bool = False, group_best: int = 2,
-                 renorm: float | None = None) -> tuple[torch.Tensor, torch.Tensor]:
+                 groups: int = 1, keep: int = 1, softmax: "bool | str" = False, group_best: int = 2,
+                 renorm: float | None = None, bias: torch.Tensor | None = None) -> tuple[torch.Tensor, torch.Tensor]:
     """Scores are sigmoids of the logits (float32 [T, E]), or their softmax; the `top` experts with the largest score +
     correction[e] are chosen, among the `keep` groups (of `groups` equal groups of neighbouring experts) with the
     largest group scores: the sum of a group's two largest choice scores (group_best 2) or its largest (1).  Returns
     (experts int32 [T, top], weights float32 [T, top] = score * scale, the score without the correction, divided by the
-    chosen scores' sum + renorm unless renorm is None), largest choice first."""
-    _dev(logits, correction)
+    chosen scores' sum + renorm unless renorm is None), largest choice first.  softmax 'chosen': the scores are the logits
+    themselves, and the weights the softmax among the chosen ones.  bias [E]: added to the logits first."""
+    _dev(logits, correction, bias)
     T, E = logits.shape
     if logits.dtype != torch.float32:
         raise KernelError("route_choice: the router's logits are float32")
     if correction is not None and (correction.numel() != E or not correction.is_contiguous()):
         raise KernelError(f"route_choice: a correction of {correction.numel()} entries for {E} experts")
+    if bias is not None and (bias.numel() != E or not bias.is_contiguous()):
+        raise KernelError(f"route_choice: a bias of {bias.numel()} entries for {E} experts")
+    if softmax not in (False, True, "chosen") or (softmax == "chosen" and renorm is not None):
+        raise KernelError("route_choice: softmax is False, True or 'chosen' (whose weights sum to one: no renorm)")
     experts = torch.empty((T, top), dtype=torch.int32, device=logits.device)
     weights = torch.empty((T, top), dtype=torch.float32, device=logits.device)
     _lib.call("sa_route_choice", _ptr(logits), _rows(logits, "route_choice: logits"), T, E, int(top), float(scale),
+              _ptr(bias), _code(bias) if bias is not None else 0,
               _ptr(correction), _code(correction) if correction is not None else 0, int(groups), int(keep),
-              int(bool(softmax)), int(group_best), -1.0 if renorm is None else float(renorm), _ptr(experts), _ptr(weights),
+              2 if softmax == "chosen" else int(softmax), int(group_best), -1.0 if renorm is None else float(renorm), _ptr(experts), _ptr(weights),
               _stream())
     return experts, weights
 

@@ -15,6 +15,7 @@ from .. import parts as _parts  # noqa: F401  (registers the built-in parts)
 from ..config.spec import LayerSpec, ModelSpec, PartSpec
 from ..kernels import ops
 from ..parts.base import Block, ParamSpec, Part, PendingNorm
+from ..parts.streams import StreamSum, begin_streams
 from ..registry import BLOCKS, EMBEDDINGS, FEED_FORWARDS, HEADS, MIXERS, NORMS, PASS_INPUTS, STREAM_PARTS
 from ..weights import binding
 
@@ -38,6 +39,7 @@ class DecoderModel:
         self.final_norm = NORMS.build(spec.final_norm.kind, **spec.final_norm.params)
         self.pass_input = None if spec.pass_input is None else PASS_INPUTS.build(spec.pass_input.kind, **spec.pass_input.params)
         self.layers: list[Block] = [_build_layer(ls) for ls in spec.layers]
+        self.stream_sum = None if spec.streams is None else StreamSum(spec.streams)
         self.loaded = False
 
     # ------------------------------------------------------------------ tensors
@@ -46,6 +48,8 @@ class DecoderModel:
         if self.pass_input is not None:
             out.append((self.pass_input, self.spec.pass_input))
         for block, ls in zip(self.layers, self.spec.layers):
+            if ls.block.tensors:   # (a block arrangement with weights of its own)
+                out.append((block, ls.block))
             out.append((block.mixer, ls.mixer))
             if ls.feed_forward is not None:
                 out.append((block.feed_forward, ls.feed_forward))
@@ -101,6 +105,8 @@ class DecoderModel:
                 part.load(per_part.get(id(part), (part, {}))[1])
         finally:
             packing.clear_cache()   # sharing of re-laid tensors (tied table and head) ends with the load
+        if self.stream_sum is not None:
+            self.stream_sum.to_device(next(iter(tensors.values())).device)
         self.loaded = True
 
     # ------------------------------------------------------------------ cache
@@ -129,6 +135,8 @@ class DecoderModel:
         # a pass of a loop that is given the input again adds the embedding's output to the stream, or begins with a
         # part that reads both
         again = h.clone() if any(e.add_embedding or e.begins_pass is not None for e in schedule) else None
+        if self.stream_sum is not None:
+            h = begin_streams(h, self.spec.streams)
         normed = None
         for i, entry in enumerate(schedule):
             block = self.layers[entry.layer]
@@ -148,9 +156,11 @@ class DecoderModel:
             if after_layer is not None:
                 if isinstance(normed, PendingNorm):
                     h = normed.settle()
-                after_layer(i, h)
+                after_layer(i, h if self.stream_sum is None else self.stream_sum.plain(h))
         if logit_rows is None or logit_rows.numel() == 0:
             return None
+        if self.stream_sum is not None:
+            return self.head.forward(self.stream_sum.normed_rows(h, logit_rows, self.final_norm, ctx.dtype), out=logits_out)
         if isinstance(normed, PendingNorm):
             # the last block's residual sum is still pending: the final norm of the wanted rows comes out of the
             # same kernel (the residual stream itself is of no use to anyone after the last block)

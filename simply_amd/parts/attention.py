@@ -132,6 +132,8 @@ class SinkAttention(Mixer):
                                   if position_encoding is not None else None)
         if self.position_encoding is not None and not hasattr(self.position_encoding, "frequencies"):
             raise ValueError("sink_attention: the position encoding must give frequencies() (partial_rope)")
+        if getattr(self.position_encoding, "mult", 1.0) != 1.0:
+            raise ValueError("sink_attention: its kernel has no factor on the sines and cosines")
         self.in_proj = self.o_proj = self.sink = self.vmix = self.in_bias = self.o_bias = None
 
     def param_specs(self):

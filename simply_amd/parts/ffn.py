@@ -101,9 +101,11 @@ class RoutedExperts(FeedForward):
 
       gated       True: an expert is down(act(gate x) * (up x)); False: down(act(up x)), and there are no gate tensors
       activation  of the gated form also 'clamped_glu', with `limit` (`shared_limit` for the shared feed-forward)
-      router      scores (32-bit) are the softmax of the router's logits over all experts ('softmax') or sigmoids of the
-                  logits ('sigmoid'); the choice goes by score + a stored correction per expert (`correction`), and the
+      router      scores (32-bit) are the softmax of the router's logits over all experts ('softmax'), sigmoids of the
+                  logits ('sigmoid'), or ('chosen_softmax') the logits themselves, and the weights are then the softmax
+                  over the chosen experts' logits alone; the choice goes by score + a stored correction per expert (`correction`), and the
                   weights are the scores without the correction
+      router_bias a stored bias per expert, added to the logits (32-bit)
       num_groups  equal groups of neighbouring experts; only experts of the `keep_groups` best can be chosen.  A group's
                   score: `group_score` 'two_largest', the sum of its two largest choice scores, or 'largest'
       renormalize None, or a small constant e: the weights are the chosen scores divided by their sum + e
@@ -114,14 +116,16 @@ class RoutedExperts(FeedForward):
                  activation: str = "silu", shared_size: int | None = None, shared_gate: bool = True, gated: bool = True,
                  router: str = "softmax", correction: bool = False, num_groups: int = 1, keep_groups: int = 1,
                  group_score: str = "two_largest", renormalize: float | None = None, limit: float | None = None,
-                 shared_limit: float | None = None):
+                 shared_limit: float | None = None, router_bias: bool = False):
         self.hidden_size, self.num_experts, self.top = int(hidden_size), int(num_experts), int(top)
         self.expert_size, self.router_scale = int(expert_size), float(router_scale)
         if not 1 <= self.top <= self.num_experts:
             raise ValueError(f"routed_experts: top {top} of {num_experts} experts")
-        if router not in ("softmax", "sigmoid"):
-            raise ValueError(f"routed_experts: the router is 'softmax' or 'sigmoid', not {router!r}")
-        self.router_kind, self.correction = router, bool(correction)
+        if router not in ("softmax", "sigmoid", "chosen_softmax"):
+            raise ValueError(f"routed_experts: the router is 'softmax', 'sigmoid' or 'chosen_softmax', not {router!r}")
+        if router == "chosen_softmax" and renormalize is not None:
+            raise ValueError("routed_experts: weights that are the chosen logits' softmax sum to one by themselves")
+        self.router_kind, self.correction, self.router_bias = router, bool(correction), bool(router_bias)
         self.num_groups, self.keep_groups = int(num_groups), int(keep_groups)
         if group_score not in ("two_largest", "largest"):
             raise ValueError(f"routed_experts: a group's score is its 'two_largest' or its 'largest', not {group_score!r}")
@@ -140,13 +144,15 @@ class RoutedExperts(FeedForward):
         elif shared_size:
             self.shared = Dense(hidden_size, int(shared_size), activation)
         self.shared_gate = bool(shared_gate) and self.shared is not None
-        self.router = self.gate_w = self.up_w = self.down_w = self.correction_w = None
+        self.router = self.gate_w = self.up_w = self.down_w = self.correction_w = self.router_bias_w = None
 
     def param_specs(self):
         D, F, E = self.hidden_size, self.expert_size, self.num_experts
         specs = {"router": ParamSpec((E, D))}
         if self.correction:
             specs["correction"] = ParamSpec((E,), role="vector", init="norm")
+        if self.router_bias:
+            specs["router_bias"] = ParamSpec((E,), role="vector", init="norm")
         for e in range(E):
             if self.gated:
                 specs[f"e{e}.gate"] = ParamSpec((F, D))
@@ -168,18 +174,21 @@ class RoutedExperts(FeedForward):
         self.up_w = stack_experts(tensors[f"e{e}.up"] for e in range(E))
         self.down_w = stack_experts(tensors[f"e{e}.down"] for e in range(E))
         self.correction_w = tensors["correction"].contiguous() if self.correction else None
+        self.router_bias_w = tensors["router_bias"].contiguous() if self.router_bias else None
         if self.shared is not None:
             self.shared.load({n: tensors["shared." + n] for n in self.shared.param_specs()})
 
     def forward(self, x: torch.Tensor, ctx=None) -> torch.Tensor:
         E = self.num_experts
         logits = ops.gemm(x, self.router, out_dtype=torch.float32)
-        plain = self.router_kind == "softmax" and not self.correction and self.num_groups == 1 and self.renormalize is None
+        plain = self.router_kind == "softmax" and not self.correction and self.num_groups == 1 and self.renormalize is None \
+            and not self.router_bias
         if not plain:
             experts, weights = ops.route_choice(logits[:, :E], self.top, self.router_scale, correction=self.correction_w,
                                                 groups=self.num_groups, keep=self.keep_groups,
-                                                softmax=self.router_kind == "softmax", group_best=self.group_best,
-                                                renorm=self.renormalize)
+                                                softmax={"softmax": True, "sigmoid": False}.get(self.router_kind, "chosen"),
+                                                group_best=self.group_best, renorm=self.renormalize,
+                                                bias=self.router_bias_w)
         else:
             experts, weights = ops.route(logits[:, :E], self.top, self.router_scale)
         shared = self.shared.forward(x, ctx) if self.shared is not None else None

@@ -9,7 +9,7 @@ the scores:
                   heads share; 'row': by the root mean square of the whole projection (all heads at once), times a
                   weight per entry; None: no norm
   position_encoding  'partial_rope': the first entries of every head of q and k turn in pairs (i, i + dims / 2),
-                  after the norm
+                  after the norm (with the encoding's factor on sines and cosines, if it has one)
   query_temperature  (coef, every): the query at position p times 1 + coef ln(floor((p + 1) / every) + 1)
   values          'projected': a projection of their own; 'keys': the keys as projected (before norm and rotation) are
                   the values, and there is no value projection
@@ -175,7 +175,7 @@ class GatedAttention(Mixer):
                                  in_bias=self.in_bias if bias_later else None,
                                  tails=state, norm=self.qk_norm,
                                  q_weight=self.q_norm, k_weight=self.k_norm, eps=self.norm_eps, inv_freq=inv_freq,
-                                 rot_dims=rot_dims, temp_coef=coef, temp_every=every, q_mult=self.scale if mfma else 1.0,
+                                 rot_dims=rot_dims, rot_mult=getattr(pe, "mult", 1.0), temp_coef=coef, temp_every=every, q_mult=self.scale if mfma else 1.0,
                                  slot_mapping=group.slot_mapping if self.own else None,
                                  k_pages=pages.k_pages if self.own else None, v_pages=pages.v_pages if self.own else None)
         if mfma:
@@ -187,6 +187,13 @@ class GatedAttention(Mixer):
                 ops.paged_attention_decode(q, pages.k_pages, pages.v_pages, group.block_table, units, 0, few, H, **kw)
             if many:
                 ops.paged_attention_prefill(q, pages.k_pages, pages.v_pages, group.block_table, units, few, many, H, **kw)
+        elif self.sinks is None and self.slopes is None and \
+                ops.attention_maps_units_takes(q, pages.k_pages, pages.v_pages, H):
+            # bfloat16 with values of a size of their own: the matrix-core kernel whose sizes are launch arguments
+            units, few, many, max_q = ctx.attention_units(16 // ops.attention_maps_heads_per_unit(H, K))
+            o = ops.paged_attention_maps_units(q, pages.k_pages, pages.v_pages, group.block_table, units, 0, few + many, H,
+                                               scale=self.scale, window=self.window, max_kv_len=ctx.max_kv_len,
+                                               max_q_len=max_q)
         else:
             o = ops.paged_attention_sink(q, pages.k_pages, pages.v_pages, group.block_table, ctx.token_seq,
                                          ctx.positions, H, scale=self.scale, sinks=self.sinks, slopes=self.slopes,

@@ -21,7 +21,7 @@ STAND_INS = ("embed", "rmsnorm", "add_rmsnorm", "rope_cache_write", "rope", "gat
              "exp_gates", "linear_state", "normalized_readout", "route", "routed_experts", "residual_add_next_norm",
              "paged_attention_maps", "attention_maps_units_takes", "norm_rope_cache_write", "short_conv",
              "head_product", "rglru_scan", "attention_inputs", "route_choice", "token_shift", "low_rank_decay",
-             "concat_rows", "gemm_sections")
+             "concat_rows", "gemm_sections", "streams", "ssm_inputs", "gated_group_norm")
 
 EPILOGUE_NONE, EPILOGUE_GATED_GELU, EPILOGUE_SOFT_CAP = 0, 1, 2
 ALGO_AUTO, ALGO_GENERIC, ALGO_SKINNY, ALGO_TILED = 0, 1, 2, 3
@@ -560,7 +560,7 @@ def exp_gates(raw, bias, cap, num_heads, m_state, seq_meta, num_seqs):
 
 
 def linear_state(proj, q_at, k_at, v_at, q_mult, gates, scalar, num_heads, key_dim, value_dim, ones, state, seq_meta,
-                 num_seqs, *, decay_bias=None, tau=None, bonus=None):
+                 num_seqs, *, decay_bias=None, tau=None, bonus=None, key_heads=None, skip=None):
     H, dk, dv = num_heads, key_dim, value_dim
     if tau is not None:   # the gates are z: a = sigmoid(z + bias)^(1 / tau)
         z = _f(gates) + (_f(decay_bias) if decay_bias is not None else 0.0)
@@ -572,8 +572,9 @@ def linear_state(proj, q_at, k_at, v_at, q_mult, gates, scalar, num_heads, key_d
     for slot, first, count, _ in seq_meta[:num_seqs].tolist():
         S = _f(state[slot, :H * dk * CT]).view(H, CT, dk).clone()   # column by column
         for t in range(first, first + count):
-            q = p[t, q_at:q_at + H * dk].view(H, dk) * q_mult
-            k = p[t, k_at:k_at + H * dk].view(H, dk)
+            G = key_heads or H
+            q = p[t, q_at:q_at + G * dk].view(G, dk).repeat_interleave(H // G, 0) * q_mult
+            k = p[t, k_at:k_at + G * dk].view(G, dk).repeat_interleave(H // G, 0)
             v = p[t, v_at:v_at + H * dv].view(H, dv)
             if ones:
                 v = torch.cat([v, torch.ones((H, 1), dtype=v.dtype, device=v.device)], dim=1)
@@ -585,6 +586,8 @@ def linear_state(proj, q_at, k_at, v_at, q_mult, gates, scalar, num_heads, key_d
             read = S + _f(bonus).view(H, 1, dk) * kv if bonus is not None else a * S + kv
             S = a * S + kv
             out[t] = torch.einsum("hcd,hd->hc", read, q).reshape(-1)
+            if skip is not None:
+                out[t] += (_f(skip)[:, None] * v).reshape(-1)
         if count > 0:
             state[slot, :H * dk * CT] = S.reshape(-1).to(torch.float32)
     return out.to(torch.float32)
@@ -607,8 +610,10 @@ def route(logits, top, scale):
     return best.indices.to(torch.int32).contiguous(), (best.values * scale).to(torch.float32).contiguous()
 
 
-def route_choice(logits, top, scale, *, correction=None, groups=1, keep=1, softmax=False, group_best=2, renorm=None):
-    s = torch.softmax(_f(logits), -1) if softmax else torch.sigmoid(_f(logits))
+def route_choice(logits, top, scale, *, correction=None, groups=1, keep=1, softmax=False, group_best=2, renorm=None,
+                 bias=None):
+    z = _f(logits) + (_f(bias) if bias is not None else 0.0)
+    s = z if softmax == "chosen" else torch.softmax(z, -1) if softmax else torch.sigmoid(z)
     T, E = s.shape
     c = s + _f(correction) if correction is not None else s.clone()
     if groups > 1:
@@ -620,6 +625,8 @@ def route_choice(logits, top, scale, *, correction=None, groups=1, keep=1, softm
         c = torch.where(stay[:, :, None].expand(T, groups, per).reshape(T, E), c, torch.full_like(c, float("-inf")))
     chosen = torch.topk(c, top, dim=-1).indices
     w = torch.gather(s, 1, chosen)
+    if softmax == "chosen":
+        w = torch.softmax(w, -1)
     if renorm is not None:
         w = w / (w.sum(-1, keepdim=True) + renorm)
     return chosen.to(torch.int32).contiguous(), (w * scale).to(torch.float32).contiguous()
@@ -810,7 +817,7 @@ def rglru_scan(u, gates, block, r_bias, i_bias, lam, y, y_bias, state, seq_meta,
 
 def attention_inputs(proj, seq_meta, num_seqs, max_q_len, num_heads, num_kv_heads, key_dim, value_dim, *,
                      values_are_keys=False, taps=None, tails=None, norm=None, q_weight=None, k_weight=None, eps=0.0,
-                     inv_freq=None, rot_dims=0, temp_coef=0.0, temp_every=0, q_mult=1.0, taps_by_tap=None, in_bias=None,
+                     inv_freq=None, rot_dims=0, rot_mult=1.0, temp_coef=0.0, temp_every=0, q_mult=1.0, taps_by_tap=None, in_bias=None,
                      slot_mapping=None, k_pages=None, v_pages=None):
     H, K, dk, dv = num_heads, num_kv_heads, key_dim, value_dim
     own = k_pages is not None
@@ -842,7 +849,7 @@ def attention_inputs(proj, seq_meta, num_seqs, max_q_len, num_heads, num_kv_head
         if rot_dims:
             half = rot_dims // 2
             a = pos.to(torch.float32)[:, None] * inv_freq.to(torch.float32)[None, :]
-            cos, sin = torch.cos(a).to(v.dtype)[:, None, :], torch.sin(a).to(v.dtype)[:, None, :]
+            cos, sin = rot_mult * torch.cos(a).to(v.dtype)[:, None, :], rot_mult * torch.sin(a).to(v.dtype)[:, None, :]
             u, w_ = v[..., :half], v[..., half:rot_dims]
             v = torch.cat([u * cos - w_ * sin, w_ * cos + u * sin, v[..., rot_dims:]], dim=-1)
         return v
@@ -892,3 +899,42 @@ def concat_rows(x, y, out_dtype):
 def gemm_sections(a, w):
     S, K = len(w.parts), w.cols
     return torch.cat([gemm(a[:, s * K:(s + 1) * K], w.parts[s]) for s in range(S)], dim=1)
+
+
+# --------------------------------------------------------------------------- streams, state-space mixers
+
+
+def streams(x, *, y=None, mix=None, out_weights=None, in_weights=None, weight=None, eps=0.0, rows=None,
+            out_dtype=torch.float32):
+    v = _f(x)
+    h = x
+    if y is not None:
+        yv = _f(y.materialize() if hasattr(y, "materialize") else y)
+        v = torch.einsum("tsd,sq->tqd", v, _f(mix).reshape(v.shape[1], v.shape[1])) + _f(out_weights)[None, :, None] * yv[:, None]
+        h = v.to(torch.float32)
+        v = _f(h)
+        if x.is_contiguous():
+            x.copy_(h)
+            h = x
+    z = None
+    if in_weights is not None:
+        u = (v if rows is None else v[rows.long()]).mul(_f(in_weights)[None, :, None]).sum(1)
+        if weight is not None:
+            u = u / torch.sqrt((u * u).mean(-1, keepdim=True) + eps) * _f(weight)
+        z = u.to(out_dtype)
+    return h, z
+
+
+def ssm_inputs(proj, x_at, dt_at, channels, num_heads, taps_by_tap, bias, dt_bias, a_log, tails, seq_meta, num_seqs,
+               max_q_len):
+    y = short_conv(proj[:, x_at:x_at + channels], taps_by_tap.t(), tails, seq_meta, num_seqs, max_q_len, out_bias=bias,
+                   silu=True)
+    dt = torch.nn.functional.softplus(_f(proj[:, dt_at:dt_at + num_heads]) + _f(dt_bias), threshold=30.0)
+    log_decay = -torch.exp(_f(a_log)) * dt
+    return y.to(proj.dtype), torch.cat([torch.exp(log_decay), dt, log_decay], -1).to(torch.float32)
+
+
+def gated_group_norm(y, z, groups, weight, eps):
+    v = (_f(y) * silu(_f(z))).reshape(y.shape[0], groups, -1)
+    v = v / torch.sqrt((v * v).mean(-1, keepdim=True) + eps)
+    return (v.reshape(y.shape) * _f(weight)).to(z.dtype)
