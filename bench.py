@@ -677,6 +677,63 @@ def run_kolorax(args):
             torch.cuda.empty_cache()
 
 
+# --only nozizen: layer sizes that resemble a real model's, for the Nozizen design (in turn a layer with the token-shift
+# recurrence, two with the state-space recurrence of twice the width in heads of 64 with a state of 128, one with attention
+# behind a window; dense feed-forwards and routed experts of a quarter of the dense size in turn, three of 16 chosen; four
+# residual streams; layers 2 and 3 looped twice) and, beside it, the closest model that the engine has, Kolorax, at equal
+# width, depth, heads and head size, with the same loop
+NOZIZEN_WINDOW = 1024
+
+
+def nozizen_config(size: dict, layers: int) -> dict:
+    W, H, K, d, ff = size["width"], size["heads"], size["kv_heads"], size["dim"], size["ff"]
+    out = []
+    for i in range(layers):
+        mlp = {"kind": "dense", "ff": ff} if i % 2 == 0 else \
+            {"kind": "moe", "expert": {"ff": ff // 4}, "router": {"experts": 16, "top": 3}}
+        if i % 4 == 0:
+            out.append({"type": "wkv", "mlp": mlp, "mixer": {"heads": H, "dim": d, "rank": 64}})
+        elif i % 4 == 3:
+            out.append({"type": "attention", "mlp": mlp,
+                        "mixer": {"heads": H, "kv_heads": K, "dim": d, "vdim": d, "scale": d ** -0.5,
+                                  "mask": {"size": NOZIZEN_WINDOW},
+                                  "rot": {"dims": d, "base": 50000.0,
+                                          "scaling": {"factor": 8.0, "original": 4096, "fast": 32.0, "slow": 1.0}}}})
+        else:
+            out.append({"type": "mamba2", "mlp": mlp,
+                        "mixer": {"heads": 2 * W // 64, "vdim": 64, "state": 128, "groups": 8, "conv": 4, "norm_groups": 8}})
+    d = {"architecture": "Nozizen", "vocab": size["vocab"], "width": W, "streams": 4, "norm": {"eps": 1e-5},
+         "embedding": {"scale": 1.0}, "layers": out}
+    if layers >= KOLORAX_LOOP["stop"]:
+        d["loop"] = dict(KOLORAX_LOOP)
+    return d
+
+
+def run_nozizen(args):
+    import torch
+    from simply_amd.config import config_from_dict
+    from simply_amd.engine.loading import random_model
+
+    tdtype = torch.bfloat16 if args.dtype == "bfloat16" else torch.float32
+    layers = args.layers or 8
+    for name in args.sizes.split(","):
+        size = ZENUZEN_SIZES[name]
+        for label, d in (("nozizen", nozizen_config(size, layers)), ("kolorax-equal-size", kolorax_config(size, layers))):
+            if args.alone and label != "nozizen":
+                continue
+            model = random_model(config_from_dict(d), 0, tdtype, torch.device("cuda:0"), std=0.02)
+            pt, dt = run_executor_bench(model, size["vocab"], args.prefill_tokens, args.batch, args.context, args.steps,
+                                        args.warmup, args.page_size, args.dtype)
+            print(json.dumps({"metric": "prefill and decode tokens/s through the step function", "model": label,
+                              "size": name, "width": size["width"], "layers": layers, "layer_runs": len(model.spec.schedule),
+                              "prefill_tokens": args.prefill_tokens, "prefill_tokens_per_s": round(args.prefill_tokens / pt, 1),
+                              "prefill_ms": round(pt * 1e3, 3), "batch": args.batch, "context": args.context,
+                              "decode_tokens_per_s": round(args.batch / dt, 1), "decode_ms_per_step": round(dt * 1e3, 3),
+                              "dtype": args.dtype, "data": "synthetic"}), flush=True)
+            del model
+            torch.cuda.empty_cache()
+
+
 def main():
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -693,7 +750,7 @@ def main():
     ap.add_argument("--contexts", default="1024,4096,8192", help="--only decode-grid: the context lengths")
     ap.add_argument("--only", default="all", choices=["all", "decode", "decode-grid", "prefill", "prefill-chunked", "products",
                                                       "gated-products", "ceilings", "zenuzen", "nemidra", "tabupel",
-                                                      "rudutar", "kolorax"],
+                                                      "rudutar", "kolorax", "nozizen"],
                     help="measure one part alone (for profiles); the line then holds that part only.  products / "
                          "gated-products: the sweep of the product kernels over rows and weight sizes; ceilings: "
                          "what the GPU itself reaches in reading HBM and in bfloat16 MFMA instructions")
@@ -701,8 +758,8 @@ def main():
                     help="decode steps run one at a time after the timed ones, for the p50 and p99 of a step's latency")
     ap.add_argument("--shape", default="2b", choices=sorted(SHAPES), help="layer sizes: Gemma 2 2B (the default), 9B, 27B")
     ap.add_argument("--sizes", default="small,medium,large",
-                    help="--only zenuzen / nemidra / tabupel / rudutar / kolorax: which of the layer sizes small, medium, large (8 layers each, or --layers)")
-    ap.add_argument("--alone", action="store_true", help="--only nemidra / tabupel / rudutar / kolorax: without the closest model beside it (for profiles)")
+                    help="--only zenuzen / nemidra / tabupel / rudutar / kolorax / nozizen: which of the layer sizes small, medium, large (8 layers each, or --layers)")
+    ap.add_argument("--alone", action="store_true", help="--only nemidra / tabupel / rudutar / kolorax / nozizen: without the closest model beside it (for profiles)")
     ap.add_argument("--alone-model", default="kolorax", choices=["kolorax", "nemidra-equal-size"],
                     help="--only kolorax --alone: which of the two models runs")
     ap.add_argument("--requests", type=int, default=0,
@@ -742,6 +799,9 @@ def main():
         return
     if args.only == "kolorax":
         run_kolorax(args)
+        return
+    if args.only == "nozizen":
+        run_nozizen(args)
         return
     d = dict(GEMMA2_2B, **SHAPES[args.shape])
     full_layers = d["num_hidden_layers"]

@@ -476,6 +476,14 @@ int sa_linear_state(const void* proj, int dtype, int64_t proj_stride, int q_at, 
                     const void* bonus, int bonus_dtype, const void* skip, int skip_dtype, int H, int key_heads, int dk, int dv,
                     int ones, float* state, int64_t state_stride, const int* seq_meta, int num_seqs, float* out,
                     hipStream_t stream);
+// sa_linear_state with scalar = 1, ones = 0, q_mult = 1 for requests that bring many tokens, 64 at a time on the matrix cores
+// (state_chunks.hip).  gates [T, >= 3 H]: decays, input factors, the decays' logarithms (the first are not read).
+// sa_state_chunks_takes: key sizes up to 128 in multiples of 8, value sizes in multiples of 4, columns and rows of proj in
+// multiples of 8, state rows in multiples of 4.
+int sa_state_chunks_takes(int dk, int dv, int q_at, int k_at, int v_at, int64_t proj_stride, int64_t state_stride);
+int sa_state_chunks(const void* proj, int dtype, int64_t proj_stride, int q_at, int k_at, int v_at, const float* gates,
+                    int64_t gates_stride, const void* skip, int skip_dtype, int H, int key_heads, int dk, int dv, float* state,
+                    int64_t state_stride, const int* seq_meta, int num_seqs, float* out, hipStream_t stream);
 // x [T, H, size + 1] -> out[t, h, :] = unit_rms(x[t, h, :size] / (max(|x[t, h, size]|, floor[t, h]) + 1e-6)) * w[h, :]
 // * sigmoid(g[t, h, :]).
 int sa_normalized_readout(const float* x, const float* floor, int64_t floor_stride, const void* g, int g_dtype,

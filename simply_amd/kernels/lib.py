@@ -97,6 +97,8 @@ _SIGNATURES = {
     "sa_token_shift": [_P, _I, _L, _P, _I, _I, _P, _L, _P, _I, _I, _P, _I, _P],
     "sa_low_rank_decay": [_P, _I, _L, _P, _I, _I, _P, _I, _P, _I, _I, _I, _P],
     "sa_gemm_sections": [_P, _L, _P, _P, _I, _L, _I, _I, _I, _I, _I, _P, _L, _P],
+    "sa_state_chunks_takes": [_I, _I, _I, _I, _I, _L, _L],
+    "sa_state_chunks": [_P, _I, _L, _I, _I, _I, _P, _L, _P, _I, _I, _I, _I, _I, _P, _L, _P, _I, _P, _P],
     "sa_streams": [_P, _L, _L, _P, _I, _P, _I, _L, _I, _P, _P, _P, _P, _I, _F, _P, _P, _I, _I, _I, _P],
     "sa_ssm_inputs": [_P, _I, _L, _I, _I, _I, _P, _P, _I, _I, _P, _P, _I, _P, _L, _P, _I, _I, _P, _P, _I, _P],
     "sa_gated_group_norm": [_P, _L, _P, _I, _L, _P, _I, _F, _P, _I, _L, _I, _I, _P],

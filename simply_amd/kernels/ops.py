@@ -1571,7 +1571,7 @@ def linear_state(proj: torch.Tensor, q_at: int, k_at: int, v_at: int, q_mult: fl
                  num_heads: int, key_dim: int, value_dim: int, ones: bool, state: torch.Tensor, seq_meta: torch.Tensor,
                  num_seqs: int, *, decay_bias: torch.Tensor | None = None, tau: float | None = None,
                  bonus: torch.Tensor | None = None, key_heads: int | None = None,
-                 skip: torch.Tensor | None = None) -> torch.Tensor:
+                 skip: torch.Tensor | None = None, out: torch.Tensor | None = None) -> torch.Tensor:
     """S <- diag(a) S + c k v^T, o = S^T (q * q_mult) along each request's tokens, from and into state float32 [slots,
     >= H * dk * (dv + ones)] (per head [dv + ones][dk]).  q, k, v: columns q_at, k_at, v_at of proj's rows, H heads
     each.  scalar: gates float32 [T, >= 2 H] hold a and c per head; else [T, H * dk] hold a per key channel, c = 1;
@@ -1579,7 +1579,7 @@ def linear_state(proj: torch.Tensor, q_at: int, k_at: int, v_at: int, q_mult: fl
     bonus [H * dk] (decays per key channel): o = (S_before + diag(bonus) k v^T)^T q, the state before the token.
     ones: one more column whose value is always 1 (a normalizer).  key_heads (with scalar): q and k have that many heads,
     each shared by H / key_heads neighbouring ones; skip [H] (with scalar, without ones): o += skip * v.  Returns float32
-    [T, H * (dv + ones)]."""
+    [T, H * (dv + ones)] (out: written where the requests of seq_meta have their rows)."""
     _dev(proj, gates, state, seq_meta, skip)
     T = proj.shape[0]
     H, dk, dv, CT = int(num_heads), int(key_dim), int(value_dim), int(value_dim) + int(bool(ones))
@@ -1598,12 +1598,49 @@ def linear_state(proj: torch.Tensor, q_at: int, k_at: int, v_at: int, q_mult: fl
     if skip is not None and (not scalar or ones or skip.numel() != H or not skip.is_contiguous()):
         raise KernelError("linear_state: a skip has one entry per head and goes with decays per head, without a normalizer")
     _dev(decay_bias, bonus)
-    out = torch.empty((T, H * CT), dtype=torch.float32, device=proj.device)
+    if out is None:
+        out = torch.empty((T, H * CT), dtype=torch.float32, device=proj.device)
+    elif out.dtype != torch.float32 or tuple(out.shape) != (T, H * CT) or not out.is_contiguous():
+        raise KernelError("linear_state: out must be contiguous float32 [T, H * (dv + ones)]")
     _lib.call("sa_linear_state", _ptr(proj), _code(proj), _rows(proj, "linear_state: proj"), int(q_at), int(k_at), int(v_at),
               float(q_mult), _ptr(gates), _rows(gates, "linear_state: gates"), _ptr(decay_bias),
               _code(decay_bias) if decay_bias is not None else 0, float(tau or 0.0), int(bool(scalar)), _ptr(bonus),
               _code(bonus) if bonus is not None else 0, _ptr(skip), _code(skip) if skip is not None else 0, H, key_heads, dk, dv,
               int(bool(ones)), _ptr(state), state.stride(0), _ptr(seq_meta), int(num_seqs), _ptr(out), _stream())
+    return out
+
+
+def state_chunks_takes(proj: torch.Tensor, q_at: int, k_at: int, v_at: int, key_dim: int, value_dim: int,
+                       state: torch.Tensor) -> bool:
+    """Whether `state_chunks` takes these sizes (key sizes up to 128 in multiples of 8, value sizes in multiples of 4, aligned
+    columns and rows)."""
+    return bool(_lib.load().sa_state_chunks_takes(int(key_dim), int(value_dim), int(q_at), int(k_at), int(v_at),
+                                                  _rows(proj, "state_chunks: proj"), state.stride(0))) \
+        and proj.data_ptr() % 16 == 0 and state.data_ptr() % 16 == 0
+
+
+def state_chunks(proj: torch.Tensor, q_at: int, k_at: int, v_at: int, gates: torch.Tensor, num_heads: int, key_heads: int,
+                 key_dim: int, value_dim: int, state: torch.Tensor, seq_meta: torch.Tensor, num_seqs: int, *,
+                 skip: torch.Tensor | None = None, out: torch.Tensor | None = None) -> torch.Tensor:
+    """`linear_state` with a decay and an input factor per head (scalar, no normalizer, q_mult 1) for requests that bring
+    many tokens: 64 at a time on the matrix cores, the state in 32-bit.  gates float32 [T, >= 3 H]: decays (not read), input
+    factors, the decays' logarithms."""
+    _dev(proj, gates, state, seq_meta, skip, out)
+    T, H, dk, dv = proj.shape[0], int(num_heads), int(key_dim), int(value_dim)
+    if gates.dtype != torch.float32 or gates.shape[0] != T:
+        raise KernelError("state_chunks: gates must be float32 with one row per token")
+    if state.dtype != torch.float32 or state.dim() != 2 or state.stride(1) != 1 or state.shape[1] < H * dk * dv:
+        raise KernelError("state_chunks: the state must be float32 [slots, >= H * dk * dv]")
+    if skip is not None and (skip.numel() != H or not skip.is_contiguous()):
+        raise KernelError("state_chunks: a skip has one entry per head")
+    _seq_meta(seq_meta, num_seqs, "state_chunks")
+    if out is None:
+        out = torch.empty((T, H * dv), dtype=torch.float32, device=proj.device)
+    elif out.dtype != torch.float32 or tuple(out.shape) != (T, H * dv) or not out.is_contiguous():
+        raise KernelError("state_chunks: out must be contiguous float32 [T, H * dv]")
+    _lib.call("sa_state_chunks", _ptr(proj), _code(proj), _rows(proj, "state_chunks: proj"), int(q_at), int(k_at), int(v_at),
+              _ptr(gates), _rows(gates, "state_chunks: gates"), _ptr(skip), _code(skip) if skip is not None else 0, H,
+              int(key_heads), dk, dv, _ptr(state), state.stride(0), _ptr(seq_meta), int(num_seqs), _ptr(out), _stream())
     return out
 
 

@@ -23,6 +23,8 @@ class StateSpace(Mixer):
     #: the mixer's input enters one product only: for a few rows the norm in front of it runs in that product's kernel
     accepts_pending = True
     defers_sum = True
+    #: tokens of a request in a step from which the recurrence is worked through in pieces
+    PIECES_FROM = 12
 
     def __init__(self, hidden_size: int, num_heads: int, num_groups: int, state_dim: int, value_dim: int, conv_taps: int,
                  norm_groups: int, norm_eps: float):
@@ -77,8 +79,17 @@ class StateSpace(Mixer):
         u, gates = ops.ssm_inputs(proj, inner, inner + self.channels, self.channels, H, self.taps, self.conv_bias,
                                   self.dt_bias, self.a_log, cache.state[:, self.tails_at:], ctx.seq_meta, ctx.num_seqs,
                                   ctx.max_q_len)
-        # queries C, keys B, values x; a decay and an input factor (the step size) per head
-        y = ops.linear_state(u, inner + G * N, inner, 0, 1.0, gates, True, H, N, dv, False, cache.state, ctx.seq_meta,
-                             ctx.num_seqs, key_heads=G, skip=self.skip)
+        # queries C, keys B, values x; a decay and an input factor (the step size) per head.  Requests with few tokens go
+        # through the recurrence token by token, portions of prompts in pieces on the matrix cores where these take the sizes
+        at = (inner + G * N, inner, 0)
+        y = torch.empty((u.shape[0], inner), dtype=torch.float32, device=u.device)
+        short = ctx.num_seqs
+        if ctx.max_q_len >= self.PIECES_FROM and ops.state_chunks_takes(u, *at, N, dv, cache.state):
+            short, _ = ctx.short_requests(self.PIECES_FROM - 1)
+            ops.state_chunks(u, *at, gates, H, G, N, dv, cache.state, ctx.seq_meta[short:], ctx.num_seqs - short,
+                             skip=self.skip, out=y)
+        if short:
+            ops.linear_state(u, *at, 1.0, gates, True, H, N, dv, False, cache.state, ctx.seq_meta, short, key_heads=G,
+                             skip=self.skip, out=y)
         z = ops.gated_group_norm(y, proj[:, :inner], self.norm_groups, self.norm, self.norm_eps)
         return ops.gemm(z, self.o_proj, defer_sum=defer_sum)

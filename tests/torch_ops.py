@@ -21,7 +21,8 @@ STAND_INS = ("embed", "rmsnorm", "add_rmsnorm", "rope_cache_write", "rope", "gat
              "exp_gates", "linear_state", "normalized_readout", "route", "routed_experts", "residual_add_next_norm",
              "paged_attention_maps", "attention_maps_units_takes", "norm_rope_cache_write", "short_conv",
              "head_product", "rglru_scan", "attention_inputs", "route_choice", "token_shift", "low_rank_decay",
-             "concat_rows", "gemm_sections", "streams", "ssm_inputs", "gated_group_norm")
+             "concat_rows", "gemm_sections", "streams", "ssm_inputs", "gated_group_norm",
+             "state_chunks_takes", "state_chunks")
 
 EPILOGUE_NONE, EPILOGUE_GATED_GELU, EPILOGUE_SOFT_CAP = 0, 1, 2
 ALGO_AUTO, ALGO_GENERIC, ALGO_SKINNY, ALGO_TILED = 0, 1, 2, 3
@@ -560,7 +561,7 @@ def exp_gates(raw, bias, cap, num_heads, m_state, seq_meta, num_seqs):
 
 
 def linear_state(proj, q_at, k_at, v_at, q_mult, gates, scalar, num_heads, key_dim, value_dim, ones, state, seq_meta,
-                 num_seqs, *, decay_bias=None, tau=None, bonus=None, key_heads=None, skip=None):
+                 num_seqs, *, decay_bias=None, tau=None, bonus=None, key_heads=None, skip=None, out=None):
     H, dk, dv = num_heads, key_dim, value_dim
     if tau is not None:   # the gates are z: a = sigmoid(z + bias)^(1 / tau)
         z = _f(gates) + (_f(decay_bias) if decay_bias is not None else 0.0)
@@ -568,7 +569,7 @@ def linear_state(proj, q_at, k_at, v_at, q_mult, gates, scalar, num_heads, key_d
     CT = dv + int(bool(ones))
     T = proj.shape[0]
     p, g = _f(proj), _f(gates)
-    out = torch.zeros((T, H * CT), dtype=p.dtype, device=proj.device)
+    into, out = out, torch.zeros((T, H * CT), dtype=p.dtype, device=proj.device)
     for slot, first, count, _ in seq_meta[:num_seqs].tolist():
         S = _f(state[slot, :H * dk * CT]).view(H, CT, dk).clone()   # column by column
         for t in range(first, first + count):
@@ -590,7 +591,43 @@ def linear_state(proj, q_at, k_at, v_at, q_mult, gates, scalar, num_heads, key_d
                 out[t] += (_f(skip)[:, None] * v).reshape(-1)
         if count > 0:
             state[slot, :H * dk * CT] = S.reshape(-1).to(torch.float32)
-    return out.to(torch.float32)
+            if into is not None:
+                into[first:first + count] = out[first:first + count].to(torch.float32)
+    return out.to(torch.float32) if into is None else into
+
+
+def state_chunks_takes(proj, q_at, k_at, v_at, key_dim, value_dim, state):
+    return key_dim % 8 == 0 and value_dim % 4 == 0
+
+
+def state_chunks(proj, q_at, k_at, v_at, gates, num_heads, key_heads, key_dim, value_dim, state, seq_meta, num_seqs, *,
+                 skip=None, out=None, piece=64):
+    """In pieces, as the kernel does it: within one the tokens' weights, between them the state."""
+    H, dk, dv, G = num_heads, key_dim, value_dim, key_heads
+    p, g = _f(proj), _f(gates)
+    if out is None:
+        out = torch.empty((proj.shape[0], H * dv), dtype=torch.float32, device=proj.device)
+    for slot, first, count, _ in seq_meta[:num_seqs].tolist():
+        S = _f(state[slot, :H * dk * dv]).view(H, dv, dk).clone()
+        for at in range(first, first + count, piece):
+            n = min(piece, first + count - at)
+            rows = p[at:at + n]
+            q = rows[:, q_at:q_at + G * dk].view(n, G, dk).repeat_interleave(H // G, 1)
+            k = rows[:, k_at:k_at + G * dk].view(n, G, dk).repeat_interleave(H // G, 1)
+            v = rows[:, v_at:v_at + H * dv].view(n, H, dv)
+            c, cum = g[at:at + n, H:2 * H], g[at:at + n, 2 * H:3 * H].double().cumsum(0)
+            low = torch.ones(n, n, dtype=torch.bool, device=p.device).tril()
+            d = torch.exp((cum[:, None] - cum[None]).masked_fill(~low[:, :, None], float("-inf")).to(p.dtype))
+            w = torch.einsum("ihd,jhd->ijh", q, k) * d * c[None]
+            o = torch.einsum("ijh,jhv->ihv", w, v) + torch.exp(cum).to(p.dtype)[:, :, None] * torch.einsum("hvd,ihd->ihv", S, q)
+            if skip is not None:
+                o = o + _f(skip)[None, :, None] * v
+            out[at:at + n] = o.reshape(n, -1).to(torch.float32)
+            left = torch.exp(cum[-1:] - cum).to(p.dtype) * c
+            S = torch.exp(cum[-1]).to(p.dtype)[:, None, None] * S + torch.einsum("jh,jhv,jhd->hvd", left, v, k)
+        if count > 0:
+            state[slot, :H * dk * dv] = S.reshape(-1).to(torch.float32)
+    return out
 
 
 def normalized_readout(x, floor, gate, weight, eps, num_heads, size, out_dtype):
