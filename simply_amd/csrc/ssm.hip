@@ -38,6 +38,14 @@ __device__ inline void store8(float* p, const float (&v)[8]) {
   reinterpret_cast<float4*>(p)[1] = float4{v[4], v[5], v[6], v[7]};
 }
 
+// z sigmoid(z): a result that is rounded to bfloat16 takes the hardware's exponential and reciprocal, a 32-bit one the
+// library's.
+template <typename T>
+__device__ __forceinline__ float silu_for(float z) {
+  if constexpr (sizeof(T) == 2) return z * __builtin_amdgcn_rcpf(1.f + __expf(-z));
+  else return z / (1.f + expf(-z));
+}
+
 struct SsmInputs {
   int64_t row_stride, tail_stride;
   int x_at, dt_at, C, H, taps;
@@ -111,24 +119,22 @@ __global__ __launch_bounds__(kWave) void ssm_inputs_kernel(const T* __restrict__
       store8(tail + static_cast<size_t>(i) * p.C + c, v);
     }
   }
-  float next[8];
-  load8(col + static_cast<size_t>(j0) * p.row_stride, next);
-  for (int j = 0; j < jn; ++j) {
+  float in[kSsmTokens][8];
 #pragma unroll
-    for (int i = 0; i + 1 < N; ++i)
+  for (int j = 0; j < kSsmTokens; ++j) load8(col + static_cast<size_t>(j0 + (j < jn ? j : jn - 1)) * p.row_stride, in[j]);
 #pragma unroll
-      for (int e = 0; e < 8; ++e) win[i][e] = win[i + 1][e];
-#pragma unroll
-    for (int e = 0; e < 8; ++e) win[N - 1][e] = next[e];
-    if (j + 1 < jn) load8(col + static_cast<size_t>(j0 + j + 1) * p.row_stride, next);
+  for (int j = 0; j < kSsmTokens; ++j) {
+    if (j >= jn) break;   // (uniform)
     float acc[8];
 #pragma unroll
     for (int e = 0; e < 8; ++e) {
       acc[e] = 0.f;
 #pragma unroll
-      for (int i = 0; i < N; ++i) acc[e] = fmaf(w[i][e], win[i][e], acc[e]);
-      acc[e] += b[e];
-      acc[e] = acc[e] / (1.f + expf(-acc[e]));
+      for (int i = 0; i < N; ++i) {
+        const int at = j - (N - 1) + i;   // before j0: win[N + at]
+        acc[e] = fmaf(w[i][e], at >= 0 ? in[at >= 0 ? at : 0][e] : win[at < 0 ? N + at : 0][e], acc[e]);
+      }
+      acc[e] = silu_for<T>(acc[e] + b[e]);
     }
     store8(y + static_cast<size_t>(first + j0 + j) * p.C + c, acc);
   }
@@ -165,7 +171,7 @@ __global__ __launch_bounds__(kWave) void ssm_inputs_any_kernel(const T* __restri
       acc = fmaf(load_f(taps_by_tap, taps_dtype, static_cast<size_t>(i) * p.C + c), u, acc);
     }
     acc += load_f(bias, taps_dtype, c);
-    y[static_cast<size_t>(first + j) * p.C + c] = from_float<T>(acc / (1.f + expf(-acc)));
+    y[static_cast<size_t>(first + j) * p.C + c] = from_float<T>(silu_for<T>(acc));
   }
   if (j0 > 0) return;
   for (int i = 0; i < n - 1; ++i) {   // (old entries are read at places that have not been written yet)
@@ -175,10 +181,10 @@ __global__ __launch_bounds__(kWave) void ssm_inputs_any_kernel(const T* __restri
   }
 }
 
-// A workgroup per (token, group).  NP > 0: the group's entries are held in registers, NP pieces of VEC a thread; 0: they
+// A workgroup of NT threads per (token, group).  NP > 0: the group's entries are held in registers, NP pieces of VEC a thread; 0: they
 // are read twice.
-template <typename T, int VEC, int NP>
-__global__ __launch_bounds__(256) void gated_group_norm_kernel(const float* __restrict__ y, int64_t y_stride,
+template <typename T, int VEC, int NP, int NT>
+__global__ __launch_bounds__(NT) void gated_group_norm_kernel(const float* __restrict__ y, int64_t y_stride,
                                                                const T* __restrict__ z, int64_t z_stride,
                                                                const void* __restrict__ w, int w_dtype, float eps,
                                                                T* __restrict__ out, int64_t out_stride, int size) {
@@ -187,18 +193,15 @@ __global__ __launch_bounds__(256) void gated_group_norm_kernel(const float* __re
   const float* yr = y + static_cast<size_t>(t) * y_stride + c0;
   const T* zr = z + static_cast<size_t>(t) * z_stride + c0;
   T* orow = out + static_cast<size_t>(t) * out_stride + c0;
-  auto gated = [&](float yv, T zv) {
-    const float g = to_float(zv);
-    return yv * (g / (1.f + expf(-g)));
-  };
+  auto gated = [&](float yv, T zv) { return yv * silu_for<T>(to_float(zv)); };
   float ss = 0.f;
   if constexpr (NP == 0) {
-    for (int d = threadIdx.x; d < size; d += 256) {
+    for (int d = threadIdx.x; d < size; d += NT) {
       const float v = gated(yr[d], zr[d]);
       ss = fmaf(v, v, ss);
     }
-    const float r = 1.f / sqrtf(block_sum(ss, scratch) / static_cast<float>(size) + eps);
-    for (int d = threadIdx.x; d < size; d += 256)
+    const float r = 1.f / sqrtf((NT == kWave ? wave_sum(ss) : block_sum(ss, scratch)) / static_cast<float>(size) + eps);
+    for (int d = threadIdx.x; d < size; d += NT)
       orow[d] = from_float<T>(gated(yr[d], zr[d]) * r * load_f(w, w_dtype, c0 + d));
   } else {
     float v[NP][VEC];
@@ -206,7 +209,7 @@ __global__ __launch_bounds__(256) void gated_group_norm_kernel(const float* __re
     T zv[NP][VEC];
 #pragma unroll
     for (int i = 0; i < NP; ++i) {
-      const int d = (threadIdx.x + i * 256) * VEC;
+      const int d = (threadIdx.x + i * NT) * VEC;
 #pragma unroll
       for (int e = 0; e < VEC; ++e) {
         yv[i][e] = 0.f;
@@ -230,10 +233,10 @@ __global__ __launch_bounds__(256) void gated_group_norm_kernel(const float* __re
         v[i][e] = gated(yv[i][e], zv[i][e]);
         ss = fmaf(v[i][e], v[i][e], ss);
       }
-    const float r = 1.f / sqrtf(block_sum(ss, scratch) / static_cast<float>(size) + eps);
+    const float r = 1.f / sqrtf((NT == kWave ? wave_sum(ss) : block_sum(ss, scratch)) / static_cast<float>(size) + eps);
 #pragma unroll
     for (int i = 0; i < NP; ++i) {
-      const int d = (threadIdx.x + i * 256) * VEC;
+      const int d = (threadIdx.x + i * NT) * VEC;
       if (d >= size) continue;
       T o[VEC];
 #pragma unroll
@@ -252,17 +255,19 @@ static void launch_gated_group_norm(const float* y, int64_t y_stride, const void
   const T* z = static_cast<const T*>(z_);
   T* out = static_cast<T*>(out_);
   const dim3 grid(T_, groups);
-#define SA_GROUP_NORM(VEC, NP) \
-  gated_group_norm_kernel<T, VEC, NP><<<grid, 256, 0, stream>>>(y, y_stride, z, z_stride, w, w_dtype, eps, out, out_stride, size)
+#define SA_GROUP_NORM(VEC, NP, NT) \
+  gated_group_norm_kernel<T, VEC, NP, NT><<<grid, NT, 0, stream>>>(y, y_stride, z, z_stride, w, w_dtype, eps, out, out_stride, size)
   auto aligned = [](const void* p) { return reinterpret_cast<uintptr_t>(p) % 16 == 0; };
   const bool vec = size % 4 == 0 && y_stride % 4 == 0 && z_stride % 4 == 0 && out_stride % 4 == 0 && aligned(y) && aligned(z) &&
                    aligned(out);
-  if (vec && size <= 1024) SA_GROUP_NORM(4, 1);
-  else if (vec && size <= 2048) SA_GROUP_NORM(4, 2);
-  else if (vec && size <= 4096) SA_GROUP_NORM(4, 4);
-  else if (vec && size <= 8192) SA_GROUP_NORM(4, 8);
-  else if (!vec && size <= 512) SA_GROUP_NORM(1, 2);
-  else SA_GROUP_NORM(1, 0);
+  if (vec && size <= 256) SA_GROUP_NORM(4, 1, 64);
+  else if (vec && size <= 512) SA_GROUP_NORM(4, 2, 64);
+  else if (vec && size <= 1024) SA_GROUP_NORM(4, 1, 256);
+  else if (vec && size <= 2048) SA_GROUP_NORM(4, 2, 256);
+  else if (vec && size <= 4096) SA_GROUP_NORM(4, 4, 256);
+  else if (vec && size <= 8192) SA_GROUP_NORM(4, 8, 256);
+  else if (!vec && size <= 512) SA_GROUP_NORM(1, 2, 256);
+  else SA_GROUP_NORM(1, 0, 256);
 #undef SA_GROUP_NORM
 }
 

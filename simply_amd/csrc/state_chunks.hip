@@ -28,7 +28,29 @@ struct StateChunks {
   int q_at, k_at, v_at, H, heads_per_key, dk, dv, skip_dtype;
 };
 
-__device__ inline double lane_up(double v, int by) { return __shfl_up(v, by, kWave); }
+// What a piece's tokens weigh, one entry per token.
+struct Piece {
+  double cum[kPieceTokens];                              // L_j
+  __attribute__((aligned(16))) float in[kPieceTokens];   // c_j
+  __attribute__((aligned(16))) float to_block[kPieceTokens];   // exp(L at the end of the token's 16 - L_j) c_j
+  __attribute__((aligned(16))) float to_end[kPieceTokens];     // exp(L at the piece's end - L_j) c_j
+};
+
+// By one wave: lane j has token j's logarithm and input factor.  The sums are 64-bit, so that the differences of sums of up
+// to 64 logarithms keep 32 bits.
+__device__ inline void weigh_piece(Piece& out, double lg, float in, int lane) {
+  double cum = lg;
+#pragma unroll
+  for (int by = 1; by < kWave; by *= 2) {
+    const double up = __shfl_up(cum, by, kWave);
+    if (lane >= by) cum += up;
+  }
+  const double block = __shfl(cum, lane | 15, kWave), end = __shfl(cum, kWave - 1, kWave);
+  out.cum[lane] = cum;
+  out.in[lane] = in;
+  out.to_block[lane] = expf(static_cast<float>(block - cum)) * in;
+  out.to_end[lane] = expf(static_cast<float>(end - cum)) * in;
+}
 
 // NT: blocks of 16 key channels (dk <= 16 NT), a multiple of four.
 template <int NT, typename XT>
@@ -44,8 +66,7 @@ __global__ __launch_bounds__(256) void state_chunks_kernel(const XT* __restrict_
   constexpr int PB = kPieceTokens * PIECES / 256;
   __shared__ __align__(16) XT k_s[kPieceTokens * ROW];
   __shared__ __align__(16) floatx4 s_s[2][NT * kWave];   // the state as the operand of the products that read it
-  __shared__ double cum_s[kPieceTokens];
-  __shared__ float in_s[kPieceTokens];
+  __shared__ Piece piece_s[2];
   const int* meta = seq_meta + 4 * blockIdx.x;
   const int slot = meta[0], first = meta[1], count = meta[2];
   if (count <= 0) return;
@@ -73,69 +94,56 @@ __global__ __launch_bounds__(256) void state_chunks_kernel(const XT* __restrict_
   uint4 kb[PB];                    // rows of k, on their way to LDS
   XT vb[16];                       // v[16 b + 4 g + r][c]
   uint4 qb[HALF ? NT / 2 : NT];    // four neighbouring entries of the wave's own rows of q per block of key channels
-  XT xb[4];                        // v of the lane's own token, four columns, for the skip
+  XT xb[4] = {};                   // v of the lane's own token, four columns, for the skip
   float lg = 0.f, in = 0.f;        // a token a lane: the decay's logarithm and the input factor
   const int own = wave * 16 + c;   // the lane's own token of the piece
+  // (tokens behind the request's last one stand for the last one again: their input factor is 0, their results go nowhere)
   auto fetch = [&](int t0) __attribute__((always_inline)) {
-    const int tn = count - t0 < kPieceTokens ? count - t0 : kPieceTokens;
+    const int last = (count - t0 < kPieceTokens ? count - t0 : kPieceTokens) - 1;
     const XT* rows = proj + static_cast<size_t>(first + t0) * p.proj_stride;
 #pragma unroll
     for (int i = 0; i < PB; ++i) {
       const int idx = tid + i * 256, j = idx / PIECES, d = idx % PIECES * VEC;
-      kb[i] = uint4{0, 0, 0, 0};
-      if (j < tn && d < p.dk)
-        kb[i] = *reinterpret_cast<const uint4*>(rows + static_cast<size_t>(j) * p.proj_stride + p.k_at + kh * p.dk + d);
+      kb[i] = *reinterpret_cast<const uint4*>(rows + static_cast<size_t>(j < last ? j : last) * p.proj_stride + p.k_at + kh * p.dk +
+                                              (d < p.dk ? d : 0));
     }
 #pragma unroll
     for (int i = 0; i < 16; ++i) {
       const int j = i / 4 * 16 + g * 4 + i % 4;
-      vb[i] = from_float<XT>(0.f);
-      if (j < tn && col_ok) vb[i] = rows[static_cast<size_t>(j) * p.proj_stride + p.v_at + h * p.dv + col];
+      vb[i] = rows[static_cast<size_t>(j < last ? j : last) * p.proj_stride + p.v_at + h * p.dv + (col_ok ? col : 0)];
     }
-    const bool ok = own < tn;
-    const XT* mine = rows + static_cast<size_t>(ok ? own : 0) * p.proj_stride;
+    const XT* mine = rows + static_cast<size_t>(own < last ? own : last) * p.proj_stride;
 #pragma unroll
     for (int n = 0; n < NT; ++n) {
-      const int d = n * 16 + g * 4;
+      const int d = n * 16 + g * 4, at = d < p.dk ? d : 0;   // (channels behind the last meet zeros in k and in the state)
       if constexpr (HALF) {
-        uint2 v{0, 0};
-        if (ok && d < p.dk) v = *reinterpret_cast<const uint2*>(mine + p.q_at + kh * p.dk + d);
+        const uint2 v = *reinterpret_cast<const uint2*>(mine + p.q_at + kh * p.dk + at);
         if (n % 2 == 0) qb[n / 2].x = v.x, qb[n / 2].y = v.y;
         else qb[n / 2].z = v.x, qb[n / 2].w = v.y;
       } else {
-        qb[n] = uint4{0, 0, 0, 0};
-        if (ok && d < p.dk) qb[n] = *reinterpret_cast<const uint4*>(mine + p.q_at + kh * p.dk + d);
+        qb[n] = *reinterpret_cast<const uint4*>(mine + p.q_at + kh * p.dk + at);
       }
     }
+    if (skip != nullptr) {
+      const int cc = blockIdx.z * 16 + g * 4;
 #pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      const int cc = blockIdx.z * 16 + g * 4 + r;
-      xb[r] = from_float<XT>(0.f);
-      if (skip != nullptr && ok && cc < p.dv) xb[r] = mine[p.v_at + h * p.dv + cc];
+      for (int r = 0; r < 4; ++r) xb[r] = mine[p.v_at + h * p.dv + (cc + r < p.dv ? cc + r : 0)];
     }
-    const bool live = lane < tn;
-    const float* gr = gates + static_cast<size_t>(first + t0 + (live ? lane : 0)) * p.gates_stride;
-    in = live ? gr[p.H + h] : 0.f;
-    lg = live ? gr[2 * p.H + h] : 0.f;
+    if (wave == 0) {
+      const float* gr = gates + static_cast<size_t>(first + t0 + (lane < last ? lane : last)) * p.gates_stride;
+      in = lane <= last ? gr[p.H + h] : 0.f;
+      lg = lane <= last ? gr[2 * p.H + h] : 0.f;
+    }
   };
   fetch(0);
+  if (wave == 0) weigh_piece(piece_s[0], lg, in, lane);
   int now = 0;
   for (int t0 = 0; t0 < count; t0 += kPieceTokens, now ^= 1) {
     __syncthreads();   // (the piece before has been worked through)
 #pragma unroll
     for (int i = 0; i < PB; ++i) {
       const int idx = tid + i * 256;
-      *reinterpret_cast<uint4*>(&k_s[idx / PIECES * ROW + idx % PIECES * VEC]) = kb[i];
-    }
-    if (wave == 0) {
-      double cum = lg;   // (sums of up to 64 logarithms: their differences keep 32 bits)
-#pragma unroll
-      for (int by = 1; by < kWave; by *= 2) {
-        const double up = lane_up(cum, by);
-        if (lane >= by) cum += up;
-      }
-      cum_s[lane] = cum;
-      in_s[lane] = in;
+      *reinterpret_cast<uint4*>(&k_s[idx / PIECES * ROW + idx % PIECES * VEC]) = idx % PIECES * VEC < p.dk ? kb[i] : uint4{0, 0, 0, 0};
     }
     float v[16], x[4];
 #pragma unroll
@@ -164,7 +172,8 @@ __global__ __launch_bounds__(256) void state_chunks_kernel(const XT* __restrict_
 #pragma unroll
       for (int r = 0; r < 4; ++r) o = __builtin_amdgcn_mfma_f32_16x16x4f32(st[r], qf[r], o, 0, 0, 0);
     }
-    const double cum_i = cum_s[own], cum_all = cum_s[kPieceTokens - 1];
+    const Piece& pc = piece_s[now];
+    const double cum_i = pc.cum[own];
     {
       const float e = expf(static_cast<float>(cum_i));
 #pragma unroll
@@ -191,14 +200,24 @@ __global__ __launch_bounds__(256) void state_chunks_kernel(const XT* __restrict_
           for (int r = 0; r < 4; ++r) m = __builtin_amdgcn_mfma_f32_16x16x4f32(kf[r], qf[r], m, 0, 0, 0);
         }
       }
+      // exp(L_i - L_j) c_j: in an earlier block by way of that block's end, in the own one token by token (tokens behind
+      // the own one: exp of minus infinity)
+      floatx4 wgt;
+      if (b < wave) {
+        const float e = expf(static_cast<float>(cum_i - pc.cum[b * 16 + 15]));
+        wgt = *reinterpret_cast<const floatx4*>(&pc.to_block[b * 16 + g * 4]);
 #pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int j = b * 16 + g * 4 + r;
-        // (tokens behind the own one: exp of minus infinity)
-        const float d = j <= own ? static_cast<float>(cum_i - cum_s[j]) : -INFINITY;
-        const float wgt = m[r] * expf(d) * in_s[j];
-        o = __builtin_amdgcn_mfma_f32_16x16x4f32(v[b * 4 + r], wgt, o, 0, 0, 0);
+        for (int r = 0; r < 4; ++r) wgt[r] *= e;
+      } else {
+        wgt = *reinterpret_cast<const floatx4*>(&pc.in[b * 16 + g * 4]);
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const int j = b * 16 + g * 4 + r;
+          wgt[r] *= expf(j <= own ? static_cast<float>(cum_i - pc.cum[j]) : -INFINITY);
+        }
       }
+#pragma unroll
+      for (int r = 0; r < 4; ++r) o = __builtin_amdgcn_mfma_f32_16x16x4f32(v[b * 4 + r], m[r] * wgt[r], o, 0, 0, 0);
     }
     if (t0 + own < count) {
       const int cc = blockIdx.z * 16 + g * 4;
@@ -209,11 +228,12 @@ __global__ __launch_bounds__(256) void state_chunks_kernel(const XT* __restrict_
       if (cc < p.dv) *reinterpret_cast<floatx4*>(dst) = y;
     }
     // the state behind the piece
-    const float all = expf(static_cast<float>(cum_all));
+    const float all = expf(static_cast<float>(pc.cum[kPieceTokens - 1]));
 #pragma unroll
-    for (int i = 0; i < 16; ++i) {
-      const int j = i / 4 * 16 + g * 4 + i % 4;
-      v[i] *= expf(static_cast<float>(cum_all - cum_s[j])) * in_s[j];
+    for (int b = 0; b < 4; ++b) {
+      const floatx4 e = *reinterpret_cast<const floatx4*>(&pc.to_end[b * 16 + g * 4]);
+#pragma unroll
+      for (int r = 0; r < 4; ++r) v[b * 4 + r] *= e[r];
     }
 #pragma unroll
     for (int n = 0; n < NW; ++n) {
@@ -227,6 +247,8 @@ __global__ __launch_bounds__(256) void state_chunks_kernel(const XT* __restrict_
       }
       s_s[now ^ 1][nb * kWave + lane] = s[n];
     }
+    // (by the wave with the fewest blocks of tokens to go through)
+    if (wave == 0 && t0 + kPieceTokens < count) weigh_piece(piece_s[now ^ 1], lg, in, lane);
   }
 #pragma unroll
   for (int n = 0; n < NW; ++n) {
