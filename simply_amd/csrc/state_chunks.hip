@@ -28,6 +28,21 @@ struct StateChunks {
   int q_at, k_at, v_at, H, heads_per_key, dk, dv, skip_dtype;
 };
 
+// An entry's bits in a 32-bit register, and its value.
+__device__ __forceinline__ unsigned load_bits(const bf16* p) { return p->bits; }
+__device__ __forceinline__ unsigned load_bits(const float* p) { return __float_as_uint(*p); }
+template <typename XT>
+__device__ __forceinline__ float bits_float(unsigned v) {
+  return __uint_as_float(sizeof(XT) == 2 ? v << 16 : v);
+}
+
+// A run whose products have bfloat16 operands takes the hardware's exponential, a 32-bit run the library's.
+template <bool HALF>
+__device__ __forceinline__ float decay_exp(float x) {
+  if constexpr (HALF) return __expf(x);
+  else return expf(x);
+}
+
 // What a piece's tokens weigh, one entry per token.
 struct Piece {
   double cum[kPieceTokens];                              // L_j
@@ -38,6 +53,7 @@ struct Piece {
 
 // By one wave: lane j has token j's logarithm and input factor.  The sums are 64-bit, so that the differences of sums of up
 // to 64 logarithms keep 32 bits.
+template <bool HALF>
 __device__ inline void weigh_piece(Piece& out, double lg, float in, int lane) {
   double cum = lg;
 #pragma unroll
@@ -48,8 +64,8 @@ __device__ inline void weigh_piece(Piece& out, double lg, float in, int lane) {
   const double block = __shfl(cum, lane | 15, kWave), end = __shfl(cum, kWave - 1, kWave);
   out.cum[lane] = cum;
   out.in[lane] = in;
-  out.to_block[lane] = expf(static_cast<float>(block - cum)) * in;
-  out.to_end[lane] = expf(static_cast<float>(end - cum)) * in;
+  out.to_block[lane] = decay_exp<HALF>(static_cast<float>(block - cum)) * in;
+  out.to_end[lane] = decay_exp<HALF>(static_cast<float>(end - cum)) * in;
 }
 
 // NT: blocks of 16 key channels (dk <= 16 NT), a multiple of four.
@@ -92,51 +108,53 @@ __global__ __launch_bounds__(256) void state_chunks_kernel(const XT* __restrict_
 
   // what a piece needs from memory, asked for a piece ahead
   uint4 kb[PB];                    // rows of k, on their way to LDS
-  XT vb[16];                       // v[16 b + 4 g + r][c]
+  unsigned vb[16];                 // the bits of v[16 b + 4 g + r][c]
   uint4 qb[HALF ? NT / 2 : NT];    // four neighbouring entries of the wave's own rows of q per block of key channels
-  XT xb[4] = {};                   // v of the lane's own token, four columns, for the skip
+  unsigned xb[4];                  // and of v of the lane's own token, four columns, for the skip
   float lg = 0.f, in = 0.f;        // a token a lane: the decay's logarithm and the input factor
   const int own = wave * 16 + c;   // the lane's own token of the piece
-  // (tokens behind the request's last one stand for the last one again: their input factor is 0, their results go nowhere)
+  // A lane's places in a piece: 32-bit offsets from rows that are the same for all lanes, without a branch, so that nothing
+  // waits for the loads before they are used.  (tokens behind the request's last one stand for the last one again: their
+  // input factor is 0, their results go nowhere; channels behind the last meet zeros in k and in the state)
+  const int stride = static_cast<int>(p.proj_stride);
+  const int k_lane = tid / PIECES, k_d = tid % PIECES * VEC;   // (256 threads: whole rows of k each time)
+  const int k_col = k_d < p.dk ? k_d : 0, v_col = col_ok ? col : 0;
+  const int x_col = blockIdx.z * 16 + g * 4 < p.dv ? blockIdx.z * 16 + g * 4 : 0;   // (value sizes are multiples of 4)
   auto fetch = [&](int t0) __attribute__((always_inline)) {
     const int last = (count - t0 < kPieceTokens ? count - t0 : kPieceTokens) - 1;
     const XT* rows = proj + static_cast<size_t>(first + t0) * p.proj_stride;
+    auto row = [&](int j) __attribute__((always_inline)) { return (j < last ? j : last) * stride; };
+    const XT* kp = rows + p.k_at + kh * p.dk;
+    const XT* vp = rows + p.v_at + h * p.dv;
+    const XT* qp = rows + p.q_at + kh * p.dk;
 #pragma unroll
-    for (int i = 0; i < PB; ++i) {
-      const int idx = tid + i * 256, j = idx / PIECES, d = idx % PIECES * VEC;
-      kb[i] = *reinterpret_cast<const uint4*>(rows + static_cast<size_t>(j < last ? j : last) * p.proj_stride + p.k_at + kh * p.dk +
-                                              (d < p.dk ? d : 0));
-    }
+    for (int i = 0; i < PB; ++i) kb[i] = *reinterpret_cast<const uint4*>(kp + row(k_lane + i * (256 / PIECES)) + k_col);
 #pragma unroll
-    for (int i = 0; i < 16; ++i) {
-      const int j = i / 4 * 16 + g * 4 + i % 4;
-      vb[i] = rows[static_cast<size_t>(j < last ? j : last) * p.proj_stride + p.v_at + h * p.dv + (col_ok ? col : 0)];
-    }
-    const XT* mine = rows + static_cast<size_t>(own < last ? own : last) * p.proj_stride;
+    for (int i = 0; i < 16; ++i) vb[i] = load_bits(vp + row(i / 4 * 16 + g * 4 + i % 4) + v_col);
+    const int mine = row(own);
 #pragma unroll
     for (int n = 0; n < NT; ++n) {
-      const int d = n * 16 + g * 4, at = d < p.dk ? d : 0;   // (channels behind the last meet zeros in k and in the state)
+      const int d = n * 16 + g * 4, at = mine + (d < p.dk ? d : 0);
       if constexpr (HALF) {
-        const uint2 v = *reinterpret_cast<const uint2*>(mine + p.q_at + kh * p.dk + at);
+        const uint2 v = *reinterpret_cast<const uint2*>(qp + at);
         if (n % 2 == 0) qb[n / 2].x = v.x, qb[n / 2].y = v.y;
         else qb[n / 2].z = v.x, qb[n / 2].w = v.y;
       } else {
-        qb[n] = *reinterpret_cast<const uint4*>(mine + p.q_at + kh * p.dk + at);
+        qb[n] = *reinterpret_cast<const uint4*>(qp + at);
       }
     }
-    if (skip != nullptr) {
-      const int cc = blockIdx.z * 16 + g * 4;
 #pragma unroll
-      for (int r = 0; r < 4; ++r) xb[r] = mine[p.v_at + h * p.dv + (cc + r < p.dv ? cc + r : 0)];
-    }
-    if (wave == 0) {
-      const float* gr = gates + static_cast<size_t>(first + t0 + (lane < last ? lane : last)) * p.gates_stride;
-      in = lane <= last ? gr[p.H + h] : 0.f;
-      lg = lane <= last ? gr[2 * p.H + h] : 0.f;
-    }
+    for (int r = 0; r < 4; ++r) xb[r] = load_bits(vp + mine + x_col + r);
+    const float* gr = gates + static_cast<size_t>(first + t0 + (lane < last ? lane : last)) * p.gates_stride;
+    in = gr[p.H + h];
+    lg = gr[2 * p.H + h];
+  };
+  auto weigh = [&](Piece& to, int t0) __attribute__((always_inline)) {
+    const bool live = t0 + lane < count;
+    weigh_piece<HALF>(to, live ? lg : 0.f, live ? in : 0.f, lane);
   };
   fetch(0);
-  if (wave == 0) weigh_piece(piece_s[0], lg, in, lane);
+  if (wave == 0) weigh(piece_s[0], 0);
   int now = 0;
   for (int t0 = 0; t0 < count; t0 += kPieceTokens, now ^= 1) {
     __syncthreads();   // (the piece before has been worked through)
@@ -147,14 +165,14 @@ __global__ __launch_bounds__(256) void state_chunks_kernel(const XT* __restrict_
     }
     float v[16], x[4];
 #pragma unroll
-    for (int i = 0; i < 16; ++i) v[i] = to_float(vb[i]);
+    for (int i = 0; i < 16; ++i) v[i] = bits_float<XT>(vb[i]);
 #pragma unroll
-    for (int r = 0; r < 4; ++r) x[r] = to_float(xb[r]);
+    for (int r = 0; r < 4; ++r) x[r] = bits_float<XT>(xb[r]);
     uint4 q[HALF ? NT / 2 : NT];
 #pragma unroll
     for (int n = 0; n < (HALF ? NT / 2 : NT); ++n) q[n] = qb[n];
     __syncthreads();
-    if (t0 + kPieceTokens < count) fetch(t0 + kPieceTokens);
+    fetch(t0 + kPieceTokens < count ? t0 + kPieceTokens : t0);   // (behind the last piece: that one again, for nothing)
 
     // o^T[column, own token] from the state
     floatx4 o{0.f, 0.f, 0.f, 0.f};
@@ -175,11 +193,20 @@ __global__ __launch_bounds__(256) void state_chunks_kernel(const XT* __restrict_
     const Piece& pc = piece_s[now];
     const double cum_i = pc.cum[own];
     {
-      const float e = expf(static_cast<float>(cum_i));
+      const float e = decay_exp<HALF>(static_cast<float>(cum_i));
 #pragma unroll
       for (int r = 0; r < 4; ++r) o[r] *= e;
     }
-    // and from the piece's own tokens, 16 of them at a time: weights [token j, own token]
+    // and from the piece's own tokens, 16 of them at a time: weights [token j, own token], exp(L_i - L_j) c_j: in an
+    // earlier block by way of that block's end, in the own one token by token (tokens behind the own one: exp of minus
+    // infinity)
+    floatx4 own_wgt = *reinterpret_cast<const floatx4*>(&pc.in[wave * 16 + g * 4]);
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int j = wave * 16 + g * 4 + r;
+      const float d = static_cast<float>(cum_i - pc.cum[j]);
+      own_wgt[r] *= decay_exp<HALF>(j <= own ? d : -INFINITY);
+    }
 #pragma unroll
     for (int b = 0; b < 4; ++b) {
       if (b > wave) break;   // (uniform over the wave)
@@ -200,21 +227,12 @@ __global__ __launch_bounds__(256) void state_chunks_kernel(const XT* __restrict_
           for (int r = 0; r < 4; ++r) m = __builtin_amdgcn_mfma_f32_16x16x4f32(kf[r], qf[r], m, 0, 0, 0);
         }
       }
-      // exp(L_i - L_j) c_j: in an earlier block by way of that block's end, in the own one token by token (tokens behind
-      // the own one: exp of minus infinity)
-      floatx4 wgt;
+      floatx4 wgt = own_wgt;
       if (b < wave) {
-        const float e = expf(static_cast<float>(cum_i - pc.cum[b * 16 + 15]));
+        const float e = decay_exp<HALF>(static_cast<float>(cum_i - pc.cum[b * 16 + 15]));
         wgt = *reinterpret_cast<const floatx4*>(&pc.to_block[b * 16 + g * 4]);
 #pragma unroll
         for (int r = 0; r < 4; ++r) wgt[r] *= e;
-      } else {
-        wgt = *reinterpret_cast<const floatx4*>(&pc.in[b * 16 + g * 4]);
-#pragma unroll
-        for (int r = 0; r < 4; ++r) {
-          const int j = b * 16 + g * 4 + r;
-          wgt[r] *= expf(j <= own ? static_cast<float>(cum_i - pc.cum[j]) : -INFINITY);
-        }
       }
 #pragma unroll
       for (int r = 0; r < 4; ++r) o = __builtin_amdgcn_mfma_f32_16x16x4f32(v[b * 4 + r], m[r] * wgt[r], o, 0, 0, 0);
@@ -228,7 +246,7 @@ __global__ __launch_bounds__(256) void state_chunks_kernel(const XT* __restrict_
       if (cc < p.dv) *reinterpret_cast<floatx4*>(dst) = y;
     }
     // the state behind the piece
-    const float all = expf(static_cast<float>(pc.cum[kPieceTokens - 1]));
+    const float all = decay_exp<HALF>(static_cast<float>(pc.cum[kPieceTokens - 1]));
 #pragma unroll
     for (int b = 0; b < 4; ++b) {
       const floatx4 e = *reinterpret_cast<const floatx4*>(&pc.to_end[b * 16 + g * 4]);
@@ -248,7 +266,7 @@ __global__ __launch_bounds__(256) void state_chunks_kernel(const XT* __restrict_
       s_s[now ^ 1][nb * kWave + lane] = s[n];
     }
     // (by the wave with the fewest blocks of tokens to go through)
-    if (wave == 0 && t0 + kPieceTokens < count) weigh_piece(piece_s[now ^ 1], lg, in, lane);
+    if (wave == 0 && t0 + kPieceTokens < count) weigh(piece_s[now ^ 1], t0 + kPieceTokens);
   }
 #pragma unroll
   for (int n = 0; n < NW; ++n) {
@@ -282,6 +300,7 @@ extern "C" int sa_state_chunks(const void* proj, int dtype, int64_t proj_stride,
                  proj_stride >= q_at + static_cast<int64_t>(key_heads) * dk && proj_stride >= k_at + static_cast<int64_t>(key_heads) * dk &&
                  proj_stride >= v_at + static_cast<int64_t>(H) * dv,
              "state_chunks: rows of the state, the gates or the projection are too short");
+  SA_REQUIRE(proj_stride * kPieceTokens < (1LL << 31), "state_chunks: rows of %lld entries are too long", (long long)proj_stride);
   SA_REQUIRE((dtype == kF32 || dtype == kBF16) && (skip == nullptr || skip_dtype == kF32 || skip_dtype == kBF16),
              "state_chunks: unknown dtype");
   StateChunks p;
