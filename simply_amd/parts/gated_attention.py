@@ -22,6 +22,10 @@ results are multiplied by sigmoid(gate projection), entry by entry (`output_gate
 `own_keys_values` False: the layer has queries only and reads the keys and values that another schedule entry keeps
 (that entry's `cache_window` then covers this layer's window too).  What is kept per token is a `PagedKVNeed`; with a
 convolution the tails are a `StateNeed` beside it (a `CompositeNeed`: pages first, then the state).
+
+A plain layer (projections, rotation, window and nothing else of the above) whose head sizes the bfloat16 matrix-core
+kernels do not take as they are runs with its heads filled up: rows of zeros behind every head's rows of the projections and
+columns of zeros in the output projection, put in when the weights are loaded.  No score and no result changes by it.
 """
 from __future__ import annotations
 
@@ -78,7 +82,35 @@ class GatedAttention(Mixer):
         self.in_proj = self.o_proj = self.in_bias = self.taps = self.taps_by_tap = self.q_norm = self.k_norm = None
         self.sinks = self.slopes = None
 
+        #: sizes of a head's keys and values as the kernels see them (`_fill_up` may make them larger than the design's)
+        self.run_key_dim, self.run_value_dim = self.key_dim, self.value_dim
+
     # ------------------------------------------------------------------ sizes
+    #: what the matrix-core kernels ask of key and value sizes
+    KEY_UNIT, VALUE_UNIT = 32, 16
+
+    def _fill_up(self, t):
+        """The tensors of a plain layer with every head filled up to sizes that the matrix-core kernels take (bfloat16 on
+        the GPU); any other layer's as they are."""
+        w = t["o_proj"]
+        plain = (self.own and self.qk_norm is None and not self.bias and self.conv_taps == 0 and not self.values_are_keys
+                 and not self.zero_sink and self.slope_exponent is None and self.output_gate is None)
+        dk, dv = (-(-self.key_dim // self.KEY_UNIT) * self.KEY_UNIT, -(-self.value_dim // self.VALUE_UNIT) * self.VALUE_UNIT)
+        if not plain or w.dtype != torch.bfloat16 or not w.is_cuda or (dk, dv) == (self.key_dim, self.value_dim):
+            return t
+
+        def rows(name, heads, size, filled):
+            full = torch.zeros((heads, filled, self.hidden_size), dtype=w.dtype, device=w.device)
+            full[:, :size] = t[name].reshape(heads, size, self.hidden_size)
+            return full.reshape(heads * filled, self.hidden_size)
+
+        out = torch.zeros((self.hidden_size, self.num_heads, dv), dtype=w.dtype, device=w.device)
+        out[:, :, :self.value_dim] = w.reshape(self.hidden_size, self.num_heads, self.value_dim)
+        filled = {"q_proj": rows("q_proj", self.num_heads, self.key_dim, dk), "k_proj": rows("k_proj", self.num_kv_heads, self.key_dim, dk),
+                  "v_proj": rows("v_proj", self.num_kv_heads, self.value_dim, dv), "o_proj": out.reshape(self.hidden_size, -1)}
+        self.run_key_dim, self.run_value_dim = dk, dv
+        return filled
+
     @property
     def conv_channels(self) -> int:
         """Channels that pass the convolution: queries, and the layer's own keys and values."""
@@ -118,7 +150,7 @@ class GatedAttention(Mixer):
         return specs
 
     def load(self, tensors):
-        t = tensors
+        t = self._fill_up(tensors)
         sections = ["q"] + ((["k"] if self.values_are_keys else ["k", "v"]) if self.own else [])
         rows = [t[s + "_proj"] for s in sections] + ([t["gate_proj"]] if self.output_gate is not None else [])
         self.in_proj = as_product_weight(torch.cat(rows, dim=0).contiguous())
@@ -146,14 +178,14 @@ class GatedAttention(Mixer):
             self.position_encoding.to_device(device)
 
     def cache_need(self):
-        pages = PagedKVNeed(self.num_kv_heads, self.key_dim, self.cache_window, self.value_dim)
+        pages = PagedKVNeed(self.num_kv_heads, self.run_key_dim, self.cache_window, self.run_value_dim)
         if self.conv_taps > 1:
             return CompositeNeed((pages, StateNeed(((self.conv_taps - 1) * self.conv_channels,), torch.float32)))
         return pages
 
     # ------------------------------------------------------------------ forward
     def forward(self, x, ctx, cache, defer_sum=False):
-        H, K, dk, dv = self.num_heads, self.num_kv_heads, self.key_dim, self.value_dim
+        H, K, dk, dv = self.num_heads, self.num_kv_heads, self.run_key_dim, self.run_value_dim
         pages, state = (cache.parts[0], cache.parts[1].state) if self.conv_taps > 1 else (cache, None)
         if pages.write != self.own:
             raise RuntimeError("gated_attention: a layer with keys and values of its own writes its pages, one without "

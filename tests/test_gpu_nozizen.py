@@ -72,6 +72,20 @@ def test_parts_at_aligned_sizes():
         mech.attention_part(DEV, torch.bfloat16, sizes=sizes, window=window, rot=rot, page_size=16, length=300, cuts=cuts, std=0.1)
 
 
+def test_heads_filled_up_for_the_matrix_cores():
+    """Head sizes that the bfloat16 matrix-core kernels do not take as they are: the layer runs with zeros behind every
+    head's entries, in pages of the larger sizes, and gives the same results; a 32-bit layer runs as it is."""
+    cuts = ([300], [268] + [1] * 32, [17] * 17 + [11])
+    for sizes, window, rot in (((128, 6, 2, 40, 24), 64, mech.ROTATIONS[1]), ((96, 4, 4, 80, 112), None, mech.ROTATIONS[2]),
+                               ((64, 5, 1, 12, 20), 33, mech.ROTATIONS[4])):
+        mech.attention_part(DEV, torch.bfloat16, sizes=sizes, window=window, rot=rot, page_size=16, length=300, cuts=cuts, std=0.1)
+    part, _, _ = mech._attention_part(DEV, torch.bfloat16, (128, 6, 2, 40, 24), 0.1, 64, None)
+    assert (part.run_key_dim, part.run_value_dim) == (64, 32)
+    assert (part.cache_need().head_dim, part.cache_need().value_dim) == (64, 32) and (part.key_dim, part.value_dim) == (40, 24)
+    part, _, _ = mech._attention_part(DEV, torch.float32, (128, 6, 2, 40, 24), 0.1, 64, None)
+    assert (part.run_key_dim, part.run_value_dim) == (40, 24)
+
+
 @pytest.mark.parametrize("dtype", DTYPES)
 def test_window_edges(dtype):
     mech.window_edges(DEV, dtype)
