@@ -345,7 +345,7 @@ def scaled_frequencies():
 def rotated_inputs(o, device, dtype):
     """Queries and keys behind the projection: the first entries of a head turned, with the factor on sines and cosines,
     the others as they are, at positions that do not start at zero; widths with and without pieces of eight."""
-    for rot, dk, dv in ((ROTATIONS[1], 10, 14), (ROTATIONS[0], 16, 8), (ROTATIONS[2], 96, 80), (ROTATIONS[3], 8, 3)):
+    for rot, dk, dv in ((ROTATIONS[1], 10, 14), (ROTATIONS[0], 16, 8), (ROTATIONS[2], 96, 112), (ROTATIONS[3], 8, 3)):
         H, K, P = 4, 2, 4
         f, mult = plain.frequencies(rot)
         m, T = _meta([5, 1], [0, 1], [37, 900])

@@ -93,7 +93,7 @@ def test_window_edges(dtype):
     mech.window_edges(DEV, dtype, window=None, T=200)
 
 
-@pytest.mark.parametrize("sizes", [(64, 8, 2, 64, 64), (64, 4, 2, 96, 80)])
+@pytest.mark.parametrize("sizes", [(64, 8, 2, 64, 64), (64, 4, 2, 96, 112)])
 def test_window_edges_on_the_matrix_cores(sizes):
     mech.window_edges(DEV, torch.bfloat16, sizes=sizes, window=64, T=300, std=0.1)
     mech.window_edges(DEV, torch.bfloat16, sizes=sizes, window=129, T=300, std=0.1)
