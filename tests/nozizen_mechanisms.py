@@ -192,15 +192,14 @@ def _recurrence_wanted(proj, gates, skip, H, G, N, dv, S0):
         x = proj[:, h * dv:(h + 1) * dv].double()
         B = proj[:, inner + g * N:inner + (g + 1) * N].double()
         C = proj[:, inner + (G + g) * N:inner + (G + g + 1) * N].double()
-        dt, a = gates[:, H + h].double(), torch.zeros((), dtype=torch.float64)
-        # (the plain function takes the decay as exp(-exp(a) dt): hand it each token's own logarithm by way of a dt of its own)
+        dt = gates[:, H + h].double()
+        # (decays from their stored logarithms, which the plain function would compute itself)
         S, out = S0[h].T.clone(), []
         for t in range(x.shape[0]):
             S = torch.exp(gates[t, 2 * H + h].double()) * S + dt[t] * torch.outer(B[t], x[t])
             out.append(S.T @ C[t] + skip[h].double() * x[t])
         y.append(torch.stack(out))
         states.append(S.T)
-        del a
     return torch.cat(y, 1), torch.stack(states)
 
 
